@@ -15,6 +15,11 @@ line read nothing else off it):
     vocab_size: int                token ids are checked against it
     max_position_embeddings: int   the engine's `max_context` may not exceed it
     eos_token_ids: tuple[int]      tokens that end a request (merged from generation_config.json if present)
+
+and may offer
+
+    with_tensor_shapes({name: shape}) -> config    the configuration with the sizes that config.json does not give and a
+                                   checkpoint's tensor shapes do; the loader calls it before the model is built
 """
 from __future__ import annotations
 

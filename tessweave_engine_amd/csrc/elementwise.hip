@@ -32,6 +32,57 @@ extern "C" int tw_embed_gather(int dtype, const int* ids, const void* table, flo
   return TW_LAUNCH_RESULT();
 }
 
+// ---- token rows with sinusoidal positions ----------------------------------------------------------------------------
+// out[n] = scale * table[ids[n]] + s(positions[n]), entry 2 i of s(p) the sine and entry 2 i + 1 the cosine of
+// p * base^(-2 i / hidden); copy (or null) receives the same. The frequencies come as pairs of floats (freq[i] + rest[i]
+// is the frequency to twice float32's precision) and the angle is formed with the product's rounding error beside it: a
+// frequency rounded to float32 alone would put the angle of position 1,000 off by 3e-5.
+template <typename T>
+__global__ void embed_sinusoid_kernel(const int* __restrict__ ids, const T* __restrict__ table, float* __restrict__ out,
+                                      float* __restrict__ copy, const int* __restrict__ positions,
+                                      const float* __restrict__ freq, const float* __restrict__ rest, float scale, int hidden,
+                                      int vocab, const int* __restrict__ feed, int feed_count) {
+  const int n = blockIdx.x;
+  int id = ids[n];
+  if (id < 0 && feed != nullptr && -1 - id < feed_count) id = feed[-1 - id];
+  id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+  const T* row = table + (size_t)id * hidden;
+  const float p = (float)positions[n];
+  for (int i = threadIdx.x; 2 * i < hidden; i += blockDim.x) {
+    const float f = freq[i];
+    const float angle = __fmul_rn(p, f);
+    const float off = __fmaf_rn(p, rest[i], __fmaf_rn(p, f, -angle));     // what the product lost
+    float s, c;
+    sincosf(angle, &s, &c);
+    const float sine = __fmaf_rn(off, c, s), cosine = __fmaf_rn(-off, s, c);
+    const size_t at = (size_t)n * hidden + 2 * i;
+    const float a = __fmaf_rn(tw_to_float(row[2 * i]), scale, sine);
+    out[at] = a;
+    if (copy) copy[at] = a;
+    if (2 * i + 1 < hidden) {
+      const float b = __fmaf_rn(tw_to_float(row[2 * i + 1]), scale, cosine);
+      out[at + 1] = b;
+      if (copy) copy[at + 1] = b;
+    }
+  }
+}
+
+extern "C" int tw_embed_sinusoid(int dtype, const int* ids, const void* table, float* out, float* copy, const int* positions,
+                                 const float* freq, const float* rest, float scale, int n, int hidden, int vocab,
+                                 const int* feed, int feed_count, hipStream_t stream) {
+  TW_REQUIRE(ids && table && out && positions && freq && rest && n >= 0 && hidden > 0 && vocab > 0 && feed_count >= 0);
+  if (n == 0) return 0;
+  if (dtype == TW_DTYPE_F32)
+    embed_sinusoid_kernel<float><<<n, 256, 0, stream>>>(ids, (const float*)table, out, copy, positions, freq, rest, scale, hidden,
+                                                        vocab, feed, feed_count);
+  else if (dtype == TW_DTYPE_BF16)
+    embed_sinusoid_kernel<bf16_t><<<n, 256, 0, stream>>>(ids, (const bf16_t*)table, out, copy, positions, freq, rest, scale, hidden,
+                                                         vocab, feed, feed_count);
+  else
+    return TW_ERR_BAD_ARGUMENT;
+  return TW_LAUNCH_RESULT();
+}
+
 // ---- RMS norm -------------------------------------------------------------------------
 // y = x * rsqrt(mean(x^2) + eps) * w, statistics and products in float32, one
 // rounding to the output type. `rows` (optional) picks the input row of each

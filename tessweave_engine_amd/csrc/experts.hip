@@ -9,6 +9,12 @@
 //   out = sum over the chosen experts e of  p_e * expert_e(h)         (the weight multiplies the expert's OUTPUT)
 //   expert(y): down( gelu(up y) ), the exact gelu y Phi(y); no gate matrix
 //
+// A third (`kind` 2, `mode` 2): gated experts whose weights multiply their outputs, a softmax over ALL logits, and experts
+// without matrices:
+//   s = softmax(W_router h) over X + identity logits    chosen: the `top` largest of s + correction
+//   p = s of the chosen over their sum (+ 1e-20)        expert(y): down( silu(gate y) * up y ); the last `identity`
+//   out = sum over the chosen experts e of  p_e * expert_e(h)          experts return h itself
+//
 // A step runs in six launches whose shapes depend only on the number of rows: route; plan (every expert's rows are
 // laid out one expert after the other, each expert's share padded to whole tiles of 16 rows; which expert a tile
 // belongs to is a table on the device, tiles nobody uses say -1); gather (the scaled, rounded input rows in that
@@ -35,6 +41,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
                                                         const float* __restrict__ bias, int mode, int C, int X, int top,
                                                         int* __restrict__ ids, float* __restrict__ weights) {
   __shared__ float z[TW_MOE_MAX_EXPERTS];
+  __shared__ float score[TW_MOE_MAX_EXPERTS];       // mode 2: the softmax over all logits (z: what decides the choice)
   const int row = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const T* x = h + (size_t)row * ld_h;
   // A wave forms two experts' logits at a time, four elements a lane and load, eight loads in flight before the first
@@ -68,12 +75,29 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
     s0 = tw_wave_sum(s0);
     s1 = tw_wave_sum(s1);
     if (lane == 0) {
-      z[e] = s0 + (bias ? bias[e] : 0.f);
-      if (e + 1 < X) z[e + 1] = s1 + (bias ? bias[e + 1] : 0.f);
+      const bool biased = bias && mode != 2;
+      z[e] = s0 + (biased ? bias[e] : 0.f);
+      if (e + 1 < X) z[e + 1] = s1 + (biased ? bias[e + 1] : 0.f);
     }
   }
   __syncthreads();
   if (wave != 0) return;
+  if (mode == 2) {
+    float most = -INFINITY, sum = 0.f;
+    for (int e = lane; e < X; e += 64) most = fmaxf(most, z[e]);
+    most = tw_wave_max(most);
+    for (int e = lane; e < X; e += 64) {
+      score[e] = expf(z[e] - most);
+      sum += score[e];
+    }
+    sum = tw_wave_sum(sum);
+    for (int e = lane; e < X; e += 64) {             // (a lane reads and writes its own experts only)
+      score[e] /= sum;
+      z[e] = score[e] + (bias ? bias[e] : 0.f);
+    }
+    __builtin_amdgcn_wave_barrier();
+    __threadfence_block();
+  }
   for (int r = 0; r < top; ++r) {
     float best = -INFINITY;
     int at = 0x7fffffff;
@@ -87,9 +111,10 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
       const int oa = __shfl_xor(at, o, TW_WAVE);
       if (ov > best || (ov == best && oa < at)) { best = ov; at = oa; }
     }
+    at = min(at, X - 1);                             // (no logit compares as the largest if all are NaN)
     if (lane == 0) {
       ids[(size_t)row * top + r] = at;
-      weights[(size_t)row * top + r] = mode == 1 ? best : 1.f / (1.f + expf(-best));
+      weights[(size_t)row * top + r] = mode == 2 ? score[at] : mode == 1 ? best : 1.f / (1.f + expf(-best));
       z[at] = -INFINITY;
     }
     __builtin_amdgcn_wave_barrier();
@@ -106,11 +131,17 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
     }
     for (int r = 0; r < top; ++r) w[r] = w[r] / sum;
   }
+  if (mode == 2 && lane == 0) {
+    float* w = weights + (size_t)row * top;
+    float sum = 1e-20f;
+    for (int r = 0; r < top; ++r) sum += w[r];
+    for (int r = 0; r < top; ++r) w[r] = w[r] / sum;
+  }
 }
 
 extern "C" int tw_moe_route(int dtype, const void* h, long ld_h, const float* router, const float* bias, int mode, int n, int C,
                             int X, int top, int* ids, float* weights, hipStream_t stream) {
-  TW_REQUIRE(h && router && ids && weights && n >= 0 && C > 0 && ld_h >= C && (mode == 0 || mode == 1));
+  TW_REQUIRE(h && router && ids && weights && n >= 0 && C > 0 && ld_h >= C && mode >= 0 && mode <= 2);
   TW_REQUIRE(X > 0 && X <= TW_MOE_MAX_EXPERTS && top > 0 && top <= X);
   if (n == 0) return 0;
   if (dtype == TW_DTYPE_BF16)
@@ -123,7 +154,7 @@ extern "C" int tw_moe_route(int dtype, const void* h, long ld_h, const float* ro
 
 // ---- plan ----------------------------------------------------------------------------------------------------
 // items = n * top pairs (token, choice). pos[item]: the pair's row in the experts' order; src_item[row]: the pair of a
-// row, -1 for padding; tile_expert[tile]: the expert of rows 16 tile .., -1 for a tile behind the last one in use.
+// row, -1 for padding (a pair whose expert is number X or above, one without matrices, gets no row: pos -1); tile_expert[tile]: the expert of rows 16 tile .., -1 for a tile behind the last one in use.
 // Which of an expert's rows a pair gets depends on the order the atomics arrive in; no result depends on it, since
 // every row is computed for itself and a token adds its rows in the order of its choices.
 __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ ids, int items, int X, int* __restrict__ pos,
@@ -135,7 +166,7 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
   for (int r = threadIdx.x; r < capacity; r += blockDim.x) src_item[r] = -1;
   for (int t = threadIdx.x; t < tiles; t += blockDim.x) tile_expert[t] = -1;
   __syncthreads();
-  for (int i = threadIdx.x; i < items; i += blockDim.x) pos[i] = atomicAdd(&count[ids[i]], 1);
+  for (int i = threadIdx.x; i < items; i += blockDim.x) pos[i] = ids[i] < X ? atomicAdd(&count[ids[i]], 1) : -1;
   __syncthreads();
   if (threadIdx.x == 0) {
     int at = 0;
@@ -149,6 +180,7 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
   for (int e = threadIdx.x; e < X; e += blockDim.x)
     for (int t = offset[e] / TW_MOE_TILE; t < offset[e + 1] / TW_MOE_TILE; ++t) tile_expert[t] = e;
   for (int i = threadIdx.x; i < items; i += blockDim.x) {
+    if (ids[i] >= X) continue;
     const int row = offset[ids[i]] + pos[i];
     pos[i] = row;
     src_item[row] = i;
@@ -206,14 +238,14 @@ __global__ __launch_bounds__(256) void moe_gather_kernel(const T* __restrict__ h
 // MT > 1 (steps of many rows, whose experts' shares are padded to MT tiles): a workgroup takes MT tiles of one expert
 // against every fragment of the expert's matrices it reads.
 template <int N> struct MoeCount { static constexpr int value = N; };
-// ACT 0: the float32 product; 1: gate and up with the limited swish; 2: one matrix with the exact gelu (1 and 2 write the
-// next product's rows in the compute type).
+// ACT 0: the float32 product; 1: gate and up with the limited swish; 2: one matrix with the exact gelu; 3: gate and up with
+// SiLU (1 to 3 write the next product's rows in the compute type).
 template <typename T, int ACT, int NT, bool SPLITK = false, int MT = 1>
 __global__ __launch_bounds__(256) void moe_grouped_kernel(const T* __restrict__ A, long lda, const T* __restrict__ W,
                                                           const T* __restrict__ W2, const int* __restrict__ tile_expert,
                                                           void* __restrict__ out, long ldo, int N, int K, float limit) {
   constexpr int EPF = Elem<T>::kPerFrag;
-  constexpr bool GLU = ACT == 1;
+  constexpr bool GLU = ACT == 1 || ACT == 3;
   const int tile = blockIdx.x * MT;
   const int ex = tile_expert[tile];
   if (ex < 0) return;
@@ -302,7 +334,8 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(const T* __restrict__ 
           // the activations are the next product's rows: in fragment order too (ldo: the elements of a row)
           const size_t at = (size_t)(tile + m) * ldo * TW_MOE_TILE + ((size_t)(col / EPF) * TW_MOE_TILE + 4 * g + j) * EPF + col % EPF;
           const float z = acc[m][t][j];
-          ((T*)out)[at] = tw_from_float<T>(GLU ? tw_swish_limited(z, acc2[m][t][j], limit)
+          ((T*)out)[at] = tw_from_float<T>(ACT == 1 ? tw_swish_limited(z, acc2[m][t][j], limit)
+                                               : ACT == 3 ? tw_silu(z) * acc2[m][t][j]
                                                : 0.5f * z * (1.f + erff(z * 0.70710678118654752f)));
         } else {
           ((float*)out)[(size_t)((tile + m) * TW_MOE_TILE + 4 * g + j) * ldo + col] = acc[m][t][j];
@@ -316,20 +349,26 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(const T* __restrict__ 
 // weights (or null): a factor on each of the token's rows; accumulate 0: x is written, not added to. more (or null):
 // float32 [splits][n][C] partial sums of something else that belongs to the same result (a shared expert's last product
 // with its K ranges not yet added up): added here, in index order, before the experts' rows.
-template <bool VEC>
+// A choice without a row (pos -1) is an expert that returns h itself.
+template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x, long ld_x, const float* __restrict__ ys,
                                                           long ld_y, const int* __restrict__ pos, int C, int top,
                                                           const float* __restrict__ weights, int accumulate,
-                                                          const float* __restrict__ more, int splits, size_t more_stride) {
+                                                          const float* __restrict__ more, int splits, size_t more_stride,
+                                                          const T* __restrict__ h, long ld_h) {
   const int row = blockIdx.x;
   const int c = blockIdx.y * 1024 + threadIdx.x * 4;
   if (c >= C) return;
+  const T* own = h + (size_t)row * ld_h + c;
   if constexpr (VEC) {
     f32x4 sum = {0.f, 0.f, 0.f, 0.f};
     if (more)
       for (int s = 0; s < splits; ++s) sum += *reinterpret_cast<const f32x4*>(more + s * more_stride + (size_t)row * C + c);
     for (int r = 0; r < top; ++r) {
-      const f32x4 y = *reinterpret_cast<const f32x4*>(ys + (size_t)pos[(size_t)row * top + r] * ld_y + c);
+      const int at = pos[(size_t)row * top + r];
+      f32x4 y;
+      if (at >= 0) y = *reinterpret_cast<const f32x4*>(ys + (size_t)at * ld_y + c);
+      else y = f32x4{tw_to_float(own[0]), tw_to_float(own[1]), tw_to_float(own[2]), tw_to_float(own[3])};
       if (weights) sum += weights[(size_t)row * top + r] * y;
       else sum += y;
     }
@@ -341,16 +380,79 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x,
       float sum = 0.f;
       if (more)
         for (int s = 0; s < splits; ++s) sum += more[s * more_stride + (size_t)row * C + c + j];
-      for (int r = 0; r < top; ++r)
-        sum += (weights ? weights[(size_t)row * top + r] : 1.f) * ys[(size_t)pos[(size_t)row * top + r] * ld_y + c + j];
+      for (int r = 0; r < top; ++r) {
+        const int at = pos[(size_t)row * top + r];
+        sum += (weights ? weights[(size_t)row * top + r] : 1.f) * (at >= 0 ? ys[(size_t)at * ld_y + c + j] : tw_to_float(own[j]));
+      }
       if (accumulate) x[(size_t)row * ld_x + c + j] += sum;
       else x[(size_t)row * ld_x + c + j] = sum;
     }
   }
 }
 
+// The two grouped products of a step: kind 0 gated with the limited swish, 1 up alone with gelu, 2 gated with SiLU.
+template <typename T, int ACT>
+static void moe_products(const T* xs, const T* gate, const T* up, const T* down, const int* tile_expert, T* act, float* ys, int C,
+                         int Cd, int Fd, float limit, int tiles, bool wide, hipStream_t stream) {
+  const T* first = ACT == 2 ? up : gate;
+  const T* second = ACT == 2 ? nullptr : up;
+  if (tiles <= TW_MOE_SPLITK_TILES) {
+    // few rows: most tiles hold one or two rows and each streams its expert's matrices once; the waves then split K
+    moe_grouped_kernel<T, ACT, 2, true><<<dim3(tiles, tw_div_up(Fd, 16 * 2)), 256, 0, stream>>>(
+        xs, Cd, first, second, tile_expert, act, Fd, Fd, Cd, limit);
+    moe_grouped_kernel<T, 0, 2, true><<<dim3(tiles, tw_div_up(C, 16 * 2)), 256, 0, stream>>>(
+        act, Fd, down, nullptr, tile_expert, ys, C, C, Fd, 0.f);
+  } else if (wide) {
+    moe_grouped_kernel<T, ACT, 2, false, TW_MOE_WIDE><<<dim3(tiles / TW_MOE_WIDE, tw_div_up(Fd, 4 * 16 * 2)), 256, 0, stream>>>(
+        xs, Cd, first, second, tile_expert, act, Fd, Fd, Cd, limit);
+    moe_grouped_kernel<T, 0, 2, false, TW_MOE_WIDE><<<dim3(tiles / TW_MOE_WIDE, tw_div_up(C, 4 * 16 * 2)), 256, 0, stream>>>(
+        act, Fd, down, nullptr, tile_expert, ys, C, C, Fd, 0.f);
+  } else {
+    moe_grouped_kernel<T, ACT, 2><<<dim3(tiles, tw_div_up(Fd, 4 * 16 * 2)), 256, 0, stream>>>(
+        xs, Cd, first, second, tile_expert, act, Fd, Fd, Cd, limit);
+    moe_grouped_kernel<T, 0, 4><<<dim3(tiles, tw_div_up(C, 4 * 16 * 4)), 256, 0, stream>>>(
+        act, Fd, down, nullptr, tile_expert, ys, C, C, Fd, 0.f);
+  }
+}
+
+struct MoeStep {
+  const void *h, *gate, *up, *down;
+  long ld_h, ld_x;
+  const float* weights;
+  const int *src_item, *tile_expert, *pos;
+  void *xs, *act;
+  float *ys, *x;
+  const float* more;
+  int n, top, C, Cd, Fd, capacity, kind, accumulate, more_splits;
+  float limit;
+  bool wide;
+};
+
+template <typename T>
+static void moe_run(const MoeStep& s, hipStream_t stream) {
+  moe_gather_kernel<T><<<s.capacity, 256, 0, stream>>>((const T*)s.h, s.ld_h, s.kind == 0 ? s.weights : nullptr, s.src_item,
+                                                       s.tile_expert, (T*)s.xs, s.C, s.Cd, s.top);
+  const int tiles = s.capacity / TW_MOE_TILE;
+#define TW_MOE_PRODUCTS(ACT)                                                                                            \
+  moe_products<T, ACT>((const T*)s.xs, (const T*)s.gate, (const T*)s.up, (const T*)s.down, s.tile_expert, (T*)s.act,    \
+                       s.ys, s.C, s.Cd, s.Fd, s.limit, tiles, s.wide, stream)
+  if (s.kind == 0) TW_MOE_PRODUCTS(1);
+  else if (s.kind == 1) TW_MOE_PRODUCTS(2);
+  else TW_MOE_PRODUCTS(3);
+#undef TW_MOE_PRODUCTS
+  const dim3 grid(s.n, tw_div_up(s.C, 1024));
+  const size_t more_stride = (size_t)s.n * s.C;
+  const float* weights = s.kind == 0 ? nullptr : s.weights;
+  if (s.C % 4 == 0 && s.ld_x % 4 == 0 && (uintptr_t)s.x % 16 == 0 && (uintptr_t)s.ys % 16 == 0 && (uintptr_t)s.more % 16 == 0)
+    moe_combine_kernel<T, true><<<grid, 256, 0, stream>>>(s.x, s.ld_x, s.ys, s.C, s.pos, s.C, s.top, weights, s.accumulate, s.more,
+                                                          s.more_splits, more_stride, (const T*)s.h, s.ld_h);
+  else
+    moe_combine_kernel<T, false><<<grid, 256, 0, stream>>>(s.x, s.ld_x, s.ys, s.C, s.pos, s.C, s.top, weights, s.accumulate, s.more,
+                                                           s.more_splits, more_stride, (const T*)s.h, s.ld_h);
+}
+
 // h [n][C] (compute type) -> x [n][C] float32 += the routed experts' results. ids, weights [n * top] come from
-// tw_moe_route. Scratch: pos [n * top], src_item [capacity], tile_expert [capacity / 16] (int32), xs [capacity][Cd],
+// tw_moe_route (ids of X and above, where the weights multiply outputs: experts that return h). Scratch: pos [n * top], src_item [capacity], tile_expert [capacity / 16] (int32), xs [capacity][Cd],
 // act [capacity][Fd] (compute type), ys [capacity][C] (float32), capacity = tw_moe_capacity(n * top, X).
 extern "C" int tw_moe_experts(int dtype, const void* h, long ld_h, const int* ids, const float* weights, int n, int top, int X,
                               const void* gate, const void* up, const void* down, int C, int Cd, int Fd, float limit,
@@ -358,97 +460,21 @@ extern "C" int tw_moe_experts(int dtype, const void* h, long ld_h, const int* id
                               float* x, long ld_x, int kind, int accumulate, const float* more, int more_splits,
                               hipStream_t stream) {
   TW_REQUIRE(h && ids && weights && up && down && pos && src_item && tile_expert && xs && act && ys && x);
-  TW_REQUIRE((kind == 0 && gate) || kind == 1);
+  TW_REQUIRE(((kind == 0 || kind == 2) && gate) || kind == 1);
   TW_REQUIRE(more == nullptr || more_splits > 0);
   if (kind == 1) gate = up;            // (never read: the alignment test below wants a pointer)
   TW_REQUIRE(n >= 0 && top > 0 && C > 0 && Cd >= C && Cd % 32 == 0 && Fd > 0 && Fd % 32 == 0 && ld_h >= C && ld_x >= C);
   TW_REQUIRE((uintptr_t)xs % 16 == 0 && (uintptr_t)act % 16 == 0 && (uintptr_t)gate % 16 == 0 && (uintptr_t)up % 16 == 0 &&
              (uintptr_t)down % 16 == 0);
+  TW_REQUIRE(dtype == TW_DTYPE_BF16 || dtype == TW_DTYPE_F32);
   if (n == 0) return 0;
   const int code = tw_moe_plan(ids, n * top, X, pos, src_item, tile_expert, capacity, stream);
   if (code) return code;
-  const int tiles = capacity / TW_MOE_TILE;
-  const dim3 glu_grid(tiles, tw_div_up(Fd, 4 * 16 * 2)), down_grid(tiles, tw_div_up(C, 4 * 16 * 4));
-  // few rows: most tiles hold one or two rows and each streams its expert's matrices once; the waves then split K
-  const bool few = tiles <= TW_MOE_SPLITK_TILES;
-  const dim3 glu_few(tiles, tw_div_up(Fd, 16 * 2)), down_few(tiles, tw_div_up(C, 16 * 2));
   const bool wide = moe_unit((long)n * top, X) == TW_MOE_TILE * TW_MOE_WIDE;
   TW_REQUIRE(!wide || capacity % (TW_MOE_TILE * TW_MOE_WIDE) == 0);
-  const dim3 glu_wide(tiles / TW_MOE_WIDE, tw_div_up(Fd, 4 * 16 * 2)), down_wide(tiles / TW_MOE_WIDE, tw_div_up(C, 4 * 16 * 2));
-  if (dtype == TW_DTYPE_BF16) {
-    typedef bf16_t T;
-    moe_gather_kernel<T><<<capacity, 256, 0, stream>>>((const T*)h, ld_h, kind == 0 ? weights : nullptr, src_item, tile_expert,
-                                                       (T*)xs, C, Cd, top);
-    if (few) {
-      if (kind == 0)
-        moe_grouped_kernel<T, 1, 2, true><<<glu_few, 256, 0, stream>>>((const T*)xs, Cd, (const T*)gate, (const T*)up,
-                                                                       tile_expert, act, Fd, Fd, Cd, limit);
-      else
-        moe_grouped_kernel<T, 2, 2, true><<<glu_few, 256, 0, stream>>>((const T*)xs, Cd, (const T*)up, nullptr,
-                                                                       tile_expert, act, Fd, Fd, Cd, 0.f);
-      moe_grouped_kernel<T, 0, 2, true><<<down_few, 256, 0, stream>>>((const T*)act, Fd, (const T*)down, nullptr,
-                                                                         tile_expert, ys, C, C, Fd, 0.f);
-    } else if (wide) {
-      if (kind == 0)
-        moe_grouped_kernel<T, 1, 2, false, TW_MOE_WIDE><<<glu_wide, 256, 0, stream>>>(
-            (const T*)xs, Cd, (const T*)gate, (const T*)up, tile_expert, act, Fd, Fd, Cd, limit);
-      else
-        moe_grouped_kernel<T, 2, 2, false, TW_MOE_WIDE><<<glu_wide, 256, 0, stream>>>(
-            (const T*)xs, Cd, (const T*)up, nullptr, tile_expert, act, Fd, Fd, Cd, 0.f);
-      moe_grouped_kernel<T, 0, 2, false, TW_MOE_WIDE><<<down_wide, 256, 0, stream>>>(
-          (const T*)act, Fd, (const T*)down, nullptr, tile_expert, ys, C, C, Fd, 0.f);
-    } else {
-      if (kind == 0)
-        moe_grouped_kernel<T, 1, 2><<<glu_grid, 256, 0, stream>>>((const T*)xs, Cd, (const T*)gate, (const T*)up,
-                                                                  tile_expert, act, Fd, Fd, Cd, limit);
-      else
-        moe_grouped_kernel<T, 2, 2><<<glu_grid, 256, 0, stream>>>((const T*)xs, Cd, (const T*)up, nullptr,
-                                                                  tile_expert, act, Fd, Fd, Cd, 0.f);
-      moe_grouped_kernel<T, 0, 4><<<down_grid, 256, 0, stream>>>((const T*)act, Fd, (const T*)down, nullptr,
-                                                                    tile_expert, ys, C, C, Fd, 0.f);
-    }
-  } else if (dtype == TW_DTYPE_F32) {
-    typedef float T;
-    moe_gather_kernel<T><<<capacity, 256, 0, stream>>>((const T*)h, ld_h, kind == 0 ? weights : nullptr, src_item, tile_expert,
-                                                       (T*)xs, C, Cd, top);
-    if (few) {
-      if (kind == 0)
-        moe_grouped_kernel<T, 1, 2, true><<<glu_few, 256, 0, stream>>>((const T*)xs, Cd, (const T*)gate, (const T*)up,
-                                                                       tile_expert, act, Fd, Fd, Cd, limit);
-      else
-        moe_grouped_kernel<T, 2, 2, true><<<glu_few, 256, 0, stream>>>((const T*)xs, Cd, (const T*)up, nullptr,
-                                                                       tile_expert, act, Fd, Fd, Cd, 0.f);
-      moe_grouped_kernel<T, 0, 2, true><<<down_few, 256, 0, stream>>>((const T*)act, Fd, (const T*)down, nullptr,
-                                                                         tile_expert, ys, C, C, Fd, 0.f);
-    } else if (wide) {
-      if (kind == 0)
-        moe_grouped_kernel<T, 1, 2, false, TW_MOE_WIDE><<<glu_wide, 256, 0, stream>>>(
-            (const T*)xs, Cd, (const T*)gate, (const T*)up, tile_expert, act, Fd, Fd, Cd, limit);
-      else
-        moe_grouped_kernel<T, 2, 2, false, TW_MOE_WIDE><<<glu_wide, 256, 0, stream>>>(
-            (const T*)xs, Cd, (const T*)up, nullptr, tile_expert, act, Fd, Fd, Cd, 0.f);
-      moe_grouped_kernel<T, 0, 2, false, TW_MOE_WIDE><<<down_wide, 256, 0, stream>>>(
-          (const T*)act, Fd, (const T*)down, nullptr, tile_expert, ys, C, C, Fd, 0.f);
-    } else {
-      if (kind == 0)
-        moe_grouped_kernel<T, 1, 2><<<glu_grid, 256, 0, stream>>>((const T*)xs, Cd, (const T*)gate, (const T*)up,
-                                                                  tile_expert, act, Fd, Fd, Cd, limit);
-      else
-        moe_grouped_kernel<T, 2, 2><<<glu_grid, 256, 0, stream>>>((const T*)xs, Cd, (const T*)up, nullptr,
-                                                                  tile_expert, act, Fd, Fd, Cd, 0.f);
-      moe_grouped_kernel<T, 0, 4><<<down_grid, 256, 0, stream>>>((const T*)act, Fd, (const T*)down, nullptr,
-                                                                    tile_expert, ys, C, C, Fd, 0.f);
-    }
-  } else {
-    return TW_ERR_BAD_ARGUMENT;
-  }
-  const dim3 combine_grid(n, tw_div_up(C, 1024));
-  const size_t more_stride = (size_t)n * C;
-  if (C % 4 == 0 && ld_x % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)ys % 16 == 0 && (uintptr_t)more % 16 == 0)
-    moe_combine_kernel<true><<<combine_grid, 256, 0, stream>>>(x, ld_x, ys, C, pos, C, top, kind == 1 ? weights : nullptr, accumulate,
-                                                               more, more_splits, more_stride);
-  else
-    moe_combine_kernel<false><<<combine_grid, 256, 0, stream>>>(x, ld_x, ys, C, pos, C, top, kind == 1 ? weights : nullptr, accumulate,
-                                                                more, more_splits, more_stride);
+  const MoeStep s{h, gate, up, down, ld_h, ld_x, weights, src_item, tile_expert, pos, xs, act, ys, x, more,
+                  n, top, C, Cd, Fd, capacity, kind, accumulate, more_splits, limit, wide};
+  if (dtype == TW_DTYPE_BF16) moe_run<bf16_t>(s, stream);
+  else moe_run<float>(s, stream);
   return TW_LAUNCH_RESULT();
 }

@@ -97,3 +97,84 @@ extern "C" int tw_qk_finish(int dtype, const float* src, long ld, int q_col, int
   else return TW_ERR_BAD_ARGUMENT;
   return TW_LAUNCH_RESULT();
 }
+
+// ---- queries and keys normed per head, without a rotation ----------------------------------------------------------
+// What stands between the projections and the attention of a mixer whose heads are normed one by one and whose positions
+// enter as a temperature of the queries:
+//
+//   q <- temperature(p) * unit(q_h),  k <- unit(k_g),  v as it comes;   temperature(p) = 1 + coef * ln(floor((p + 1) / every) + 1)
+//
+// unit(.) over a head's D elements. q, k and v are columns of float32 rows; each result is rounded once to the compute
+// type: queries to q_out with heads of Dp elements (tails of zeros), keys and values (of E elements) into the token's page
+// slot, keys [pages][G][P][Dp], values [pages][G][Dp][P]. One wave a (token, head): H query heads, then G key/value heads.
+struct HeadFinishArgs {
+  const float* src; long ld;
+  int q_col, k_col, v_col;
+  const int* positions;
+  void* q_out; long ld_q;
+  void* keys; void* values; const int* slots;
+  int n, H, G, D, E, Dp, P;
+  int every;                    // 0: no temperature
+  float coef, eps;
+};
+
+template <typename T>
+__global__ __launch_bounds__(256) void head_finish_kernel(HeadFinishArgs a) {
+  const long unit = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (unit >= (long)a.n * (a.H + a.G)) return;
+  const int lane = threadIdx.x & 63;
+  const int n = (int)(unit / (a.H + a.G)), head = (int)(unit % (a.H + a.G));
+  const bool query = head < a.H;
+  const int g = head - a.H;
+  const float* row = a.src + (size_t)n * a.ld;
+  const float* x = row + (query ? a.q_col + head * a.D : a.k_col + g * a.D);
+  float v[4], ss = 0.f;                           // D <= 256
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int d = lane + 64 * i;
+    v[i] = d < a.D ? x[d] : 0.f;
+    ss = __fmaf_rn(v[i], v[i], ss);
+  }
+  float f = 1.f / sqrtf(tw_wave_sum(ss) / (float)a.D + a.eps);
+  if (query) {
+    if (a.every > 0) f *= __fmaf_rn(a.coef, logf((float)((a.positions[n] + 1) / a.every + 1)), 1.f);
+    T* q = (T*)a.q_out + (size_t)n * a.ld_q + (size_t)head * a.Dp;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = lane + 64 * i;
+      if (d < a.Dp) q[d] = tw_from_float<T>(v[i] * f);
+    }
+    return;
+  }
+  const int slot = a.slots[n];
+  if (slot < 0) return;
+  const int page = slot / a.P, at = slot % a.P;
+  T* k = (T*)a.keys + (((size_t)page * a.G + g) * a.P + at) * a.Dp;
+  T* vals = (T*)a.values + ((size_t)page * a.G + g) * a.Dp * a.P + at;
+  const float* value = row + a.v_col + g * a.E;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int d = lane + 64 * i;
+    if (d < a.Dp) {
+      k[d] = tw_from_float<T>(v[i] * f);
+      vals[(size_t)d * a.P] = tw_from_float<T>(d < a.E ? value[d] : 0.f);
+    }
+  }
+}
+
+extern "C" int tw_head_finish(int dtype, const float* src, long ld, int q_col, int k_col, int v_col, const int* positions,
+                              void* q_out, long ld_q, void* keys, void* values, const int* slots, int n, int H, int G, int D,
+                              int E, int Dp, int page_size, int every, float coef, float eps, hipStream_t stream) {
+  TW_REQUIRE(src && positions && q_out && keys && values && slots && n >= 0 && H > 0 && G > 0 && D > 0 && E > 0);
+  TW_REQUIRE(Dp >= D && Dp >= E && Dp <= 256 && q_col >= 0 && k_col >= 0 && v_col >= 0 && ld >= q_col + (long)H * D &&
+             ld >= k_col + (long)G * D && ld >= v_col + (long)G * E && ld_q >= (long)H * Dp);
+  TW_REQUIRE(page_size > 0 && eps > 0.f && every >= 0);
+  if (n == 0) return 0;
+  HeadFinishArgs a{src, ld, q_col, k_col, v_col, positions, q_out, ld_q, keys, values, slots, n, H, G, D, E, Dp, page_size,
+                   every, coef, eps};
+  const int blocks = tw_div_up((long)n * (H + G), 4);
+  if (dtype == TW_DTYPE_BF16) head_finish_kernel<bf16_t><<<blocks, 256, 0, stream>>>(a);
+  else if (dtype == TW_DTYPE_F32) head_finish_kernel<float><<<blocks, 256, 0, stream>>>(a);
+  else return TW_ERR_BAD_ARGUMENT;
+  return TW_LAUNCH_RESULT();
+}

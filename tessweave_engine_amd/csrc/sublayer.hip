@@ -353,3 +353,126 @@ extern "C" int tw_softcap_values(float* x, long total, float cap, hipStream_t st
   softcap_values_kernel<<<tw_div_up(total, 256), 256, 0, stream>>>(x, total, cap);
   return TW_LAUNCH_RESULT();
 }
+
+// ---- several results side by side, each normed, summed into the stream: x <- x + sum_b mult_b * w_b * unit(y_b) ----
+// Every y_b [n][hidden] is float32, or the split-K partial sums of a product that are added up here, in index order. A
+// block a row; a row of a result stays in registers between its two passes up to 4,096 elements.
+#define TW_NORMED_SUM_MOST 4
+struct NormedSumArgs {
+  float* x;
+  const float* y[TW_NORMED_SUM_MOST];
+  const float* w[TW_NORMED_SUM_MOST];
+  float mult[TW_NORMED_SUM_MOST];
+  int splits[TW_NORMED_SUM_MOST];       // partial sums of y_b (1: y_b itself), n * hidden floats apart
+  size_t stride;
+  int count, hidden;
+  float eps;
+};
+
+template <int W>
+__global__ __launch_bounds__(256) void add_normed_sum_kernel(NormedSumArgs a) {
+  __shared__ float lds[16];
+  constexpr int KEEP = 4;
+  const int units = a.hidden / W;
+  const size_t row0 = (size_t)blockIdx.x * a.hidden;
+  float* x = a.x + row0;
+  float sum[KEEP][W];
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i)
+#pragma unroll
+    for (int e = 0; e < W; ++e) sum[i][e] = 0.f;
+  for (int b = 0; b < a.count; ++b) {
+    const float* y = a.y[b] + row0;
+    const int splits = a.splits[b];
+    auto load = [&](int u, float* v) {
+#pragma unroll
+      for (int e = 0; e < W; ++e) v[e] = 0.f;
+      for (int s = 0; s < splits; ++s) {
+        if (W == 4) {
+          const f32x4 t = *reinterpret_cast<const f32x4*>(y + s * a.stride + (size_t)u * 4);
+#pragma unroll
+          for (int e = 0; e < W; ++e) v[e] += t[e];
+        } else {
+          v[0] += y[s * a.stride + u];
+        }
+      }
+    };
+    float kept[KEEP][W];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+      const int u = threadIdx.x + i * 256;
+#pragma unroll
+      for (int e = 0; e < W; ++e) kept[i][e] = 0.f;
+      if (u < units) load(u, kept[i]);
+#pragma unroll
+      for (int e = 0; e < W; ++e) ss = __fmaf_rn(kept[i][e], kept[i][e], ss);
+    }
+    for (int u = threadIdx.x + KEEP * 256; u < units; u += 256) {
+      float v[W];
+      load(u, v);
+#pragma unroll
+      for (int e = 0; e < W; ++e) ss = __fmaf_rn(v[e], v[e], ss);
+    }
+    const float f = a.mult[b] / sqrtf(tw_block_sum(ss, lds) / (float)a.hidden + a.eps);
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+      const int u = threadIdx.x + i * 256;
+      if (u < units) {
+#pragma unroll
+        for (int e = 0; e < W; ++e) sum[i][e] = __fmaf_rn(kept[i][e] * f, a.w[b][u * W + e], sum[i][e]);
+      }
+    }
+    for (int u = threadIdx.x + KEEP * 256; u < units; u += 256) {       // (longer rows: one result after the other into x)
+      float v[W];
+      load(u, v);
+#pragma unroll
+      for (int e = 0; e < W; ++e) x[u * W + e] = __fmaf_rn(v[e] * f, a.w[b][u * W + e], x[u * W + e]);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i) {
+    const int u = threadIdx.x + i * 256;
+    if (u < units) {
+#pragma unroll
+      for (int e = 0; e < W; ++e) x[u * W + e] += sum[i][e];
+    }
+  }
+}
+
+extern "C" int tw_add_normed_sum(float* x, int count, const float* const* ys, const int* splits, const float* const* ws,
+                                 const float* mults, int n, int hidden, float eps, hipStream_t stream) {
+  TW_REQUIRE(x && ys && splits && ws && mults && n >= 0 && hidden > 0 && eps > 0.f && count > 0 && count <= TW_NORMED_SUM_MOST);
+  NormedSumArgs a{};
+  a.x = x;
+  a.stride = (size_t)n * hidden;
+  a.count = count;
+  a.hidden = hidden;
+  a.eps = eps;
+  bool vec = hidden % 4 == 0 && (uintptr_t)x % 16 == 0;
+  for (int b = 0; b < count; ++b) {
+    TW_REQUIRE(ys[b] && ws[b] && splits[b] > 0);
+    a.y[b] = ys[b];
+    a.w[b] = ws[b];
+    a.mult[b] = mults[b];
+    a.splits[b] = splits[b];
+    vec = vec && (uintptr_t)ys[b] % 16 == 0;
+  }
+  if (n == 0) return 0;
+  if (vec) add_normed_sum_kernel<4><<<n, 256, 0, stream>>>(a);
+  else add_normed_sum_kernel<1><<<n, 256, 0, stream>>>(a);
+  return TW_LAUNCH_RESULT();
+}
+
+// ---- x += y over float32 values --------------------------------------------------------------------------------------
+__global__ void add_values_kernel(float* __restrict__ x, const float* __restrict__ y, long total) {
+  const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < total) x[i] += y[i];
+}
+
+extern "C" int tw_add_values(float* x, const float* y, long total, hipStream_t stream) {
+  TW_REQUIRE(x && y && total >= 0);
+  if (total == 0) return 0;
+  add_values_kernel<<<tw_div_up(total, 256), 256, 0, stream>>>(x, y, total);
+  return TW_LAUNCH_RESULT();
+}

@@ -79,6 +79,15 @@ _SIGNATURES = {
     "tw_softcap_values": (I, [P, L, F, P]),
     "tw_qk_finish": (I, [I, P, L, I, I, P, P, P, P, P, L, P, P, P, I, I, I, I, I, I, I, I, F, P]),
     "tw_mlstm": (I, [P, L, I, I, I, I, I, P, P, P, P, P, P, P, P, I, I, P, L, I, I, I, F, F, I, I, I, P]),
+    "tw_embed_sinusoid": (I, [I, P, P, P, P, P, P, P, F, I, I, I, P, I, P]),
+    "tw_head_finish": (I, [I, P, L, I, I, I, P, P, L, P, P, P, I, I, I, I, I, I, I, I, F, F, P]),
+    "tw_add_normed_sum": (I, [P, I, ctypes.POINTER(c_void_p), ctypes.POINTER(c_int), ctypes.POINTER(c_void_p),
+                              ctypes.POINTER(c_float), I, I, F, P]),
+    "tw_add_values": (I, [P, P, L, P]),
+    "tw_linear_state_workspace_floats": (L, [I, I, I, I, I]),
+    "tw_linear_state": (I, [P, L, I, I, I, I, P, L, P, L, I, P, P, P, P, P, P, I, I, I, P, L, I, I, I, F, I, P, L, P]),
+    "tw_decay_logs": (I, [P, L, P, P, F, P, L, I, I, I, P]),
+    "tw_gate_group_norm": (I, [I, P, L, P, L, P, P, L, I, I, I, F, P]),
     "tw_sampling_uniform": (F, [c_uint64, c_uint64]),
     "tw_sample_workspace_bytes": (L, [I]),
     "tw_sample_rows": (I, [P, L, I, I, P, P, P, P, P, L, P]),

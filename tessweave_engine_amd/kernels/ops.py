@@ -1136,14 +1136,15 @@ def head_norm_gate(o, gate, weight, out, heads, value_dim, eps, gate_activation=
 MOE_MAX_EXPERTS = 1024
 
 
-MOE_WEIGHTS = {"sigmoid": 0, "softmax_chosen": 1}
+MOE_WEIGHTS = {"sigmoid": 0, "softmax_chosen": 1, "softmax_all": 2}
 
 
 def moe_route(h, router, top, ids, weights, bias=None, weighting="sigmoid"):
     """ids[n, top], weights[n, top]: per row of h the `top` experts with the largest router logits router @ h + bias
     (float32 products of h's values as they are; the lowest index wins a tie), and per chosen logit its sigmoid or
-    ("softmax_chosen") its share of the softmax over the chosen logits alone."""
-    _need(weighting in MOE_WEIGHTS, "a router's weights are 'sigmoid' or 'softmax_chosen'")
+    ("softmax_chosen") its share of the softmax over the chosen logits alone. "softmax_all": s = softmax(router @ h), the
+    experts with the largest s + bias are chosen, their weights are their s over the chosen ones' sum (+ 1e-20)."""
+    _need(weighting in MOE_WEIGHTS, f"a router's weights are one of {sorted(MOE_WEIGHTS)}")
     n, C, ld_h = _rows(h, "h")
     X = router.shape[0]
     _need(router.dtype == torch.float32 and router.is_contiguous() and tuple(router.shape) == (X, C), "the router is float32 [experts, C]")
@@ -1180,18 +1181,20 @@ def moe_blocked(w):
     return w.reshape(X, N16 // 16, 16, K // (4 * epf), 4, epf).permute(0, 1, 3, 4, 2, 5).contiguous().reshape(X, N16, K)
 
 
-MOE_KINDS = {"swish_limited": 0, "gelu": 1}
+MOE_KINDS = {"swish_limited": 0, "gelu": 1, "silu": 2}
 
 
 def moe_experts(h, ids, weights, gate, up, down, limit, x, scratch, kind="swish_limited", accumulate=True, more=None):
     """kind "gelu" (gate None): x[n] (+)= sum over a row's chosen experts e of weights_e * down_e(gelu(up_e h[n])), the exact
     gelu; accumulate=False writes x instead of adding to it; more: float32 [splits, n, C] partial sums of something that
-    belongs to the same result (a shared expert's last product), added up here as well. kind "swish_limited": x[n] += sum over a row's chosen experts e of down_e(glu(gate_e y, up_e y)), y = round(weights * h[n]), glu the
+    belongs to the same result (a shared expert's last product), added up here as well. kind "silu": the same with
+    down_e(silu(gate_e h[n]) * (up_e h[n])); in these two kinds an id of X or above names an expert that returns h[n] itself.
+    kind "swish_limited": x[n] += sum over a row's chosen experts e of down_e(glu(gate_e y, up_e y)), y = round(weights * h[n]), glu the
     limited swish with LIMIT. gate, up [X, Fd, Cd], down [X, C16, Fd] in h's type, zero padded (Fd, Cd: `moe_pad` of the
     sizes, C16: C rounded up to 16) and laid out by `moe_blocked`. scratch(tag, shape, dtype) hands out the step's scratch tensors."""
     n, C, ld_h = _rows(h, "h")
     top = ids.shape[1]
-    _need(kind in MOE_KINDS and (gate is None) == (kind == "gelu"), "experts are 'swish_limited' (with a gate) or 'gelu' (without)")
+    _need(kind in MOE_KINDS and (gate is None) == (kind == "gelu"), f"experts are one of {sorted(MOE_KINDS)}, all but 'gelu' with a gate")
     X, Fd, Cd = up.shape
     _need((gate is None or (gate.is_contiguous() and gate.dtype == h.dtype and tuple(gate.shape) == (X, Fd, Cd)))
           and up.is_contiguous() and down.is_contiguous() and up.dtype == down.dtype == h.dtype,
@@ -1344,4 +1347,161 @@ def mlstm(proj, q_col, k_col, v_col, i_col, f_col, i_bias, f_bias, S, n_state, m
                              _dev(state_slots, torch.int32, "state_slots"), _dev(phase, torch.int32, "phase"), int(seq0),
                              int(n_seqs), _dev(out), ld_out, int(heads), int(dim), int(value_dim), float(q_scale), float(cap),
                              1 if walk else 0, -1 if (walk or first_row is None) else int(first_row), n, _stream()), "mlstm")
+    return out
+
+
+# ---- sinusoidal positions, per-head norms with a query temperature, linear recurrences with a decaying matrix state --------
+
+def embed_sinusoid(ids, table, positions, freq, rest, scale, out, copy=None, feed=None):
+    """out[n] = scale * table[ids[n]] + s(positions[n]), s(p)[2 i] = sin(p (freq + rest)[i]), s(p)[2 i + 1] the cosine;
+    COPY, if given, receives the same. freq, rest float32 [ceil(hidden / 2)]: a frequency and what float32 rounded off it."""
+    n = ids.numel()
+    vocab, hidden = table.shape
+    _need(table.is_contiguous() and out.is_contiguous() and tuple(out.shape) == (n, hidden), "embed_sinusoid: table and out [n, hidden] must be contiguous")
+    _need(copy is None or (copy.is_contiguous() and tuple(copy.shape) == (n, hidden)), "the copy must have out's shape")
+    half = (hidden + 1) // 2
+    for t in (freq, rest):
+        _need(t.dtype == torch.float32 and t.is_contiguous() and t.numel() == half, "frequencies are float32 [ceil(hidden / 2)]")
+    _need(positions.numel() == n, "one position per token is needed")
+    check(library().tw_embed_sinusoid(dtype_id(table.dtype), _dev(ids, torch.int32, "ids"), _dev(table), _dev(out, torch.float32, "out"),
+                                      _dev(copy, torch.float32, "copy") if copy is not None else None,
+                                      _dev(positions, torch.int32, "positions"), _dev(freq), _dev(rest), float(scale), n, hidden,
+                                      vocab, _dev(feed, torch.int32, "feed") if feed is not None else None,
+                                      feed.numel() if feed is not None else 0, _stream()), "embed_sinusoid")
+    return out
+
+
+def head_finish(src, q_col, k_col, v_col, positions, q_out, keys, values, slots, q_heads, kv_heads, dim, value_dim, eps,
+                temperature=None):
+    """Per token and head: q <- t(p) * unit(q), k <- unit(k) (unit: over the head's dim elements, x / sqrt(mean(x^2) + eps)),
+    v as it comes; t(p) = 1 + coef * ln(floor((p + 1) / every) + 1) with temperature = (coef, every), None: 1. src float32
+    rows with q, k (heads of dim) and v (of value_dim) at the given columns. q_out [n, q_heads * dim_dev] in the compute type
+    (tails of zeros); keys [pages, kv_heads, page, dim_dev], values [pages, kv_heads, dim_dev, page]; slots[n] the token's
+    page slot (-1: not stored)."""
+    n, width, ld = _rows(src, "src")
+    nq, wq, ld_q = _rows(q_out, "q_out")
+    page, dim_dev = keys.shape[2], keys.shape[3]
+    _need(src.dtype == torch.float32 and nq == n and wq == q_heads * dim_dev, "head_finish: src float32, q_out [n, q_heads * dim_dev]")
+    _need(keys.is_contiguous() and values.is_contiguous() and keys.dtype == values.dtype == q_out.dtype
+          and tuple(keys.shape[1:]) == (kv_heads, page, dim_dev) and values.numel() == keys.numel(),
+          "keys [pages, kv_heads, page, dim_dev] and values of q_out's type and the same size")
+    _need(0 < dim <= dim_dev <= 256 and 0 < value_dim <= dim_dev and min(q_col, k_col, v_col) >= 0
+          and q_col + q_heads * dim <= width and k_col + kv_heads * dim <= width and v_col + kv_heads * value_dim <= width,
+          "head_finish: columns exceed the rows")
+    _need(slots.numel() == n and positions.numel() == n, "one slot and one position per row are needed")
+    coef, every = temperature if temperature is not None else (0.0, 0)
+    check(library().tw_head_finish(dtype_id(q_out.dtype), _dev(src), ld, int(q_col), int(k_col), int(v_col),
+                                   _dev(positions, torch.int32, "positions"), _dev(q_out), ld_q, _dev(keys), _dev(values),
+                                   _dev(slots, torch.int32, "slots"), n, int(q_heads), int(kv_heads), int(dim), int(value_dim),
+                                   dim_dev, page, int(every), float(coef), float(eps), _stream()), "head_finish")
+    return q_out
+
+
+def add_normed_sum(x, results, eps):
+    """x += sum over RESULTS (y, weight, mult) of mult * weight * y / sqrt(mean(y^2) + eps); x float32 [n, hidden]; y float32
+    [n, hidden], or [splits, n, hidden] partial sums that are added up here. At most four results."""
+    import ctypes
+    _need(x.dim() == 2 and x.is_contiguous() and x.dtype == torch.float32, "add_normed_sum: x must be contiguous float32 [n, hidden]")
+    n, hidden = x.shape
+    k = len(results)
+    _need(1 <= k <= 4, "add_normed_sum takes one to four results")
+    ys, ws = (ctypes.c_void_p * k)(), (ctypes.c_void_p * k)()
+    splits, mults = (ctypes.c_int * k)(), (ctypes.c_float * k)()
+    for i, (y, w, mult) in enumerate(results):
+        _need(y.is_contiguous() and tuple(y.shape[-2:]) == (n, hidden) and y.dim() in (2, 3), "a result is [n, hidden] or [splits, n, hidden]")
+        _need(w.dtype == torch.float32 and w.is_contiguous() and w.numel() == hidden, "the norm weights are float32 [hidden]")
+        ys[i], ws[i] = _dev(y, torch.float32, "y"), _dev(w)
+        splits[i], mults[i] = (y.shape[0] if y.dim() == 3 else 1), float(mult)
+    check(library().tw_add_normed_sum(_dev(x), k, ys, splits, ws, mults, n, hidden, float(eps), _stream()), "add_normed_sum")
+    return x
+
+
+def add_values(x, y):
+    """x += y in place (contiguous float32 tensors of one size)."""
+    _need(x.is_contiguous() and y.is_contiguous() and x.numel() == y.numel(), "add_values takes contiguous tensors of one size")
+    check(library().tw_add_values(_dev(x, torch.float32, "x"), _dev(y, torch.float32, "y"), x.numel(), _stream()), "add_values")
+    return x
+
+
+LINEAR_STATE_WALK_TOKENS = 4          # sequences with up to this many tokens in a step are walked token by token
+
+
+def linear_state_workspace_floats(n_seqs, max_q_len, heads, dim, value_dim):
+    """float32 scratch the chunked form of `linear_state` needs for portions of up to max_q_len tokens (0: none)."""
+    up = lambda v: (int(v) + 15) // 16 * 16       # noqa: E731
+    return int(library().tw_linear_state_workspace_floats(int(n_seqs), int(max_q_len), int(heads), up(dim), up(value_dim)))
+
+
+def linear_state(src, q_col, k_col, v_col, state, q_start, state_slots, seq0, n_seqs, out, heads, dim, value_dim, groups=None,
+                 q_scale=1.0, logs=None, raw=None, raw_col=0, dt_bias=None, A_log=None, skip=None, walk=True, max_q_len=1,
+                 workspace=None):
+    """S <- d S + k v^T, o = S^T (q_scale q) per head over sequences seq0 .. seq0 + n_seqs - 1, from and to state float32
+    [requests, heads, Ep, Dp] (dim and value_dim rounded up to 16; a column of S is contiguous).
+
+    src float32 [n, .]: q and k of head h at q_col / k_col + (h // (heads / groups)) * dim (groups None: one per head), v at
+    v_col + h * value_dim. The decay d: logs float32 [n, >= heads * dim], its logarithm per key element; or, with logs None,
+    one number a head: delta = softplus(raw[n, raw_col + h] + dt_bias_h), d = exp(-exp(A_log_h) delta), the key then is
+    delta k, and skip_h v is added to the result. out float32 [n, heads * value_dim]. walk: token by token (steps of a few
+    tokens a sequence), else chunks of 16 on the matrix unit for portions of up to max_q_len tokens, with a float32 workspace
+    of `linear_state_workspace_floats` floats where that is not zero."""
+    n, width, ld = _rows(src, "src")
+    no, wo, ld_out = _rows(out, "out")
+    groups = heads if groups is None else int(groups)
+    _need(groups > 0 and heads % groups == 0 and 1 <= dim <= 256, "heads must be a multiple of groups, keys up to 256")
+    Dp, Ep = (dim + 15) // 16 * 16, (value_dim + 15) // 16 * 16
+    _need(src.dtype == torch.float32 and out.dtype == torch.float32 and no == n and wo == heads * value_dim, "linear_state: float32 rows")
+    _need(min(q_col, k_col, v_col) >= 0 and max(q_col, k_col) + groups * dim <= width and v_col + heads * value_dim <= width,
+          "linear_state: columns exceed the rows")
+    _need(state.dtype == torch.float32 and state.is_contiguous() and state.dim() == 4 and tuple(state.shape[1:]) == (heads, Ep, Dp),
+          "state must be float32 [requests, heads, Ep, Dp]")
+    ld_logs = ld_raw = 0
+    if logs is not None:
+        nl, wl, ld_logs = _rows(logs, "logs")
+        _need(logs.dtype == torch.float32 and nl == n and wl >= heads * dim, "logs must be float32 [n, heads * dim]")
+    else:
+        nr, wr, ld_raw = _rows(raw, "raw")
+        _need(raw.dtype == torch.float32 and nr == n and 0 <= raw_col and raw_col + heads <= wr, "raw must be float32 rows with a column per head")
+        for t, name in ((dt_bias, "dt_bias"), (A_log, "A_log")) + (((skip, "skip"),) if skip is not None else ()):
+            _need(t.dtype == torch.float32 and t.is_contiguous() and t.numel() == heads, f"{name} must be float32 [heads]")
+    _need(seq0 >= 0 and q_start.numel() >= seq0 + n_seqs + 1 and state_slots.numel() >= seq0 + n_seqs, "sequence metadata is too short")
+    need = 0 if walk else linear_state_workspace_floats(n_seqs, max_q_len, heads, dim, value_dim)
+    if need:
+        _need(workspace is not None and workspace.dtype == torch.float32 and workspace.is_contiguous() and workspace.numel() >= need,
+              "long portions need a float32 workspace of linear_state_workspace_floats floats")
+    head = logs is None
+    check(library().tw_linear_state(_dev(src), ld, int(q_col), int(k_col), int(v_col), heads // groups,
+                                    None if head else _dev(logs), ld_logs, _dev(raw) if head else None, ld_raw, int(raw_col),
+                                    _dev(dt_bias) if head else None, _dev(A_log) if head else None,
+                                    _dev(skip) if head and skip is not None else None, _dev(state),
+                                    _dev(q_start, torch.int32, "q_start"), _dev(state_slots, torch.int32, "state_slots"), int(seq0),
+                                    int(n_seqs), max(1, int(max_q_len)), _dev(out), ld_out, int(heads), int(dim), int(value_dim),
+                                    float(q_scale), 1 if walk else 0, _dev(workspace) if need else None,
+                                    workspace.numel() if need else 0, _stream()), "linear_state")
+    return out
+
+
+def decay_logs(low, up, bias, tau, out):
+    """out[n, c] = log sigmoid(low[n] @ up[:, c] + bias[c]) / tau; low float32 [n, rank], up float32 [rank, channels]."""
+    n, rank, ld = _rows(low, "low")
+    no, channels, ld_out = _rows(out, "out")
+    _need(low.dtype == up.dtype == bias.dtype == out.dtype == torch.float32 and no == n, "decay_logs takes float32 operands")
+    _need(up.is_contiguous() and tuple(up.shape) == (rank, channels) and bias.is_contiguous() and bias.numel() == channels
+          and float(tau) > 0, "up must be [rank, channels], bias [channels], tau positive")
+    check(library().tw_decay_logs(_dev(low), ld, _dev(up), _dev(bias), float(tau), _dev(out), ld_out, n, rank, channels, _stream()),
+          "decay_logs")
+    return out
+
+
+def gate_group_norm(y, gate, weight, out, parts, eps):
+    """out[n] = weight * (u in `parts` equal parts, each over its root mean square sqrt(mean + eps)), u = y * silu(gate); y and
+    gate float32, weight float32 over the whole row, out of the compute type."""
+    n, width, ld_y = _rows(y, "y")
+    ng, wg, ld_g = _rows(gate, "gate")
+    no, wo, ld_o = _rows(out, "out")
+    _need(y.dtype == torch.float32 and gate.dtype == torch.float32 and ng == n and no == n and wg == width and wo == width,
+          "gate_group_norm: y, gate float32 and out [n, width]")
+    _need(parts > 0 and width % parts == 0 and weight.dtype == torch.float32 and weight.is_contiguous() and weight.numel() == width,
+          "the parts must divide the row; the weight is float32 over the row")
+    check(library().tw_gate_group_norm(dtype_id(out.dtype), _dev(y), ld_y, _dev(gate), ld_g, _dev(weight), _dev(out), ld_o, n,
+                                       int(parts), width // int(parts), float(eps), _stream()), "gate_group_norm")
     return out

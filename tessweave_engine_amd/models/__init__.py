@@ -4,3 +4,4 @@ from . import kanavik  # noqa: F401
 from . import dinutar  # noqa: F401
 from . import rufusun  # noqa: F401
 from . import tadalorn  # noqa: F401
+from . import darolix  # noqa: F401

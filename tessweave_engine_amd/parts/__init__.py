@@ -6,7 +6,7 @@ from .positions import NoPositionEncoding, RotaryEmbedding
 from .attention import GroupedQueryAttention
 from .feedforward import GatedFeedForward, PlainFeedForward, ReluSquaredFeedForward, SwiGLU
 from .blocks import DepthMixedBlock, ParallelBlock, PostNormBlock, PreNormBlock, ResultNormBlock
-from .embedding import HashedPairEmbedding, OutputHead, PositionedEmbedding, TokenEmbedding
+from .embedding import HashedPairEmbedding, OutputHead, PositionedEmbedding, SinusoidalEmbedding, TokenEmbedding
 from .convolution import CausalConv
 from .parallel import GatedLinearRecurrence, MixedHeadAttention, MixerBranch, ParallelMixer
 from .side_input import SideTable, TokenSideInput
@@ -15,6 +15,8 @@ from .retention import Retention
 from .delta import GatedDeltaRule
 from .experts import RoutedExperts
 from .mlstm import MatrixLSTM
+from .linear_state import GatedLinearAttention, StateSpace
+from .normed_attention import NormedAttention
 from .windowed import ConvolvedWindowAttention
 from .model import DecoderModel, walk
 
@@ -25,5 +27,6 @@ __all__ = ["Block", "FeedForward", "GroupStep", "HeadHook", "LayerRun", "Mixer",
            "GatedLinearRecurrence", "MixedHeadAttention", "MixerBranch", "ParallelMixer", "SideTable", "TokenSideInput",
            "HashedPairEmbedding", "LatentAttention", "PostNormBlock", "ReluSquaredFeedForward", "Retention",
            "GatedDeltaRule", "ParallelBlock", "RoutedExperts",
+           "GatedLinearAttention", "NormedAttention", "SinusoidalEmbedding", "StateSpace",
            "ConvolvedWindowAttention", "MatrixLSTM", "PlainFeedForward", "ResultNormBlock",
            "DecoderModel", "walk"]

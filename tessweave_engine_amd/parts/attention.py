@@ -17,6 +17,43 @@ from .linear import Linear
 import torch
 
 
+def paged_attention(ctx, q, keys, values, group, out, q_heads, kv_heads, head_dim, scale, window=0, softcap=0.0):
+    """A step's causal attention over a cache group's pages: one-token sequences through the split-KV decode kernel, prompt
+    portions through the prefill kernel. q [n, >= q_heads * head_dim], out [n, q_heads * head_dim]; keys and values as
+    `ctx.cache.keys_values` gives them."""
+    n = ctx.n_tokens
+    if ctx.n_decode:
+        # A captured step is replayed for other lengths: its split count follows the step's length
+        # class (the kernel itself cuts each sequence's own keys into that many ranges).
+        longest = ctx.kv_bound if ctx.capturing else ctx.max_kv_len
+        if window:
+            longest = min(longest, window)
+        splits = ops.attn_decode_splits(ctx.n_decode, q_heads, kv_heads, longest)
+        ws = None
+        if splits > 1:
+            # sized for the most splits any length class can ask for, so that it never grows under a capture
+            most = max(splits, ops.attn_decode_splits(ctx.n_decode, q_heads, kv_heads,
+                                                      min(ctx.kv_capacity, window) if window else ctx.kv_capacity))
+            floats = ops.attn_decode_workspace_floats(ctx.n_decode, q_heads, head_dim, most)
+            ws = ctx.workspace.get("attn.split", (floats,), torch.float32)
+        ops.attn_decode(q, keys, values, group.block_table, ctx.q_start, ctx.kv_len, 0, ctx.n_decode, out,
+                        q_heads, kv_heads, head_dim, scale, window=window,
+                        splits=splits, workspace=ws, softcap=softcap)
+    if ctx.n_seqs > ctx.n_decode:
+        # long key ranges are cut into chunks for separate workgroups when there are few tiles of rows
+        longest = min(ctx.max_kv_len, window + ctx.max_q_len) if window else ctx.max_kv_len
+        split = ops.attn_prefill_split(ctx.n_seqs - ctx.n_decode, q_heads, kv_heads, ctx.max_q_len, longest)
+        ws = None
+        if split[0] > 1:
+            ws = ctx.workspace.get("attn.prefill_split", (ops.attn_prefill_workspace_floats(
+                n, q_heads, head_dim, split[0]),), torch.float32)
+        ops.attn_prefill(q, keys, values, group.block_table, ctx.q_start, ctx.kv_len, ctx.n_decode,
+                         ctx.n_seqs - ctx.n_decode, ctx.max_q_len, out, q_heads, kv_heads,
+                         head_dim, scale, window=window, split=split, workspace=ws,
+                         softcap=softcap)
+    return out
+
+
 class GroupedQueryAttention(Mixer):
     def __init__(self, prefix, hidden, q_heads, kv_heads, head_dim, position, qkv_bias=True,
                  o_bias=False, window=None, scale=None, packed=True, head_hook=None, softcap=None, value_dim=None,
@@ -98,36 +135,8 @@ class GroupedQueryAttention(Mixer):
             ops.rope_kv_write(qkv, cos, sin, group.slot_mapping, keys, values, self.q_heads, self.kv_heads,
                               self.head_dim, ctx.cache.page_size, write_cache=run.writes_cache, adjacent=adjacent)
         out = ctx.scratch("attn.out", (n, self.q_heads * self.head_dim))
-        window = self.window or 0
-        if ctx.n_decode:
-            # A captured step is replayed for other lengths: its split count follows the step's length
-            # class (the kernel itself cuts each sequence's own keys into that many ranges).
-            longest = ctx.kv_bound if ctx.capturing else ctx.max_kv_len
-            if window:
-                longest = min(longest, window)
-            splits = ops.attn_decode_splits(ctx.n_decode, self.q_heads, self.kv_heads, longest)
-            ws = None
-            if splits > 1:
-                # sized for the most splits any length class can ask for, so that it never grows under a capture
-                most = max(splits, ops.attn_decode_splits(ctx.n_decode, self.q_heads, self.kv_heads,
-                                                          min(ctx.kv_capacity, window) if window else ctx.kv_capacity))
-                floats = ops.attn_decode_workspace_floats(ctx.n_decode, self.q_heads, self.head_dim, most)
-                ws = ctx.workspace.get("attn.split", (floats,), torch.float32)
-            ops.attn_decode(qkv, keys, values, group.block_table, ctx.q_start, ctx.kv_len, 0, ctx.n_decode, out,
-                            self.q_heads, self.kv_heads, self.head_dim, self.scale, window=window,
-                            splits=splits, workspace=ws, softcap=self.softcap)
-        if ctx.n_seqs > ctx.n_decode:
-            # long key ranges are cut into chunks for separate workgroups when there are few tiles of rows
-            longest = min(ctx.max_kv_len, window + ctx.max_q_len) if window else ctx.max_kv_len
-            split = ops.attn_prefill_split(ctx.n_seqs - ctx.n_decode, self.q_heads, self.kv_heads, ctx.max_q_len, longest)
-            ws = None
-            if split[0] > 1:
-                ws = ctx.workspace.get("attn.prefill_split", (ops.attn_prefill_workspace_floats(
-                    n, self.q_heads, self.head_dim, split[0]),), torch.float32)
-            ops.attn_prefill(qkv, keys, values, group.block_table, ctx.q_start, ctx.kv_len, ctx.n_decode,
-                             ctx.n_seqs - ctx.n_decode, ctx.max_q_len, out, self.q_heads, self.kv_heads,
-                             self.head_dim, self.scale, window=window, split=split, workspace=ws,
-                             softcap=self.softcap)
+        paged_attention(ctx, qkv, keys, values, group, out, self.q_heads, self.kv_heads, self.head_dim, self.scale,
+                        window=self.window or 0, softcap=self.softcap)
         if ctx.defer_sums and not self.o.biases and self.o.deferrable(n):
             return self.o.forward_partials(ctx, out, "o")          # the next norm adds them into x
         self.o.forward(ctx, out, x, residual=x if accumulate else None)

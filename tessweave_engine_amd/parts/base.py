@@ -20,6 +20,10 @@ import torch
 #: rounded to the compute type (in float32 runs: the stream itself), for a sublayer that reads the stream as it is
 ROUNDED_STREAM = "stream.rounded"
 
+#: key of `StepContext.shared` under which an embedding that is asked to keeps its output (float32 [n, hidden]) for layer
+#: runs that add it to the stream again (`LayerRun.adds_embedding`)
+EMBEDDING_OUTPUT = "embedding.output"
+
 
 @dataclass(frozen=True)
 class LayerRun:
@@ -28,10 +32,12 @@ class LayerRun:
     block:        index into the model's blocks (an index may appear more than once)
     cache_slot:   which cache slot the block's mixer uses in this run
     writes_cache: False lets the mixer read a slot that another run wrote in this step
+    adds_embedding: the embedding's output is added to the stream before this run (the model's embedding must keep it)
     """
     block: int
     cache_slot: int
     writes_cache: bool = True
+    adds_embedding: bool = False
 
 
 class Part:
@@ -125,6 +131,10 @@ class Mixer(Part):
 
 
 class FeedForward(Part):
+    #: True if `forward` takes `more`: pending partial sums (see `Mixer.forward`) of a mixer beside it, which it adds into
+    #: X together with its own result
+    folds_beside = False
+
     def forward(self, ctx, h, x):
         """Add the feed-forward's output for normalised input H into X (float32, in place);
         returns None or pending partial sums as `Mixer.forward` does."""

@@ -51,10 +51,17 @@ class ParallelBlock(Block):
     mixer_norm, ffn_norm: `RMSNorm` parts (weights and eps; both norms are one kernel: the row is read and its
     statistic formed once). ffn / ffn_norm may be None: the layer then has only the mixer. Both sublayers add into
     the stream after both norms have read it. The sublayers' sums are complete when the block returns (a model of
-    such blocks is built with `defer_sums=False`)."""
+    such blocks is built with `defer_sums=False`).
 
-    def __init__(self, hidden, mixer_norm, mixer, ffn_norm=None, ffn=None):
-        if (ffn is None) != (ffn_norm is None):
+    shared_norm: there is one norm and both sublayers read its result: x <- x + (mixer(h) + ff(h)), h = norm1(x). The
+    norm takes sums the block before left pending, and the mixer may leave its own to the feed-forward that
+    `folds_beside`, or, without a feed-forward, to the next block's norm (`defer_sums` may stay on)."""
+
+    def __init__(self, hidden, mixer_norm, mixer, ffn_norm=None, ffn=None, shared_norm=False):
+        self.shared_norm = bool(shared_norm)
+        if self.shared_norm and ffn_norm is not None:
+            raise ValueError("sublayers that share a norm have no second one")
+        if not self.shared_norm and (ffn is None) != (ffn_norm is None):
             raise ValueError("a feed-forward and its norm come together")
         if ffn_norm is not None and ffn_norm.eps != mixer_norm.eps:
             raise ValueError("the two norms of a parallel block share their eps")
@@ -72,6 +79,17 @@ class ParallelBlock(Block):
             p.bind(tensors, dtype, device)
 
     def forward(self, ctx, run, x, pending=None):
+        if self.shared_norm:
+            h = normalise(self.mixer_norm, ctx, x, pending)
+            left = self.mixer.forward(ctx, run, h, x)
+            if self.ffn is None:
+                return left
+            if left is None:
+                return self.ffn.forward(ctx, h, x)
+            if self.ffn.folds_beside:
+                return self.ffn.forward(ctx, h, x, more=left)
+            fold_pending(x, left)
+            return self.ffn.forward(ctx, h, x)
         pending = fold_pending(x, pending)
         n = ctx.n_tokens
         h1 = ctx.scratch("norm.out", (n, self.hidden))

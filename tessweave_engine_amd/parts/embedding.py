@@ -12,7 +12,7 @@ import torch
 from ..cache.spec import CacheNeed, FixedState
 from ..kernels import ops
 from ..weights.spec import MATRIX, NORMAL, TensorSpec
-from .base import ROUNDED_STREAM, Part
+from .base import EMBEDDING_OUTPUT, ROUNDED_STREAM, Part
 
 
 class TokenEmbedding(Part):
@@ -59,6 +59,38 @@ class PositionedEmbedding(TokenEmbedding):
             tag, leading = self.keep
             copy = ctx.workspace.get(tag, (leading, ctx.max_tokens, self.hidden), torch.float32)[0, :ctx.n_tokens]
         return ops.add_table_rows(x, self.positions, ctx.positions[0], copy=copy)
+
+
+class SinusoidalEmbedding(TokenEmbedding):
+    """Token embedding times a scale, plus fixed sinusoids of the position (Vaswani et al., "Attention Is All You Need"):
+
+        x = scale * table[token] + s(p),   s(p)[2 i] = sin(p * base^(-2 i / hidden)),  s(p)[2 i + 1] the cosine
+
+    Nothing bounds a position. keep: the sum is also left under `ctx.shared[EMBEDDING_OUTPUT]`, for layer runs that
+    add it to the stream again."""
+
+    def __init__(self, name, vocab, hidden, scale=1.0, base=10000.0, suffix=".weight", keep=False):
+        super().__init__(name, vocab, hidden, suffix)
+        self.scale, self.base, self.keep = float(scale), float(base), bool(keep)
+        self.freq = self.rest = None
+
+    def bind(self, tensors, dtype, device):
+        super().bind(tensors, dtype, device)
+        i = torch.arange((self.hidden + 1) // 2, dtype=torch.float64)
+        exact = self.base ** (-2.0 * i / self.hidden)
+        self.freq = exact.to(torch.float32)
+        self.rest = (exact - self.freq.to(torch.float64)).to(torch.float32).to(device)
+        self.freq = self.freq.to(device)
+
+    def forward(self, ctx):
+        n = ctx.n_tokens
+        x = ctx.scratch("residual", (n, self.hidden), torch.float32)
+        copy = ctx.scratch("embedding.output", (n, self.hidden), torch.float32) if self.keep else None
+        ops.embed_sinusoid(ctx.token_ids, self.weight, ctx.positions[0], self.freq, self.rest, self.scale, x, copy=copy,
+                           feed=ctx.token_feed)
+        if copy is not None:
+            ctx.shared[EMBEDDING_OUTPUT] = copy
+        return x
 
 
 class HashedPairEmbedding(TokenEmbedding):

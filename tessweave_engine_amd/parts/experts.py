@@ -9,6 +9,11 @@ A second kind (`kind="gelu"`, `weighting="softmax_chosen"`, `router_bias`): expe
 down(gelu(up y)) with the exact gelu; the router's logits take a bias; a token's weights are the softmax over its chosen
 logits alone and multiply the experts' OUTPUTS:  x += sum_e p_e expert_e(h)  (+ shared(h)).
 
+A third kind (`kind="silu"`, `weighting="softmax_all"`, `correction`, `identity`): gated experts, expert(y) =
+down(silu(gate y) * up y); s = softmax(z) over all experts, the `top` largest of s + correction are chosen, a token's weights
+are its chosen s over their sum and multiply the OUTPUTS; the last `identity` experts of the router have no matrices and
+return h itself.
+
 Experts have no biases. The experts' matrices are stacked on the device ([experts, inner, width] and [experts, width,
 inner], the reduction sizes padded to multiples of 32 with zeros, in the order the matrix unit's fragments are read:
 `ops.moe_blocked`) and all experts of a step run in two grouped
@@ -20,32 +25,42 @@ import torch
 
 from ..kernels import ops
 from ..weights.spec import MATRIX, NORMAL, VECTOR, TensorSpec
-from .base import FeedForward
+from .base import FeedForward, fold_pending
 
 
 class RoutedExperts(FeedForward):
+    folds_beside = True
+
     def __init__(self, prefix, hidden, experts, top, intermediate, limit=None, shared=None, router_name="router",
-                 expert_names=None, kind="swish_limited", weighting="sigmoid", router_bias=None):
+                 expert_names=None, kind="swish_limited", weighting="sigmoid", router_bias=None, identity=0, correction=None):
         """shared: a `FeedForward` part that every token runs as well (or None). expert_names: the checkpoint's
         names, behind the prefix, of expert number {}'s matrices (gate, up, down; up, down for kind "gelu").
-        kind: "swish_limited" (gated, needs `limit`, weights on the experts' inputs) or "gelu" (no gate, weights on the
-        outputs); weighting: "sigmoid" of each chosen logit or "softmax_chosen"; router_bias: the checkpoint's name,
-        behind the prefix, of a bias on the router's logits (or None)."""
+        kind: "swish_limited" (gated, needs `limit`, weights on the experts' inputs), "gelu" (no gate, weights on the
+        outputs) or "silu" (gated, weights on the outputs); weighting: "sigmoid" of each chosen logit, "softmax_chosen" or
+        "softmax_all"; router_bias: the checkpoint's name, behind the prefix, of a bias on the router's logits (or None);
+        correction: the name of what is added to the scores of "softmax_all" for the choice alone (or None);
+        identity: experts behind the others that return their input (kinds whose weights multiply outputs)."""
         self.prefix, self.hidden, self.experts, self.top = prefix, int(hidden), int(experts), int(top)
         self.intermediate, self.shared = int(intermediate), shared
         if kind not in ops.MOE_KINDS or weighting not in ops.MOE_WEIGHTS:
-            raise ValueError("experts are 'swish_limited' or 'gelu', their weights 'sigmoid' or 'softmax_chosen'")
-        self.kind, self.weighting = kind, weighting
-        self.gated = kind == "swish_limited"
+            raise ValueError(f"experts are one of {sorted(ops.MOE_KINDS)}, their weights one of {sorted(ops.MOE_WEIGHTS)}")
+        self.kind, self.weighting, self.identity = kind, weighting, int(identity)
+        self.gated = kind != "gelu"
+        self.choices = self.experts + self.identity          # what the router scores
+        if self.identity < 0 or (self.identity and kind == "swish_limited"):
+            raise ValueError("identity experts go with weights on the experts' outputs")
+        if correction and (weighting != "softmax_all" or router_bias):
+            raise ValueError("a correction belongs to 'softmax_all' (and takes the place of a bias)")
         self.limit = float(limit) if limit is not None else 0.0
-        if not 0 < self.top <= self.experts <= ops.MOE_MAX_EXPERTS:
+        if not (0 < self.top <= self.choices <= ops.MOE_MAX_EXPERTS and self.experts > 0):
             raise ValueError(f"1 to {ops.MOE_MAX_EXPERTS} experts, of which `top` are chosen")
-        if self.gated and not self.limit > 0:
+        if kind == "swish_limited" and not self.limit > 0:
             raise ValueError("the experts' limit must be positive")
         if expert_names is None:
             expert_names = ("e{}.gate", "e{}.up", "e{}.down") if self.gated else ("e{}.up", "e{}.down")
         self.router_name, self.expert_names = router_name, tuple(expert_names)
-        self.router_bias_name = prefix + router_bias if router_bias else None
+        extra = router_bias or correction                    # (one tensor either way: see `ops.moe_route`)
+        self.router_bias_name = prefix + extra if extra else None
         self.router = self.router_bias = self.gate = self.up = self.down = None
 
     def parts(self):
@@ -56,9 +71,9 @@ class RoutedExperts(FeedForward):
 
     def tensor_specs(self):
         C, F = self.hidden, self.intermediate
-        specs = [TensorSpec(self.prefix + self.router_name, (self.experts, C), VECTOR, NORMAL)]
+        specs = [TensorSpec(self.prefix + self.router_name, (self.choices, C), VECTOR, NORMAL)]
         if self.router_bias_name:
-            specs.append(TensorSpec(self.router_bias_name, (self.experts,), VECTOR, NORMAL))
+            specs.append(TensorSpec(self.router_bias_name, (self.choices,), VECTOR, NORMAL))
         for e in range(self.experts):
             *ins, down = self._names(e)
             specs += [TensorSpec(name, (F, C), MATRIX, NORMAL) for name in ins] + [TensorSpec(down, (C, F), MATRIX, NORMAL)]
@@ -91,12 +106,17 @@ class RoutedExperts(FeedForward):
         """Bytes of one expert's three matrices on the device."""
         return sum(t[0].numel() * t.element_size() for t in (self.gate, self.up, self.down) if t is not None)
 
-    def forward(self, ctx, h, x, accumulate=True):
+    def forward(self, ctx, h, x, accumulate=True, more=None):
         n = h.shape[0]
         # (with accumulate=False the shared expert writes x and the routed ones add to it, or it leaves the split-K sums of
         # its last product pending and the kernel that adds up a token's experts adds those too)
         pending = self.shared.forward(ctx, h, x, accumulate=accumulate) if self.shared is not None else None
         wrote = self.shared is not None and pending is None
+        if more is not None:                                 # a mixer's sums, added up by the kernel that adds up the experts
+            if pending is None:
+                pending = more
+            else:
+                fold_pending(x, more)                        # (a shared expert left sums of its own: plain operations)
         ids = ctx.scratch("moe.ids", (n, self.top), torch.int32)
         weights = ctx.scratch("moe.weights", (n, self.top), torch.float32)
         ops.moe_route(h, self.router, self.top, ids, weights, bias=self.router_bias, weighting=self.weighting)

@@ -4,7 +4,8 @@ from __future__ import annotations
 import torch
 
 from ..cache.spec import CacheLayout
-from .base import LayerRun, Norm, Part, PositionEncoding
+from ..kernels import ops
+from .base import EMBEDDING_OUTPUT, LayerRun, Norm, Part, PositionEncoding
 from .blocks import normalise
 
 
@@ -118,6 +119,12 @@ class DecoderModel(Part):
         x = self.embedding.forward(ctx)
         pending = None              # partial sums a block left for the next norm to add into x
         for i, run in enumerate(self.schedule):
+            if run.adds_embedding:
+                first = ctx.shared[EMBEDDING_OUTPUT]
+                if pending is None:
+                    pending = first.unsqueeze(0)          # the run's first norm adds it, like any pending sum
+                else:
+                    ops.add_values(x, first)
             pending = self.blocks[run.block].forward(ctx, run, x, pending)
             if ctx.segment_end is not None:
                 ctx.segment_end(i)

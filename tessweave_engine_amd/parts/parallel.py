@@ -3,7 +3,9 @@
 `ParallelMixer` reads h once: the input matrices of all its branches are one packed product, each branch
 works on its own columns of the result, writes its output (times its weight in the sum, times the
 block's residual multiplier) into its own columns of one buffer, and ONE joined output product adds
-sum_b scale_b * W_o,b out_b into the residual stream.
+sum_b scale_b * W_o,b out_b into the residual stream. With a norm on each branch's RESULT
+(`result_norms`) every branch has an output product of its own and one kernel adds
+sum_b scale_b * norm_b(W_o,b out_b).
 
 `MixedHeadAttention`: grouped-query attention over the paged cache without rotation, whose scores lose
 slope_h * distance, are mixed across heads by a learned [H, H] matrix before the softmax, see a sliding
@@ -229,9 +231,11 @@ class GatedLinearRecurrence(MixerBranch):
 
 
 class ParallelMixer(Mixer):
-    def __init__(self, hidden, branches, scales, out_scale=1.0, suffix=""):
+    def __init__(self, hidden, branches, scales, out_scale=1.0, suffix="", result_norms=None, proj_dtype=None):
         """branches: `MixerBranch`es reading the same input; scales: each one's weight in the sum;
-        out_scale multiplies the whole sum (a block's residual multiplier)."""
+        out_scale multiplies the whole sum (a block's residual multiplier); result_norms: an `RMSNorm` part per branch
+        (of one eps) that its result passes before it is weighed and summed, or None; proj_dtype: the type of the packed
+        product's rows (None: the compute type; torch.float32 for branches that norm or accumulate them in 32-bit)."""
         if len(branches) != len(scales) or not branches:
             raise ValueError("one scale per branch is needed")
         self.hidden, self.branches = int(hidden), list(branches)
@@ -240,8 +244,16 @@ class ParallelMixer(Mixer):
         self.proj = Linear([m[0] for m in ins], hidden, [m[1] for m in ins], bias=[m[2] for m in ins],
                            pad_out=[m[3] for m in ins], suffixes=(suffix, ".b"))
         outs = [b.out_matrix() for b in self.branches]
-        self.out = JoinedLinear([o[0] for o in outs], [o[1] for o in outs], hidden, pad_ins=[o[2] for o in outs],
-                                suffix=suffix)
+        self.proj_dtype = proj_dtype
+        self.result_norms = list(result_norms) if result_norms else None
+        if self.result_norms:
+            if len(self.result_norms) != len(self.branches) or len({n.eps for n in self.result_norms}) != 1:
+                raise ValueError("one result norm per branch is needed, all of one eps")
+            self.outs = [Linear([name], columns, [hidden], pad_in=pad, suffixes=(suffix, ".b")) for name, columns, pad in outs]
+        else:
+            self.outs = []
+            self.out = JoinedLinear([o[0] for o in outs], [o[1] for o in outs], hidden, pad_ins=[o[2] for o in outs],
+                                    suffix=suffix)
         widths, at = self.proj.device_out, 0
         self.in_columns = []
         for b in self.branches:
@@ -249,21 +261,19 @@ class ParallelMixer(Mixer):
             self.in_columns.append((sum(widths[:at]), sum(widths[at:at + k])))
             at += k
         self.out_columns, col = [], 0
-        for w in self.out.device_in_parts:
+        for w in [] if self.result_norms else self.out.device_in_parts:
             self.out_columns.append((col, w))
             col += w
 
     def parts(self):
-        return [self.proj, self.out, *self.branches]
+        return [self.proj, *(self.outs + self.result_norms if self.result_norms else [self.out]), *self.branches]
 
     def tensor_specs(self):
-        return self.proj.tensor_specs() + self.out.tensor_specs() + [s for b in self.branches for s in b.tensor_specs()]
+        return [s for p in self.parts() for s in p.tensor_specs()]
 
     def bind(self, tensors, dtype, device):
-        self.proj.bind(tensors, dtype, device)
-        self.out.bind(tensors, dtype, device)
-        for b in self.branches:
-            b.bind(tensors, dtype, device)
+        for p in self.parts():
+            p.bind(tensors, dtype, device)
 
     def cache_need(self):
         need = CacheNeed()
@@ -273,8 +283,21 @@ class ParallelMixer(Mixer):
 
     def forward(self, ctx, run, h, x):
         n = ctx.n_tokens
-        proj = ctx.scratch("parallel.proj", (n, sum(self.proj.device_out)))
+        proj = ctx.scratch("parallel.proj", (n, sum(self.proj.device_out)), self.proj_dtype)
         self.proj.forward(ctx, h, proj)
+        if self.result_norms:
+            results = []
+            for i, (b, out, norm) in enumerate(zip(self.branches, self.outs, self.result_norms)):
+                c0, w = self.in_columns[i]
+                branch = ctx.scratch(f"parallel.out.{i}", (n, out.device_in))
+                b.forward(ctx, run, proj[:, c0:c0 + w], branch, 1.0)
+                if out.deferrable(n):
+                    y = out.forward_partials(ctx, branch, f"parallel.{i}")          # added up by the norm
+                else:
+                    y = out.forward(ctx, branch, ctx.scratch(f"parallel.result.{i}", (n, self.hidden), torch.float32))
+                results.append((y, norm.weight, self.scales[i]))
+            ops.add_normed_sum(x, results, self.result_norms[0].eps)
+            return None
         joined = ctx.scratch("parallel.out", (n, self.out.device_in))
         for b, (c0, w), (o0, ow), scale in zip(self.branches, self.in_columns, self.out_columns, self.scales):
             b.forward(ctx, run, proj[:, c0:c0 + w], joined[:, o0:o0 + ow], scale)

@@ -138,12 +138,27 @@ def read_tensors(folder, specs, compute_dtype, device):
     return tensors
 
 
+def tensor_shapes(folder):
+    """{name: shape} of every tensor of FOLDER's checkpoint, from the files' headers."""
+    from safetensors import safe_open
+
+    folder, shapes = Path(folder), {}
+    for name in shard_names(folder):
+        if not (folder / name).exists():
+            raise WeightError(other=[f"shard {name} does not exist in {folder}"])
+        with safe_open(str(folder / name), framework="pt", device="cpu") as shard:
+            shapes.update({key: tuple(shard.get_slice(key).get_shape()) for key in shard.keys()})
+    return shapes
+
+
 def load_model(folder, dtype="bfloat16", device="cuda", **build_options):
     """Model of FOLDER (config.json picks the class) with its weights on DEVICE."""
     from ..config import read_model_config, build_model
 
     folder = Path(folder).resolve(strict=True)
     config = read_model_config(folder)
+    if hasattr(config, "with_tensor_shapes"):          # sizes that config.json leaves to the tensors
+        config = config.with_tensor_shapes(tensor_shapes(folder))
     model = build_model(config, **build_options)
     compute_dtype = resolve_dtype(dtype)
     tensors = read_tensors(folder, model.tensor_specs(), compute_dtype, device)
