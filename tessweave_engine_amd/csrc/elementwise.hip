@@ -54,7 +54,9 @@ __global__ void embed_sinusoid_kernel(const int* __restrict__ ids, const T* __re
     const float off = __fmaf_rn(p, rest[i], __fmaf_rn(p, f, -angle));     // what the product lost
     float s, c;
     sincosf(angle, &s, &c);
-    const float sine = __fmaf_rn(off, c, s), cosine = __fmaf_rn(-off, s, c);
+    const float off2 = off * off;                                         // (sin and cos of a few hundredths at most)
+    const float so = off * __fmaf_rn(-off2, 1.f / 6.f, 1.f), co = -0.5f * off2;
+    const float sine = __fmaf_rn(so, c, __fmaf_rn(co, s, s)), cosine = __fmaf_rn(-so, s, __fmaf_rn(co, c, c));
     const size_t at = (size_t)n * hidden + 2 * i;
     const float a = __fmaf_rn(tw_to_float(row[2 * i]), scale, sine);
     out[at] = a;
