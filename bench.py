@@ -19,7 +19,7 @@ as the weights; `prefill_32k_prompts`: tokens a second over those prompts, which
 go through in portions of 2,048); and 1,024-token prompts with 512 generated tokens at batch 1, 8 and 64
 (`gen512_b*`, decoded tokens a second over the generated part).
 
-Other sizes of the architecture: --shape 14b|32b. --design kanavik|dinutar|rufusun|tadalorn measures that
+Other sizes of the architecture: --shape 14b|32b. --design kanavik|dinutar|rufusun|tadalorn|darolix measures that
 design's prefill and decode at a few layer sizes, each beside the Qwen2 decoder at equal
 width, heads, feed-forward and depth (one JSON line a size). --serve measures continuous
 batching under Poisson arrivals instead (prompts of 128..4,096 tokens, 256
@@ -89,7 +89,7 @@ def parse():
                    help="with --serve: the largest prompt portion in one step (larger: more prompt tokens a second and "
                         "a shorter time to the first token, longer steps for the requests that are decoding)")
     p.add_argument("--rate", type=float, default=16.0, help="mean arrivals a second (0: all at once)")
-    p.add_argument("--design", default="", choices=["", "kanavik", "dinutar", "rufusun", "tadalorn"],
+    p.add_argument("--design", default="", choices=["", "kanavik", "dinutar", "rufusun", "tadalorn", "darolix"],
                    help="instead: prefill and decode throughput of another design at a few layer sizes (--design-sizes), "
                         "each beside the Qwen2 decoder at equal width, heads, feed-forward and depth; one JSON line a size")
     p.add_argument("--design-sizes", default="1b,3b,7b", help="which of the design's sizes to run, comma separated")
@@ -195,6 +195,24 @@ def tadalorn_config(size, layers, context):
             "logit_softcap": 30.0, "layers": out}
 
 
+# The Darolix design at those widths: layers in the order state space, side by side. State space: twice the width in heads of
+# 64, eight groups with states of 128, convolutions of four taps. Side by side: attention with the size's heads and key heads
+# (a soft cap of 30, a temperature), gated linear attention with the size's heads, keys of half the head size and values of
+# the head size. Every layer has routed experts (16 of a quarter of the dense inner size beside four identities, two a
+# token; the Rufusun run beside it has as many experts of that size, and a shared one, in every second layer).
+def darolix_config(size, layers, context):
+    width, heads, kv_heads, dim, ff, _ = DESIGN_SIZES[size]
+    mlp = {"kind": "moe", "router": {"experts": 16, "identity": 4, "top": 2}, "expert": {"ff": ff // 4}}
+    space = {"heads": 2 * width // 64, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8}
+    beside = {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "softcap": 30.0,
+                       "q_temp": {"coef": 0.1, "every": 1024}},
+              "right": {"heads": heads, "dim": dim // 2, "vdim": dim, "tau": 16.0}}
+    out = [{"type": "parallel", "mixer": beside, "mlp": mlp} if i % 2 else {"type": "mamba2", "mixer": space, "mlp": mlp}
+           for i in range(layers)]
+    return {"architecture": "Darolix", "vocab": DESIGN_VOCAB, "width": width, "norm": {"eps": 1e-6},
+            "embedding": {"scale": width ** 0.5}, "layers": out}
+
+
 def qwen2_config_like(size, layers, context):
     width, heads, kv_heads, dim, ff, _ = DESIGN_SIZES[size]
     return dict(QWEN25_7B, num_hidden_layers=layers, hidden_size=width, num_attention_heads=heads,
@@ -216,10 +234,10 @@ def design_run(args, torch):
                 "batch": args.batch, "context": args.context, "prefill_tokens": args.prefill_tokens,
                 "data": "synthetic: uniform-random token ids, random weights"}
         make = {"kanavik": kanavik_config, "dinutar": dinutar_config, "rufusun": rufusun_config,
-                "tadalorn": tadalorn_config}[args.design]
+                "tadalorn": tadalorn_config, "darolix": darolix_config}[args.design]
         models = [(args.design, make(size, args.design_layers, args.context))]
         if not args.design_only:
-            if args.design == "tadalorn":          # the closest design of the engine (experts, a recurrence, attention)
+            if args.design in ("tadalorn", "darolix"):          # the closest design of the engine (experts, a recurrence, attention)
                 models.append(("rufusun", rufusun_config(size, args.design_layers, args.context)))
             models.append(("qwen2", qwen2_config_like(size, args.design_layers, args.context)))
         for name, cfg in models:

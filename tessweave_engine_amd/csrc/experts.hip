@@ -15,7 +15,7 @@
 //   p = s of the chosen over their sum (+ 1e-20)        expert(y): down( silu(gate y) * up y ); the last `identity`
 //   out = sum over the chosen experts e of  p_e * expert_e(h)          experts return h itself
 //
-// A step runs in six launches whose shapes depend only on the number of rows: route; plan (every expert's rows are
+// A step runs in six launches (four where there are few pairs: see PLAN below) whose shapes depend only on the number of rows: route; plan (every expert's rows are
 // laid out one expert after the other, each expert's share padded to whole tiles of 16 rows; which expert a tile
 // belongs to is a table on the device, tiles nobody uses say -1); gather (the scaled, rounded input rows in that
 // order); two grouped products on the matrix unit, one workgroup a (tile, range of columns), whose weights are the
@@ -36,52 +36,73 @@
 #define TW_MOE_SPLITK_TILES 64        /* up to this many tiles a step, the waves of a workgroup split K */
 
 // ---- route ---------------------------------------------------------------------------------------------------
-template <typename T>
-__global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h, long ld_h, const float* __restrict__ router,
-                                                        const float* __restrict__ bias, int mode, int C, int X, int top,
-                                                        int* __restrict__ ids, float* __restrict__ weights) {
-  __shared__ float z[TW_MOE_MAX_EXPERTS];
-  __shared__ float score[TW_MOE_MAX_EXPERTS];       // mode 2: the softmax over all logits (z: what decides the choice)
-  const int row = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const T* x = h + (size_t)row * ld_h;
-  // A wave forms two experts' logits at a time, four elements a lane and load, eight loads in flight before the first
-  // is used: a logit is a chain of loads from memory, and their latency is all it costs.
+// Four consecutive elements of a row as floats.
+__device__ __forceinline__ f32x4 moe_four(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
+__device__ __forceinline__ f32x4 moe_four(const bf16_t* p) {
+  const bf16x4 v = *reinterpret_cast<const bf16x4*>(p);
+  return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
+}
+
+// A workgroup takes R rows: a wave forms two experts' logits for all of them at a time, four elements a lane and load,
+// several loads in flight before the first is used (a logit is a chain of loads from memory, and their latency is all it
+// costs: few rows get many waves each, many rows share a read of the router). Then a wave a row chooses.
+template <typename T, int R, int WAVES>
+__global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(const T* __restrict__ h, long ld_h, const float* __restrict__ router,
+                                                               const float* __restrict__ bias, int mode, int n, int C, int X,
+                                                               int top, int* __restrict__ ids, float* __restrict__ weights) {
+  __shared__ float z_s[R][TW_MOE_MAX_EXPERTS];
+  __shared__ float score_s[R][TW_MOE_MAX_EXPERTS];   // mode 2: the softmax over all logits (z: what decides the choice)
+  const int row0 = blockIdx.x * R, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const T* x[R];
+#pragma unroll
+  for (int r = 0; r < R; ++r) x[r] = h + (size_t)min(row0 + r, n - 1) * ld_h;
   const bool vec = C % 4 == 0 && ld_h % 4 == 0 && ((uintptr_t)h % 16 == 0) && ((uintptr_t)router % 16 == 0);
-  for (int e = 2 * wave; e < X; e += 8) {
+  for (int e = 2 * wave; e < X; e += 2 * WAVES) {
     const float* w0 = router + (size_t)e * C;
     const float* w1 = router + (size_t)min(e + 1, X - 1) * C;
-    float s0 = 0.f, s1 = 0.f;
+    float s0[R], s1[R];
+#pragma unroll
+    for (int r = 0; r < R; ++r) s0[r] = s1[r] = 0.f;
     if (vec) {
 #pragma unroll 4
       for (int c = 4 * lane; c < C; c += 256) {
         const f32x4 a = *reinterpret_cast<const f32x4*>(w0 + c);
         const f32x4 b = *reinterpret_cast<const f32x4*>(w1 + c);
-        float xv[4];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) xv[j] = tw_to_float(x[c + j]);
+        for (int r = 0; r < R; ++r) {
+          const f32x4 xv = moe_four(x[r] + c);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          s0 = __fmaf_rn(a[j], xv[j], s0);
-          s1 = __fmaf_rn(b[j], xv[j], s1);
+          for (int j = 0; j < 4; ++j) {
+            s0[r] = __fmaf_rn(a[j], xv[j], s0[r]);
+            s1[r] = __fmaf_rn(b[j], xv[j], s1[r]);
+          }
         }
       }
     } else {
       for (int c = lane; c < C; c += 64) {
-        const float xv = tw_to_float(x[c]);
-        s0 = __fmaf_rn(w0[c], xv, s0);
-        s1 = __fmaf_rn(w1[c], xv, s1);
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+          const float xv = tw_to_float(x[r][c]);
+          s0[r] = __fmaf_rn(w0[c], xv, s0[r]);
+          s1[r] = __fmaf_rn(w1[c], xv, s1[r]);
+        }
       }
     }
-    s0 = tw_wave_sum(s0);
-    s1 = tw_wave_sum(s1);
-    if (lane == 0) {
-      const bool biased = bias && mode != 2;
-      z[e] = s0 + (biased ? bias[e] : 0.f);
-      if (e + 1 < X) z[e + 1] = s1 + (biased ? bias[e + 1] : 0.f);
+    const bool biased = bias && mode != 2;
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const float t0 = tw_wave_sum(s0[r]), t1 = tw_wave_sum(s1[r]);
+      if (lane == 0) {
+        z_s[r][e] = t0 + (biased ? bias[e] : 0.f);
+        if (e + 1 < X) z_s[r][e + 1] = t1 + (biased ? bias[e + 1] : 0.f);
+      }
     }
   }
   __syncthreads();
-  if (wave != 0) return;
+  if (wave >= R || row0 + wave >= n) return;
+  const int row = row0 + wave;
+  float* z = z_s[wave];
+  float* score = score_s[wave];
   if (mode == 2) {
     float most = -INFINITY, sum = 0.f;
     for (int e = lane; e < X; e += 64) most = fmaxf(most, z[e]);
@@ -144,11 +165,16 @@ extern "C" int tw_moe_route(int dtype, const void* h, long ld_h, const float* ro
   TW_REQUIRE(h && router && ids && weights && n >= 0 && C > 0 && ld_h >= C && mode >= 0 && mode <= 2);
   TW_REQUIRE(X > 0 && X <= TW_MOE_MAX_EXPERTS && top > 0 && top <= X);
   if (n == 0) return 0;
-  if (dtype == TW_DTYPE_BF16)
-    moe_route_kernel<bf16_t><<<n, 256, 0, stream>>>((const bf16_t*)h, ld_h, router, bias, mode, C, X, top, ids, weights);
-  else if (dtype == TW_DTYPE_F32)
-    moe_route_kernel<float><<<n, 256, 0, stream>>>((const float*)h, ld_h, router, bias, mode, C, X, top, ids, weights);
+#define TW_MOE_ROUTE(T)                                                                                                 \
+  do {                                                                                                                  \
+    if (n <= 64) moe_route_kernel<T, 1, 16><<<n, 1024, 0, stream>>>((const T*)h, ld_h, router, bias, mode, n, C, X, top, ids, weights);                \
+    else if (n <= 512) moe_route_kernel<T, 1, 4><<<n, 256, 0, stream>>>((const T*)h, ld_h, router, bias, mode, n, C, X, top, ids, weights);            \
+    else moe_route_kernel<T, 4, 8><<<tw_div_up(n, 4), 512, 0, stream>>>((const T*)h, ld_h, router, bias, mode, n, C, X, top, ids, weights);            \
+  } while (0)
+  if (dtype == TW_DTYPE_BF16) TW_MOE_ROUTE(bf16_t);
+  else if (dtype == TW_DTYPE_F32) TW_MOE_ROUTE(float);
   else return TW_ERR_BAD_ARGUMENT;
+#undef TW_MOE_ROUTE
   return TW_LAUNCH_RESULT();
 }
 
@@ -240,17 +266,69 @@ __global__ __launch_bounds__(256) void moe_gather_kernel(const T* __restrict__ h
 template <int N> struct MoeCount { static constexpr int value = N; };
 // ACT 0: the float32 product; 1: gate and up with the limited swish; 2: one matrix with the exact gelu; 3: gate and up with
 // SiLU (1 to 3 write the next product's rows in the compute type).
-template <typename T, int ACT, int NT, bool SPLITK = false, int MT = 1>
+// PLAN (the first product of steps of at most 64 (token, choice) pairs whose weights multiply outputs): there is no plan
+// and no gather launch. Every wave finds the tiles itself, lane i holding pair i: a pair whose expert has 16 m pairs before
+// it opens a tile, the tiles are numbered in the order of the pairs that open them, and the rows are read where they lie in
+// h. The tile's first workgroup writes what the second product and the combination read: tile_expert, pos.
+struct MoePairs {
+  const int* ids;       // [items]
+  int items, top, X;
+  long ld_h;
+  int* tile_expert;
+  int* pos;
+};
+template <typename T, int ACT, int NT, bool SPLITK = false, int MT = 1, bool PLAN = false>
 __global__ __launch_bounds__(256) void moe_grouped_kernel(const T* __restrict__ A, long lda, const T* __restrict__ W,
                                                           const T* __restrict__ W2, const int* __restrict__ tile_expert,
-                                                          void* __restrict__ out, long ldo, int N, int K, float limit) {
+                                                          void* __restrict__ out, long ldo, int N, int K, float limit,
+                                                          MoePairs pairs = {}) {
   constexpr int EPF = Elem<T>::kPerFrag;
   constexpr bool GLU = ACT == 1 || ACT == 3;
   const int tile = blockIdx.x * MT;
-  const int ex = tile_expert[tile];
-  if (ex < 0) return;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int r = lane & 15, g = lane >> 4;
+  int ex, row_of_lane = 0;                           // PLAN: the row of h that lane's row r of the tile is
+  if constexpr (PLAN) {
+    const int mine = lane < pairs.items ? pairs.ids[lane] : -1;
+    const bool real = mine >= 0 && mine < pairs.X;
+    int before = 0;                                  // pairs of the same expert before this one
+    for (int i = 0; i < pairs.items; ++i) {
+      const int other = __builtin_amdgcn_readlane(mine, i);
+      before += (i < lane && other == mine) ? 1 : 0;
+    }
+    const unsigned long long opens = __ballot(real && before % TW_MOE_TILE == 0);
+    int opener = -1;                                 // the pair that opens this tile
+    {
+      unsigned long long left = opens;
+      for (int i = 0; i < tile && left; ++i) left &= left - 1;
+      if (left) opener = __ffsll((unsigned long long)left) - 1;
+    }
+    const bool leads = blockIdx.y == 0 && wave == 0;
+    if (leads && tile == 0 && lane < pairs.items && !real) pairs.pos[lane] = -1;
+    if (opener < 0) {
+      if (leads && lane == 0) pairs.tile_expert[tile] = -1;
+      return;
+    }
+    ex = __builtin_amdgcn_readlane(mine, opener);
+    const int from = __builtin_amdgcn_readlane(before, opener);
+    const bool here = real && mine == ex && before >= from && before < from + TW_MOE_TILE;
+    unsigned long long members = __ballot(here);
+    if (leads) {
+      if (lane == 0) pairs.tile_expert[tile] = ex;
+      if (here) pairs.pos[lane] = tile * TW_MOE_TILE + before - from;
+    }
+    // row j of the tile is its j-th member; rows behind the last repeat the first (nobody reads what they give)
+    int pair = opener;
+    for (int i = 0; i < TW_MOE_TILE && members; ++i) {
+      const int m = __ffsll((unsigned long long)members) - 1;
+      members &= members - 1;
+      if (i == r) pair = m;
+    }
+    row_of_lane = pair / pairs.top;
+  } else {
+    ex = tile_expert[tile];
+    if (ex < 0) return;
+  }
   const int col0 = (SPLITK ? blockIdx.y : blockIdx.y * 4 + wave) * 16 * NT;
   if (col0 >= N) return;
   constexpr int KSTEP = 4 * EPF;
@@ -259,7 +337,7 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(const T* __restrict__ 
   const int k_first = SPLITK ? wave * BLK : 0;
   const size_t tile_elems = (size_t)K * TW_MOE_TILE;  // all steps of one tile of 16 rows
   const int n_blocks = (N + 15) / 16;
-  const T* a_ptr = A + (size_t)tile * tile_elems + lane * EPF;
+  const T* a_ptr = PLAN ? A + (size_t)row_of_lane * pairs.ld_h + g * EPF : A + (size_t)tile * tile_elems + lane * EPF;
   const T* w_ptr[NT];
   const T* w2_ptr[NT];
 #pragma unroll
@@ -280,13 +358,16 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(const T* __restrict__ 
 #pragma unroll
     for (int u = 0; u < U; ++u) {
 #pragma unroll
-      for (int m = 0; m < MT; ++m) a[u][m] = tw_load_frag(a_ptr + (size_t)m * tile_elems + k + u * k_stride);
+      for (int m = 0; m < MT; ++m) a[u][m] = tw_load_frag(PLAN ? a_ptr + (k + u * k_stride) / TW_MOE_TILE
+                                                                          : a_ptr + (size_t)m * tile_elems + k + u * k_stride);
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
-        b[u][t] = tw_load_frag(w_ptr[t] + k + u * k_stride);
-        if (GLU) b2[u][t] = tw_load_frag(w2_ptr[t] + k + u * k_stride);
+        // (few rows: an expert's matrices are read once a step)
+        b[u][t] = SPLITK ? tw_load_frag_stream(w_ptr[t] + k + u * k_stride) : tw_load_frag(w_ptr[t] + k + u * k_stride);
+        if (GLU) b2[u][t] = SPLITK ? tw_load_frag_stream(w2_ptr[t] + k + u * k_stride) : tw_load_frag(w2_ptr[t] + k + u * k_stride);
       }
     }
+    __builtin_amdgcn_sched_barrier(0);               // (the scheduler would put each load in front of its use to save registers)
 #pragma unroll
     for (int u = 0; u < U; ++u)
 #pragma unroll
@@ -419,27 +500,50 @@ struct MoeStep {
   const void *h, *gate, *up, *down;
   long ld_h, ld_x;
   const float* weights;
-  const int *src_item, *tile_expert, *pos;
+  const int *ids, *src_item, *tile_expert, *pos;
   void *xs, *act;
   float *ys, *x;
   const float* more;
-  int n, top, C, Cd, Fd, capacity, kind, accumulate, more_splits;
+  int n, top, X, C, Cd, Fd, capacity, kind, accumulate, more_splits;
   float limit;
-  bool wide;
+  bool wide, few;
 };
+
+template <typename T, int ACT>
+static void moe_products_few(const MoeStep& s, hipStream_t stream) {
+  // (every tile is opened by a pair of its own, and the tiles in use never exceed what a plan could need)
+  const int tiles = s.n * s.top < s.capacity / TW_MOE_TILE ? s.n * s.top : s.capacity / TW_MOE_TILE;
+  const MoePairs pairs{s.ids, s.n * s.top, s.top, s.X, s.ld_h, const_cast<int*>(s.tile_expert), const_cast<int*>(s.pos)};
+  moe_grouped_kernel<T, ACT, 2, true, 1, true><<<dim3(tiles, tw_div_up(s.Fd, 16 * 2)), 256, 0, stream>>>(
+      (const T*)s.h, s.Cd, (const T*)(ACT == 2 ? s.up : s.gate), (const T*)(ACT == 2 ? nullptr : s.up), nullptr, s.act, s.Fd, s.Fd,
+      s.Cd, s.limit, pairs);
+  moe_grouped_kernel<T, 0, 2, true><<<dim3(tiles, tw_div_up(s.C, 16 * 2)), 256, 0, stream>>>(
+      (const T*)s.act, s.Fd, (const T*)s.down, nullptr, s.tile_expert, s.ys, s.C, s.C, s.Fd, 0.f);
+}
+
+// Can the first product find its tiles and rows itself? (few pairs, rows of h that are whole fragments)
+static bool moe_few(int dtype, const void* h, long ld_h, int n, int top, int C, int Cd, int kind) {
+  const int epf = dtype == TW_DTYPE_BF16 ? 8 : 4;
+  return kind != 0 && n * top <= 64 && C == Cd && C % (4 * epf) == 0 && ld_h % epf == 0 && (uintptr_t)h % 16 == 0;
+}
 
 template <typename T>
 static void moe_run(const MoeStep& s, hipStream_t stream) {
-  moe_gather_kernel<T><<<s.capacity, 256, 0, stream>>>((const T*)s.h, s.ld_h, s.kind == 0 ? s.weights : nullptr, s.src_item,
-                                                       s.tile_expert, (T*)s.xs, s.C, s.Cd, s.top);
-  const int tiles = s.capacity / TW_MOE_TILE;
+  if (s.few) {
+    if (s.kind == 1) moe_products_few<T, 2>(s, stream);
+    else moe_products_few<T, 3>(s, stream);
+  } else {
+    moe_gather_kernel<T><<<s.capacity, 256, 0, stream>>>((const T*)s.h, s.ld_h, s.kind == 0 ? s.weights : nullptr, s.src_item,
+                                                         s.tile_expert, (T*)s.xs, s.C, s.Cd, s.top);
+    const int tiles = s.capacity / TW_MOE_TILE;
 #define TW_MOE_PRODUCTS(ACT)                                                                                            \
-  moe_products<T, ACT>((const T*)s.xs, (const T*)s.gate, (const T*)s.up, (const T*)s.down, s.tile_expert, (T*)s.act,    \
-                       s.ys, s.C, s.Cd, s.Fd, s.limit, tiles, s.wide, stream)
-  if (s.kind == 0) TW_MOE_PRODUCTS(1);
-  else if (s.kind == 1) TW_MOE_PRODUCTS(2);
-  else TW_MOE_PRODUCTS(3);
+    moe_products<T, ACT>((const T*)s.xs, (const T*)s.gate, (const T*)s.up, (const T*)s.down, s.tile_expert, (T*)s.act,    \
+                         s.ys, s.C, s.Cd, s.Fd, s.limit, tiles, s.wide, stream)
+    if (s.kind == 0) TW_MOE_PRODUCTS(1);
+    else if (s.kind == 1) TW_MOE_PRODUCTS(2);
+    else TW_MOE_PRODUCTS(3);
 #undef TW_MOE_PRODUCTS
+  }
   const dim3 grid(s.n, tw_div_up(s.C, 1024));
   const size_t more_stride = (size_t)s.n * s.C;
   const float* weights = s.kind == 0 ? nullptr : s.weights;
@@ -468,12 +572,15 @@ extern "C" int tw_moe_experts(int dtype, const void* h, long ld_h, const int* id
              (uintptr_t)down % 16 == 0);
   TW_REQUIRE(dtype == TW_DTYPE_BF16 || dtype == TW_DTYPE_F32);
   if (n == 0) return 0;
-  const int code = tw_moe_plan(ids, n * top, X, pos, src_item, tile_expert, capacity, stream);
-  if (code) return code;
+  const bool few = moe_few(dtype, h, ld_h, n, top, C, Cd, kind);
+  if (!few) {
+    const int code = tw_moe_plan(ids, n * top, X, pos, src_item, tile_expert, capacity, stream);
+    if (code) return code;
+  }
   const bool wide = moe_unit((long)n * top, X) == TW_MOE_TILE * TW_MOE_WIDE;
   TW_REQUIRE(!wide || capacity % (TW_MOE_TILE * TW_MOE_WIDE) == 0);
-  const MoeStep s{h, gate, up, down, ld_h, ld_x, weights, src_item, tile_expert, pos, xs, act, ys, x, more,
-                  n, top, C, Cd, Fd, capacity, kind, accumulate, more_splits, limit, wide};
+  const MoeStep s{h, gate, up, down, ld_h, ld_x, weights, ids, src_item, tile_expert, pos, xs, act, ys, x, more,
+                  n, top, X, C, Cd, Fd, capacity, kind, accumulate, more_splits, limit, wide, few};
   if (dtype == TW_DTYPE_BF16) moe_run<bf16_t>(s, stream);
   else moe_run<float>(s, stream);
   return TW_LAUNCH_RESULT();

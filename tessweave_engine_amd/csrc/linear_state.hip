@@ -32,7 +32,9 @@
 struct LsArgs {
   const float* src; long ld;            // q of head h at q_col + h / share * D, k at k_col + h / share * D, v at v_col + h * E
   int q_col, k_col, v_col, share;
-  const float* logs; long ld_logs;      // channel: logarithm of head h's decay at h * D
+  const float* logs; long ld_logs;      // channel: logarithm of head h's decay at h * D, or (logs null, walked steps only)
+  const float* low; long ld_low; int rank;          // what tw_decay_logs forms it from: rows [n][rank],
+  const float* up; const float* up_bias; float tau; // up [rank][H D], its bias
   const float* raw; long ld_raw;        // head: the step size before its bias at raw_col + h
   int raw_col;
   const float* dt_bias; const float* A_log; const float* skip;   // [H]
@@ -51,6 +53,9 @@ struct LsSegments {
 };
 
 __device__ __forceinline__ float ls_softplus(float x) { return x > 20.f ? x : log1pf(expf(x)); }
+__device__ __forceinline__ float ls_log_decay(float x, float tau) {        // log sigmoid(x) / tau
+  return (x >= 0.f ? -log1pf(expf(-x)) : x - log1pf(expf(x))) / tau;
+}
 
 template <int CTRL>
 __device__ __forceinline__ float ls_turned(float v) {
@@ -120,7 +125,23 @@ __global__ __launch_bounds__(256) void ls_walk_kernel(LsArgs a) {
     const float* row = a.src + (size_t)t * a.ld;
     const float* q = row + a.q_col + (size_t)group * a.D;
     const float* k = row + a.k_col + (size_t)group * a.D;
-    f32x4 qv, kv, dv;
+    f32x4 qv, kv, dv, lv = {0.f, 0.f, 0.f, 0.f};
+    if (CHANNEL && !a.logs && held) {
+      const float* low = a.low + (size_t)t * a.ld_low;
+      const float* up = a.up + (size_t)head * a.D + d0;
+      const size_t stride = (size_t)a.H * a.D;
+      f32x4 z = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+      for (int r = 0; r < a.rank; ++r) {
+        const float l = low[r];
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (d0 + j < a.D) z[j] = __fmaf_rn(up[r * stride + j], l, z[j]);
+      }
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (d0 + j < a.D) lv[j] = ls_log_decay(z[j] + a.up_bias[(size_t)head * a.D + d0 + j], a.tau);
+    }
     float step = 1.f, decay = 1.f;
     if (!CHANNEL) {
       step = ls_softplus(a.raw[(size_t)t * a.ld_raw + a.raw_col + head] + bias);
@@ -131,7 +152,7 @@ __global__ __launch_bounds__(256) void ls_walk_kernel(LsArgs a) {
       const bool in = d0 + j < a.D;
       qv[j] = in ? q[d0 + j] * a.q_scale : 0.f;
       kv[j] = in ? k[d0 + j] * step : 0.f;
-      dv[j] = CHANNEL ? (in ? expf(a.logs[(size_t)t * a.ld_logs + (size_t)head * a.D + d0 + j]) : 1.f) : decay;
+      dv[j] = CHANNEL ? (in ? expf(a.logs ? a.logs[(size_t)t * a.ld_logs + (size_t)head * a.D + d0 + j] : lv[j]) : 1.f) : decay;
     }
     const float* v = row + a.v_col + (size_t)head * a.E;
 #pragma unroll
@@ -531,23 +552,25 @@ static int ls_launch(const LsArgs& a, const LsSegments& sg, int n_seqs, int walk
   return ls_chunk_launch<16, CHANNEL>(a, sg, n_seqs, stream);
 }
 
-// Sequences seq0 .. seq0 + n_seqs - 1. logs given: the channel form; else the head form (raw, dt_bias, A_log; skip or
-// null). walk != 0: token by token; else chunks, for portions of up to max_q_len tokens.
+// Sequences seq0 .. seq0 + n_seqs - 1. logs given, or, walked, what they are formed from (low, up, up_bias, tau): the
+// channel form; else the head form (raw, dt_bias, A_log; skip or null). walk != 0: token by token; else chunks, for portions of up to max_q_len tokens.
 extern "C" int tw_linear_state(const float* src, long ld, int q_col, int k_col, int v_col, int share, const float* logs,
-                               long ld_logs, const float* raw, long ld_raw, int raw_col, const float* dt_bias,
+                               long ld_logs, const float* low, long ld_low, int rank, const float* up,
+                               const float* up_bias, float tau, const float* raw, long ld_raw, int raw_col, const float* dt_bias,
                                const float* A_log, const float* skip, float* state, const int* q_start,
                                const int* state_slots, int seq0, int n_seqs, int max_q_len, float* out, long ld_out, int H,
                                int D, int E, float q_scale, int walk, float* workspace, long workspace_floats,
                                hipStream_t stream) {
-  TW_REQUIRE(src && state && q_start && state_slots && out && (logs || (raw && dt_bias && A_log)));
+  TW_REQUIRE(src && state && q_start && state_slots && out && (logs || low || (raw && dt_bias && A_log)));
+  TW_REQUIRE(!low || (walk && up && up_bias && rank > 0 && ld_low >= rank && tau > 0.f));
   TW_REQUIRE(seq0 >= 0 && n_seqs >= 0 && max_q_len >= 1 && H > 0 && D > 0 && D <= 256 && E > 0 && share > 0 && H % share == 0);
   TW_REQUIRE(q_col >= 0 && k_col >= 0 && v_col >= 0 && ld >= (long)max(q_col, k_col) + (long)(H / share) * D &&
              ld >= (long)v_col + (long)H * E && ld_out >= (long)H * E);
-  TW_REQUIRE(logs ? ld_logs >= (long)H * D : (raw_col >= 0 && ld_raw >= (long)raw_col + H));
+  TW_REQUIRE(logs ? ld_logs >= (long)H * D : low ? true : (raw_col >= 0 && ld_raw >= (long)raw_col + H));
   TW_REQUIRE((uintptr_t)state % 16 == 0 && n_seqs <= 65535 && H <= 65535);
   if (n_seqs == 0) return 0;
   const int Dp = (D + 15) / 16 * 16, Ep = (E + 15) / 16 * 16;
-  LsArgs a{src, ld, q_col, k_col, v_col, share, logs, ld_logs, raw, ld_raw, raw_col, dt_bias, A_log, skip, state, q_start,
+  LsArgs a{src, ld, q_col, k_col, v_col, share, logs, ld_logs, low, ld_low, rank, up, up_bias, tau, raw, ld_raw, raw_col, dt_bias, A_log, skip, state, q_start,
            state_slots, seq0, out, ld_out, H, D, E, Dp, Ep, q_scale};
   LsSegments sg{nullptr, nullptr, 0, 1};
   if (!walk) {
@@ -560,7 +583,7 @@ extern "C" int tw_linear_state(const float* src, long ld, int q_col, int k_col, 
     }
     TW_REQUIRE(sg.count <= 65535);
   }
-  return logs ? ls_launch<true>(a, sg, n_seqs, walk, stream) : ls_launch<false>(a, sg, n_seqs, walk, stream);
+  return logs || low ? ls_launch<true>(a, sg, n_seqs, walk, stream) : ls_launch<false>(a, sg, n_seqs, walk, stream);
 }
 
 // ---- the logarithms of a channel's decay --------------------------------------------------------------------------
@@ -583,6 +606,7 @@ __global__ __launch_bounds__(256) void ls_decay_kernel(const float* __restrict__
     for (int i = threadIdx.x; i < rows * rs; i += 256) low_s[i / rs][i % rs] = low[(size_t)(n0 + i / rs) * ld + r0 + i % rs];
     __syncthreads();
     if (c < channels) {
+#pragma unroll 8
       for (int rr = 0; rr < rs; ++rr) {
         const float w = up[(size_t)(r0 + rr) * channels + c];
 #pragma unroll
@@ -595,9 +619,7 @@ __global__ __launch_bounds__(256) void ls_decay_kernel(const float* __restrict__
 #pragma unroll
   for (int t = 0; t < LS_GATE_TOKENS; ++t) {
     if (t >= rows) break;
-    const float x = z[t] + b;
-    const float ls = x >= 0.f ? -log1pf(expf(-x)) : x - log1pf(expf(x));
-    out[(size_t)(n0 + t) * ld_out + c] = ls / tau;
+    out[(size_t)(n0 + t) * ld_out + c] = ls_log_decay(z[t] + b, tau);
   }
 }
 

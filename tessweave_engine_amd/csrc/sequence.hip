@@ -233,7 +233,11 @@ __global__ __launch_bounds__(256) void causal_conv_tile_kernel(ConvArgs a, int n
   __syncthreads();
   const int K = a.K, C = a.C;
   const SrcT* src = (const SrcT*)a.src;
-  for (int c = threadIdx.x * 4; c < C; c += blockDim.x * 4) {
+  for (int c = (blockIdx.y * blockDim.x + threadIdx.x) * 4; c < C; c += gridDim.y * blockDim.x * 4) {
+    f32x4 rows_in[TW_CONV_TILE];                          // the tile's own rows, all on their way at once
+#pragma unroll
+    for (int i = 0; i < TW_CONV_TILE; ++i)
+      rows_in[i] = i < rows ? conv_load4(src + (size_t)(row0 + i) * a.ld_src + c) : f32x4{0.f, 0.f, 0.f, 0.f};
     f32x4 w[TW_CONV_MAX_TAPS];                            // w[j][e]: tap j of channel c + e
 #pragma unroll
     for (int j = 0; j < TW_CONV_MAX_TAPS; ++j)
@@ -242,7 +246,9 @@ __global__ __launch_bounds__(256) void causal_conv_tile_kernel(ConvArgs a, int n
     const f32x4 bias = a.bias ? conv_load4(a.bias + c) : f32x4{0.f, 0.f, 0.f, 0.f};
     const f32x4 nw = NORM ? conv_load4(a.norm_w + c) : f32x4{1.f, 1.f, 1.f, 1.f};
     f32x4 v[TW_CONV_MAX_TAPS];                            // v[j]: the input that meets tap j; v[K - 1] the current row's
-    for (int i = 0; i < rows; ++i) {
+#pragma unroll
+    for (int i = 0; i < TW_CONV_TILE; ++i) {
+      if (i >= rows) break;
       const int row = row0 + i;
       const int first = info[i][0], start = info[i][1], len = info[i][2];
       const int pos = start + (row - first);
@@ -264,7 +270,7 @@ __global__ __launch_bounds__(256) void causal_conv_tile_kernel(ConvArgs a, int n
           }
         }
       }
-      f32x4 cur = conv_load4(src + (size_t)row * a.ld_src + c);
+      f32x4 cur = rows_in[i];
       if (NORM) cur = cur * a.row_rinv[row] * nw;
       f32x4 acc = bias + a.identity * cur;
 #pragma unroll
@@ -348,7 +354,7 @@ extern "C" int tw_causal_conv(int dtype, int src_f32, const void* src, long ld_s
   const bool tiled = vec && n_tokens >= 512 && (!norm_w || row_rinv);
 #define TW_CONV_LAUNCH(S, O, N)                                                                    \
   do {                                                                                             \
-    if (tiled) causal_conv_tile_kernel<S, O, N><<<tw_div_up(n_tokens, TW_CONV_TILE), 256, 0, stream>>>(a, n_tokens); \
+    if (tiled) causal_conv_tile_kernel<S, O, N><<<dim3(tw_div_up(n_tokens, TW_CONV_TILE), tw_div_up(C, 1024)), 256, 0, stream>>>(a, n_tokens); \
     else if (vec) causal_conv_kernel<S, O, N, true><<<n_blocks, 256, 0, stream>>>(a);              \
     else causal_conv_kernel<S, O, N, false><<<n_blocks, 256, 0, stream>>>(a);                      \
   } while (0)

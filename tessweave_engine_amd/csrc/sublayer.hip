@@ -356,7 +356,7 @@ extern "C" int tw_softcap_values(float* x, long total, float cap, hipStream_t st
 
 // ---- several results side by side, each normed, summed into the stream: x <- x + sum_b mult_b * w_b * unit(y_b) ----
 // Every y_b [n][hidden] is float32, or the split-K partial sums of a product that are added up here, in index order. A
-// block a row; a row of a result stays in registers between its two passes up to 4,096 elements.
+// block a row.
 #define TW_NORMED_SUM_MOST 4
 struct NormedSumArgs {
   float* x;
@@ -369,75 +369,88 @@ struct NormedSumArgs {
   float eps;
 };
 
-template <int W>
+// PER groups of four consecutive elements a thread, COUNT results: all rows are on their way before the first is used, and
+// their sums of squares meet in one reduction.
+template <int COUNT, int PER>
+__global__ __launch_bounds__(1024) void add_normed_sum_vec4_kernel(NormedSumArgs a) {
+  __shared__ float lds[COUNT][16];
+  const size_t row0 = (size_t)blockIdx.x * a.hidden;
+  const int chunks = a.hidden / 4;
+  f32x4 v[COUNT][PER];
+  float ss[COUNT];
+#pragma unroll
+  for (int b = 0; b < COUNT; ++b) {
+    ss[b] = 0.f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int c = threadIdx.x + i * blockDim.x;
+      v[b][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (c < chunks) {
+        const float* y = a.y[b] + row0 + 4 * c;
+#pragma unroll 8
+        for (int s = 0; s < a.splits[b]; ++s) v[b][i] += *reinterpret_cast<const f32x4*>(y + s * a.stride);
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss[b] = __fmaf_rn(v[b][i][e], v[b][i][e], ss[b]);
+    }
+  }
+  const int wave = threadIdx.x / TW_WAVE, waves = blockDim.x / TW_WAVE;
+#pragma unroll
+  for (int b = 0; b < COUNT; ++b) {
+    const float t = tw_wave_sum(ss[b]);
+    if (threadIdx.x % TW_WAVE == 0) lds[b][wave] = t;
+  }
+  __syncthreads();
+  float f[COUNT];
+#pragma unroll
+  for (int b = 0; b < COUNT; ++b) {
+    float t = 0.f;
+    for (int w = 0; w < waves; ++w) t += lds[b][w];
+    f[b] = a.mult[b] / sqrtf(t / (float)a.hidden + a.eps);
+  }
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = threadIdx.x + i * blockDim.x;
+    if (c < chunks) {
+      f32x4* x = reinterpret_cast<f32x4*>(a.x + row0 + 4 * c);
+      f32x4 sum = *x;
+#pragma unroll
+      for (int b = 0; b < COUNT; ++b)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) sum[e] = __fmaf_rn(v[b][i][e] * f[b], a.w[b][4 * c + e], sum[e]);
+      *x = sum;
+    }
+  }
+}
+
+// Any row length: every result is read twice.
 __global__ __launch_bounds__(256) void add_normed_sum_kernel(NormedSumArgs a) {
   __shared__ float lds[16];
-  constexpr int KEEP = 4;
-  const int units = a.hidden / W;
   const size_t row0 = (size_t)blockIdx.x * a.hidden;
-  float* x = a.x + row0;
-  float sum[KEEP][W];
-#pragma unroll
-  for (int i = 0; i < KEEP; ++i)
-#pragma unroll
-    for (int e = 0; e < W; ++e) sum[i][e] = 0.f;
   for (int b = 0; b < a.count; ++b) {
     const float* y = a.y[b] + row0;
-    const int splits = a.splits[b];
-    auto load = [&](int u, float* v) {
-#pragma unroll
-      for (int e = 0; e < W; ++e) v[e] = 0.f;
-      for (int s = 0; s < splits; ++s) {
-        if (W == 4) {
-          const f32x4 t = *reinterpret_cast<const f32x4*>(y + s * a.stride + (size_t)u * 4);
-#pragma unroll
-          for (int e = 0; e < W; ++e) v[e] += t[e];
-        } else {
-          v[0] += y[s * a.stride + u];
-        }
-      }
+    auto value = [&](int c) {
+      float v = 0.f;
+      for (int s = 0; s < a.splits[b]; ++s) v += y[s * a.stride + c];
+      return v;
     };
-    float kept[KEEP][W];
     float ss = 0.f;
-#pragma unroll
-    for (int i = 0; i < KEEP; ++i) {
-      const int u = threadIdx.x + i * 256;
-#pragma unroll
-      for (int e = 0; e < W; ++e) kept[i][e] = 0.f;
-      if (u < units) load(u, kept[i]);
-#pragma unroll
-      for (int e = 0; e < W; ++e) ss = __fmaf_rn(kept[i][e], kept[i][e], ss);
-    }
-    for (int u = threadIdx.x + KEEP * 256; u < units; u += 256) {
-      float v[W];
-      load(u, v);
-#pragma unroll
-      for (int e = 0; e < W; ++e) ss = __fmaf_rn(v[e], v[e], ss);
+    for (int c = threadIdx.x; c < a.hidden; c += 256) {
+      const float v = value(c);
+      ss = __fmaf_rn(v, v, ss);
     }
     const float f = a.mult[b] / sqrtf(tw_block_sum(ss, lds) / (float)a.hidden + a.eps);
-#pragma unroll
-    for (int i = 0; i < KEEP; ++i) {
-      const int u = threadIdx.x + i * 256;
-      if (u < units) {
-#pragma unroll
-        for (int e = 0; e < W; ++e) sum[i][e] = __fmaf_rn(kept[i][e] * f, a.w[b][u * W + e], sum[i][e]);
-      }
-    }
-    for (int u = threadIdx.x + KEEP * 256; u < units; u += 256) {       // (longer rows: one result after the other into x)
-      float v[W];
-      load(u, v);
-#pragma unroll
-      for (int e = 0; e < W; ++e) x[u * W + e] = __fmaf_rn(v[e] * f, a.w[b][u * W + e], x[u * W + e]);
-    }
+    for (int c = threadIdx.x; c < a.hidden; c += 256) a.x[row0 + c] = __fmaf_rn(value(c) * f, a.w[b][c], a.x[row0 + c]);
   }
-#pragma unroll
-  for (int i = 0; i < KEEP; ++i) {
-    const int u = threadIdx.x + i * 256;
-    if (u < units) {
-#pragma unroll
-      for (int e = 0; e < W; ++e) x[u * W + e] += sum[i][e];
-    }
-  }
+}
+
+template <int COUNT>
+static void add_normed_sum_launch(const NormedSumArgs& a, int n, hipStream_t stream) {
+  const int chunks = a.hidden / 4;
+  const int per = chunks <= 1024 ? 1 : 2;
+  const int threads = (tw_div_up(chunks, per) + 63) / 64 * 64;
+  if (per == 1) add_normed_sum_vec4_kernel<COUNT, 1><<<n, threads, 0, stream>>>(a);
+  else add_normed_sum_vec4_kernel<COUNT, 2><<<n, threads, 0, stream>>>(a);
 }
 
 extern "C" int tw_add_normed_sum(float* x, int count, const float* const* ys, const int* splits, const float* const* ws,
@@ -459,8 +472,14 @@ extern "C" int tw_add_normed_sum(float* x, int count, const float* const* ys, co
     vec = vec && (uintptr_t)ys[b] % 16 == 0;
   }
   if (n == 0) return 0;
-  if (vec) add_normed_sum_kernel<4><<<n, 256, 0, stream>>>(a);
-  else add_normed_sum_kernel<1><<<n, 256, 0, stream>>>(a);
+  if (vec && hidden <= 8192) {
+    if (count == 1) add_normed_sum_launch<1>(a, n, stream);
+    else if (count == 2) add_normed_sum_launch<2>(a, n, stream);
+    else if (count == 3) add_normed_sum_launch<3>(a, n, stream);
+    else add_normed_sum_launch<4>(a, n, stream);
+  } else {
+    add_normed_sum_kernel<<<n, 256, 0, stream>>>(a);
+  }
   return TW_LAUNCH_RESULT();
 }
 

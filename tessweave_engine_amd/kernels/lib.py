@@ -85,7 +85,7 @@ _SIGNATURES = {
                               ctypes.POINTER(c_float), I, I, F, P]),
     "tw_add_values": (I, [P, P, L, P]),
     "tw_linear_state_workspace_floats": (L, [I, I, I, I, I]),
-    "tw_linear_state": (I, [P, L, I, I, I, I, P, L, P, L, I, P, P, P, P, P, P, I, I, I, P, L, I, I, I, F, I, P, L, P]),
+    "tw_linear_state": (I, [P, L, I, I, I, I, P, L, P, L, I, P, P, F, P, L, I, P, P, P, P, P, P, I, I, I, P, L, I, I, I, F, I, P, L, P]),
     "tw_decay_logs": (I, [P, L, P, P, F, P, L, I, I, I, P]),
     "tw_gate_group_norm": (I, [I, P, L, P, L, P, P, L, I, I, I, F, P]),
     "tw_sampling_uniform": (F, [c_uint64, c_uint64]),

@@ -1433,14 +1433,14 @@ def linear_state_workspace_floats(n_seqs, max_q_len, heads, dim, value_dim):
 
 
 def linear_state(src, q_col, k_col, v_col, state, q_start, state_slots, seq0, n_seqs, out, heads, dim, value_dim, groups=None,
-                 q_scale=1.0, logs=None, raw=None, raw_col=0, dt_bias=None, A_log=None, skip=None, walk=True, max_q_len=1,
+                 q_scale=1.0, logs=None, low_rank=None, raw=None, raw_col=0, dt_bias=None, A_log=None, skip=None, walk=True, max_q_len=1,
                  workspace=None):
     """S <- d S + k v^T, o = S^T (q_scale q) per head over sequences seq0 .. seq0 + n_seqs - 1, from and to state float32
     [requests, heads, Ep, Dp] (dim and value_dim rounded up to 16; a column of S is contiguous).
 
     src float32 [n, .]: q and k of head h at q_col / k_col + (h // (heads / groups)) * dim (groups None: one per head), v at
-    v_col + h * value_dim. The decay d: logs float32 [n, >= heads * dim], its logarithm per key element; or, with logs None,
-    one number a head: delta = softplus(raw[n, raw_col + h] + dt_bias_h), d = exp(-exp(A_log_h) delta), the key then is
+    v_col + h * value_dim. The decay d: logs float32 [n, >= heads * dim], its logarithm per key element, or, walked, low_rank =
+    (low, up, bias, tau), what `decay_logs` forms it from (one launch less); with neither, one number a head: delta = softplus(raw[n, raw_col + h] + dt_bias_h), d = exp(-exp(A_log_h) delta), the key then is
     delta k, and skip_h v is added to the result. out float32 [n, heads * value_dim]. walk: token by token (steps of a few
     tokens a sequence), else chunks of 16 on the matrix unit for portions of up to max_q_len tokens, with a float32 workspace
     of `linear_state_workspace_floats` floats where that is not zero."""
@@ -1454,10 +1454,18 @@ def linear_state(src, q_col, k_col, v_col, state, q_start, state_slots, seq0, n_
           "linear_state: columns exceed the rows")
     _need(state.dtype == torch.float32 and state.is_contiguous() and state.dim() == 4 and tuple(state.shape[1:]) == (heads, Ep, Dp),
           "state must be float32 [requests, heads, Ep, Dp]")
-    ld_logs = ld_raw = 0
+    ld_logs = ld_raw = ld_low = rank = 0
+    low = up = up_bias = None
+    tau = 1.0
     if logs is not None:
         nl, wl, ld_logs = _rows(logs, "logs")
         _need(logs.dtype == torch.float32 and nl == n and wl >= heads * dim, "logs must be float32 [n, heads * dim]")
+    elif low_rank is not None:
+        low, up, up_bias, tau = low_rank
+        nl, rank, ld_low = _rows(low, "low")
+        _need(walk and low.dtype == up.dtype == up_bias.dtype == torch.float32 and nl == n and up.is_contiguous()
+              and tuple(up.shape) == (rank, heads * dim) and up_bias.is_contiguous() and up_bias.numel() == heads * dim and float(tau) > 0,
+              "low_rank (for walked steps): low [n, rank], up [rank, heads * dim], bias [heads * dim], all float32, tau positive")
     else:
         nr, wr, ld_raw = _rows(raw, "raw")
         _need(raw.dtype == torch.float32 and nr == n and 0 <= raw_col and raw_col + heads <= wr, "raw must be float32 rows with a column per head")
@@ -1468,9 +1476,11 @@ def linear_state(src, q_col, k_col, v_col, state, q_start, state_slots, seq0, n_
     if need:
         _need(workspace is not None and workspace.dtype == torch.float32 and workspace.is_contiguous() and workspace.numel() >= need,
               "long portions need a float32 workspace of linear_state_workspace_floats floats")
-    head = logs is None
+    head = logs is None and low is None
     check(library().tw_linear_state(_dev(src), ld, int(q_col), int(k_col), int(v_col), heads // groups,
-                                    None if head else _dev(logs), ld_logs, _dev(raw) if head else None, ld_raw, int(raw_col),
+                                    _dev(logs) if logs is not None else None, ld_logs, _dev(low) if low is not None else None, ld_low,
+                                    rank, _dev(up) if low is not None else None, _dev(up_bias) if low is not None else None,
+                                    float(tau), _dev(raw) if head else None, ld_raw, int(raw_col),
                                     _dev(dt_bias) if head else None, _dev(A_log) if head else None,
                                     _dev(skip) if head and skip is not None else None, _dev(state),
                                     _dev(q_start, torch.int32, "q_start"), _dev(state_slots, torch.int32, "state_slots"), int(seq0),

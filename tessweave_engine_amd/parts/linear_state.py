@@ -42,12 +42,17 @@ def state_need(heads, dim, value_dim):
     return FixedState((heads, _round_up(value_dim, 16), _round_up(dim, 16)), "float32")
 
 
+def all_walked(ctx):
+    """Does every sequence of the step bring so few tokens that it is walked?"""
+    return ctx.max_q_len <= ops.LINEAR_STATE_WALK_TOKENS
+
+
 def run_linear_state(ctx, src, state, out, heads, dim, value_dim, **options):
     """A step's sequences through the recurrence: few tokens a sequence walked, prompt portions in chunks."""
     common = (state, ctx.q_start, ctx.state_slots)
     columns = [options.pop(k) for k in ("q_col", "k_col", "v_col")]
     portions = ctx.n_seqs - ctx.n_decode
-    walked = ctx.n_seqs if ctx.max_q_len <= ops.LINEAR_STATE_WALK_TOKENS else ctx.n_decode
+    walked = ctx.n_seqs if all_walked(ctx) else ctx.n_decode
     if walked:
         ops.linear_state(src, *columns, *common, 0, walked, out, heads, dim, value_dim, walk=True, **options)
     if portions and walked < ctx.n_seqs:
@@ -172,9 +177,12 @@ class GatedLinearAttention(MixerBranch):
             raise ValueError("this branch's result is not scaled: give the mixer result norms")
         n, H, D, E = ctx.n_tokens, self.heads, self.dim, self.value_dim
         q, k, v, g, low = self.columns
-        logs = ctx.scratch("linear_attention.logs", (n, H * D), torch.float32)
-        ops.decay_logs(proj[:, low:low + self.rank], self.up, self.bias, self.tau, logs)
+        if all_walked(ctx):                                      # the walking kernel forms the decays itself
+            decays = dict(low_rank=(proj[:, low:low + self.rank], self.up, self.bias, self.tau))
+        else:
+            decays = dict(logs=ctx.scratch("linear_attention.logs", (n, H * D), torch.float32))
+            ops.decay_logs(proj[:, low:low + self.rank], self.up, self.bias, self.tau, decays["logs"])
         o = ctx.scratch("linear_attention.o", (n, H * E), torch.float32)
         run_linear_state(ctx, proj, ctx.cache.states[run.cache_slot][self.STATE], o, H, D, E, q_col=q, k_col=k, v_col=v,
-                         q_scale=D ** -0.5, logs=logs)
+                         q_scale=D ** -0.5, **decays)
         ops.head_norm_gate(o, proj[:, g:g + H * E], self.norm_weight, out, H, E, self.eps)
