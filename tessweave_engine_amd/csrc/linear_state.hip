@@ -44,6 +44,7 @@ struct LsArgs {
   float* out; long ld_out;              // [rows][H E]
   int H, D, E, Dp, Ep;
   float q_scale;
+  bool vec;                             // q and k of every head and row are whole 16-byte pieces
 };
 
 struct LsSegments {
@@ -94,9 +95,22 @@ __device__ __forceinline__ void ls_lds_barrier() {            // (loads from mem
   asm volatile("" ::: "memory");
 }
 
+// elements d0 .. d0 + 3 of a vector of D, zeros behind its end. vec: D is a multiple of 4 and the address of 16 bytes.
+__device__ __forceinline__ f32x4 ls_four(const float* p, int d0, int D, bool vec) {
+  f32x4 v = {0.f, 0.f, 0.f, 0.f};
+  if (vec) {
+    if (d0 < D) v = *reinterpret_cast<const f32x4*>(p + d0);
+  } else {
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (d0 + j < D) v[j] = p[d0 + j];
+  }
+  return v;
+}
+
 // ---- token by token -------------------------------------------------------------------------------------------------
 // grid (column blocks, H, n_seqs). LPC lanes hold a value column, four key elements each; a thread holds its elements of
-// CPT columns.
+// CPT columns. Decays given by their low-rank product: the workgroup's threads share out (key element, part of the rank).
 template <int LPC, int CPT, bool CHANNEL>
 __global__ __launch_bounds__(256) void ls_walk_kernel(LsArgs a) {
   constexpr int CW = 256 / LPC;                               // columns a pass
@@ -121,39 +135,45 @@ __global__ __launch_bounds__(256) void ls_walk_kernel(LsArgs a) {
     bias = a.dt_bias[head];
     skip = a.skip ? a.skip[head] : 0.f;
   }
+  constexpr int KM = 4 * LPC, PARTS = 256 / KM;               // key elements, threads that share one's product
+  __shared__ float part_s[CHANNEL ? PARTS : 1][KM];
+  __shared__ __attribute__((aligned(16))) float decay_s[KM];
   for (int t = r0; t < r1; ++t) {
     const float* row = a.src + (size_t)t * a.ld;
     const float* q = row + a.q_col + (size_t)group * a.D;
     const float* k = row + a.k_col + (size_t)group * a.D;
-    f32x4 qv, kv, dv, lv = {0.f, 0.f, 0.f, 0.f};
-    if (CHANNEL && !a.logs && held) {
-      const float* low = a.low + (size_t)t * a.ld_low;
-      const float* up = a.up + (size_t)head * a.D + d0;
-      const size_t stride = (size_t)a.H * a.D;
-      f32x4 z = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-      for (int r = 0; r < a.rank; ++r) {
-        const float l = low[r];
+    f32x4 qv = ls_four(q, d0, a.D, a.vec), kv = ls_four(k, d0, a.D, a.vec), dv;
+    if constexpr (CHANNEL) {
+      if (a.logs) {
+        dv = ls_four(a.logs + (size_t)t * a.ld_logs + (size_t)head * a.D, d0, a.D, false);
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
-          if (d0 + j < a.D) z[j] = __fmaf_rn(up[r * stride + j], l, z[j]);
+        for (int j = 0; j < 4; ++j) dv[j] = expf(dv[j]);      // (behind the last element: 1)
+      } else {
+        const float* low = a.low + (size_t)t * a.ld_low;
+        const int d = threadIdx.x % KM, part = threadIdx.x / KM;
+        const size_t stride = (size_t)a.H * a.D;
+        const float* up = a.up + (size_t)head * a.D + min(d, a.D - 1);
+        float z = 0.f;
+#pragma unroll 8
+        for (int r = part; r < a.rank; r += PARTS) z = __fmaf_rn(up[r * stride], low[r], z);
+        part_s[part][d] = z;
+        ls_lds_barrier();
+        if (threadIdx.x < KM) {
+          float sum = part_s[0][d];
+#pragma unroll
+          for (int i = 1; i < PARTS; ++i) sum += part_s[i][d];
+          decay_s[d] = d < a.D ? expf(ls_log_decay(sum + a.up_bias[(size_t)head * a.D + d], a.tau)) : 1.f;
+        }
+        ls_lds_barrier();
+        dv = *reinterpret_cast<const f32x4*>(&decay_s[d0]);
       }
-#pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (d0 + j < a.D) lv[j] = ls_log_decay(z[j] + a.up_bias[(size_t)head * a.D + d0 + j], a.tau);
+    } else {
+      const float step = ls_softplus(a.raw[(size_t)t * a.ld_raw + a.raw_col + head] + bias);
+      const float decay = expf(rate * step);
+      kv *= step;
+      dv = f32x4{decay, decay, decay, decay};
     }
-    float step = 1.f, decay = 1.f;
-    if (!CHANNEL) {
-      step = ls_softplus(a.raw[(size_t)t * a.ld_raw + a.raw_col + head] + bias);
-      decay = expf(rate * step);
-    }
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const bool in = d0 + j < a.D;
-      qv[j] = in ? q[d0 + j] * a.q_scale : 0.f;
-      kv[j] = in ? k[d0 + j] * step : 0.f;
-      dv[j] = CHANNEL ? (in ? expf(a.logs ? a.logs[(size_t)t * a.ld_logs + (size_t)head * a.D + d0 + j] : lv[j]) : 1.f) : decay;
-    }
+    qv *= a.q_scale;
     const float* v = row + a.v_col + (size_t)head * a.E;
 #pragma unroll
     for (int c = 0; c < CPT; ++c) {
@@ -553,7 +573,8 @@ static int ls_launch(const LsArgs& a, const LsSegments& sg, int n_seqs, int walk
 }
 
 // Sequences seq0 .. seq0 + n_seqs - 1. logs given, or, walked, what they are formed from (low, up, up_bias, tau): the
-// channel form; else the head form (raw, dt_bias, A_log; skip or null). walk != 0: token by token; else chunks, for portions of up to max_q_len tokens.
+// channel form; else the head form (raw, dt_bias, A_log; skip or null). walk != 0: token by token; else chunks, for portions
+// of up to max_q_len tokens.
 extern "C" int tw_linear_state(const float* src, long ld, int q_col, int k_col, int v_col, int share, const float* logs,
                                long ld_logs, const float* low, long ld_low, int rank, const float* up,
                                const float* up_bias, float tau, const float* raw, long ld_raw, int raw_col, const float* dt_bias,
@@ -570,8 +591,10 @@ extern "C" int tw_linear_state(const float* src, long ld, int q_col, int k_col, 
   TW_REQUIRE((uintptr_t)state % 16 == 0 && n_seqs <= 65535 && H <= 65535);
   if (n_seqs == 0) return 0;
   const int Dp = (D + 15) / 16 * 16, Ep = (E + 15) / 16 * 16;
-  LsArgs a{src, ld, q_col, k_col, v_col, share, logs, ld_logs, low, ld_low, rank, up, up_bias, tau, raw, ld_raw, raw_col, dt_bias, A_log, skip, state, q_start,
-           state_slots, seq0, out, ld_out, H, D, E, Dp, Ep, q_scale};
+  LsArgs a{src, ld, q_col, k_col, v_col, share, logs, ld_logs, low, ld_low, rank, up, up_bias, tau, raw, ld_raw, raw_col,
+           dt_bias, A_log, skip, state, q_start,
+           state_slots, seq0, out, ld_out, H, D, E, Dp, Ep, q_scale,
+           D % 4 == 0 && ld % 4 == 0 && q_col % 4 == 0 && k_col % 4 == 0 && (uintptr_t)src % 16 == 0};
   LsSegments sg{nullptr, nullptr, 0, 1};
   if (!walk) {
     ls_segments(n_seqs, max_q_len, H, Ep, &sg.len, &sg.count);

@@ -216,7 +216,8 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(ConvArgs a) {
 // statistics come from `row_rinv`. What a row reads and writes is exactly what `causal_conv_kernel` reads and
 // writes for it.
 #define TW_CONV_TILE 8
-template <typename SrcT, typename OutT, bool NORM>
+// TAPS: their number, where it is known (else 0).
+template <typename SrcT, typename OutT, bool NORM, int TAPS>
 __global__ __launch_bounds__(256) void causal_conv_tile_kernel(ConvArgs a, int n_tokens) {
   __shared__ int info[TW_CONV_TILE][5];                   // per row of the tile: first row, start, length, slot, phase
   const int row0 = blockIdx.x * TW_CONV_TILE;
@@ -231,21 +232,31 @@ __global__ __launch_bounds__(256) void causal_conv_tile_kernel(ConvArgs a, int n
     info[threadIdx.x][4] = a.phase[s] & 1;
   }
   __syncthreads();
-  const int K = a.K, C = a.C;
+  constexpr int MOST = TAPS ? TAPS : TW_CONV_MAX_TAPS;
+  const int K = TAPS ? TAPS : a.K, C = a.C;
   const SrcT* src = (const SrcT*)a.src;
   for (int c = (blockIdx.y * blockDim.x + threadIdx.x) * 4; c < C; c += gridDim.y * blockDim.x * 4) {
     f32x4 rows_in[TW_CONV_TILE];                          // the tile's own rows, all on their way at once
 #pragma unroll
     for (int i = 0; i < TW_CONV_TILE; ++i)
       rows_in[i] = i < rows ? conv_load4(src + (size_t)(row0 + i) * a.ld_src + c) : f32x4{0.f, 0.f, 0.f, 0.f};
-    f32x4 w[TW_CONV_MAX_TAPS];                            // w[j][e]: tap j of channel c + e
+    f32x4 w[MOST];                                        // w[j][e]: tap j of channel c + e
+    if constexpr (TAPS == 4) {
 #pragma unroll
-    for (int j = 0; j < TW_CONV_MAX_TAPS; ++j)
+      for (int e = 0; e < 4; ++e) {
+        const f32x4 own = conv_load4(a.taps + (size_t)(c + e) * 4);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) w[j][e] = j < K ? a.taps[(size_t)(c + e) * K + j] : 0.f;
+        for (int j = 0; j < 4; ++j) w[j][e] = own[j];
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < MOST; ++j)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) w[j][e] = j < K ? a.taps[(size_t)(c + e) * K + j] : 0.f;
+    }
     const f32x4 bias = a.bias ? conv_load4(a.bias + c) : f32x4{0.f, 0.f, 0.f, 0.f};
     const f32x4 nw = NORM ? conv_load4(a.norm_w + c) : f32x4{1.f, 1.f, 1.f, 1.f};
-    f32x4 v[TW_CONV_MAX_TAPS];                            // v[j]: the input that meets tap j; v[K - 1] the current row's
+    f32x4 v[MOST];                                        // v[j]: the input that meets tap j; v[K - 1] the current row's
 #pragma unroll
     for (int i = 0; i < TW_CONV_TILE; ++i) {
       if (i >= rows) break;
@@ -256,7 +267,7 @@ __global__ __launch_bounds__(256) void causal_conv_tile_kernel(ConvArgs a, int n
       if (i == 0 || row == first) {
         // a tile or a portion begins: the earlier inputs come from this step's rows, the state, or nothing
 #pragma unroll
-        for (int j = 0; j < TW_CONV_MAX_TAPS - 1; ++j) {
+        for (int j = 0; j < MOST - 1; ++j) {
           v[j] = f32x4{0.f, 0.f, 0.f, 0.f};
           const int p = pos - (K - 1) + j;
           if (j < K - 1) {
@@ -274,26 +285,26 @@ __global__ __launch_bounds__(256) void causal_conv_tile_kernel(ConvArgs a, int n
       if (NORM) cur = cur * a.row_rinv[row] * nw;
       f32x4 acc = bias + a.identity * cur;
 #pragma unroll
-      for (int j = 0; j < TW_CONV_MAX_TAPS - 1; ++j)
+      for (int j = 0; j < MOST - 1; ++j)
         if (j < K - 1) acc += w[j] * v[j];
       // (the current row meets the last tap, whose index is only known at run time)
 #pragma unroll
-      for (int j = 0; j < TW_CONV_MAX_TAPS; ++j)
+      for (int j = 0; j < MOST; ++j)
         if (j == K - 1) acc += w[j] * cur;
       acc = conv_act(acc, a.act);
       if (a.out) conv_store4((OutT*)a.out + (size_t)row * a.ld_out + c, acc);
       if (a.out32) conv_store4(a.out32 + (size_t)row * a.ld_out32 + c, acc);
       // shift: what met tap j + 1 meets tap j for the next row
 #pragma unroll
-      for (int j = 0; j < TW_CONV_MAX_TAPS - 2; ++j)
+      for (int j = 0; j < MOST - 2; ++j)
         if (j < K - 2) v[j] = v[j + 1];
 #pragma unroll
-      for (int j = 0; j < TW_CONV_MAX_TAPS - 1; ++j)
+      for (int j = 0; j < MOST - 1; ++j)
         if (j == K - 2) v[j] = cur;
       if (pos == len - 1) {
         float* new_state = a.state + ((size_t)info[i][3] * 2 + (1 - info[i][4])) * (size_t)(K - 1) * C;
 #pragma unroll
-        for (int j = 0; j < TW_CONV_MAX_TAPS - 1; ++j)
+        for (int j = 0; j < MOST - 1; ++j)
           if (j < K - 1) conv_store4(new_state + (size_t)j * C + c, v[j]);
       }
     }
@@ -352,9 +363,12 @@ extern "C" int tw_causal_conv(int dtype, int src_f32, const void* src, long ld_s
                    (!out32 || (ld_out32 % 4 == 0 && (uintptr_t)out32 % 16 == 0)) && (uintptr_t)state % 16 == 0 &&
                    (!bias || (uintptr_t)bias % 16 == 0) && (!norm_w || (uintptr_t)norm_w % 16 == 0);
   const bool tiled = vec && n_tokens >= 512 && (!norm_w || row_rinv);
+  const bool four = K == 4 && (uintptr_t)taps % 16 == 0;
 #define TW_CONV_LAUNCH(S, O, N)                                                                    \
   do {                                                                                             \
-    if (tiled) causal_conv_tile_kernel<S, O, N><<<dim3(tw_div_up(n_tokens, TW_CONV_TILE), tw_div_up(C, 1024)), 256, 0, stream>>>(a, n_tokens); \
+    const dim3 tiles(tw_div_up(n_tokens, TW_CONV_TILE), tw_div_up(C, 1024));                       \
+    if (tiled && four) causal_conv_tile_kernel<S, O, N, 4><<<tiles, 256, 0, stream>>>(a, n_tokens); \
+    else if (tiled) causal_conv_tile_kernel<S, O, N, 0><<<tiles, 256, 0, stream>>>(a, n_tokens);   \
     else if (vec) causal_conv_kernel<S, O, N, true><<<n_blocks, 256, 0, stream>>>(a);              \
     else causal_conv_kernel<S, O, N, false><<<n_blocks, 256, 0, stream>>>(a);                      \
   } while (0)

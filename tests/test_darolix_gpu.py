@@ -263,6 +263,40 @@ def test_decaying_states_in_segments(device, form):
         assert err < 2e-5, (s, float(err))
 
 
+@pytest.mark.parametrize("H,D,E,rank,tau", [(3, 20, 24, 1, 1.0), (2, 64, 48, 16, 16.0), (1, 13, 10, 7, 0.3), (2, 128, 33, 130, 8.0), (4, 8, 70, 5, 2.0),
+                                            (2, 200, 20, 33, 16.0)])
+def test_walked_states_that_form_their_decays(device, H, D, E, rank, tau):
+    """Steps of one to four tokens a sequence whose decays are given by their low-rank product."""
+    from tessweave_engine_amd.kernels import ops
+    g = torch.Generator().manual_seed(D + rank)
+    Dp, Ep = (D + 15) // 16 * 16, (E + 15) // 16 * 16
+    up, bias = torch.randn(H * D, rank, generator=g) / math.sqrt(rank), 2.0 * torch.randn(H * D, generator=g)
+    cuts, at = [[4, 1, 2, 1], [1, 3, 1, 4]], [0, 0]
+    rows = [torch.randn(sum(c), 2 * H * D + H * E, generator=g) for c in cuts]
+    low = [torch.randn(sum(c), rank + 3, generator=g) for c in cuts]
+    want = []
+    for s in range(2):
+        T = len(rows[s])
+        alpha = torch.sigmoid(low[s][:, 3:].double() @ up.double().T + bias.double()) ** (1.0 / tau)
+        q, k = rows[s][:, :H * D].double().view(T, H, D) * 0.7, rows[s][:, H * D:2 * H * D].double().view(T, H, D)
+        v = rows[s][:, 2 * H * D:].double().view(T, H, E)
+        want.append(torch.stack([plain.linear_attention_steps(q[:, a], k[:, a], v[:, a], alpha.view(T, H, D)[:, a]) for a in range(H)], 1))
+    state = torch.zeros(3, H, Ep, Dp, device=device)
+    for i in range(4):
+        n = [c[i] for c in cuts]
+        src = torch.cat([rows[s][at[s]:at[s] + n[s]] for s in range(2)]).to(device)
+        lo = torch.cat([low[s][at[s]:at[s] + n[s]] for s in range(2)]).to(device)
+        out = torch.full((sum(n), H * E), float("nan"), device=device)
+        ops.linear_state(src, 0, H * D, 2 * H * D, state, ints([0, n[0], sum(n)], device), ints([2, 0], device), 0, 2, out, H, D, E,
+                         q_scale=0.7, walk=True, max_q_len=max(n), low_rank=(lo[:, 3:], up.t().contiguous().to(device), bias.to(device), tau))
+        for s in range(2):
+            got = out[:n[0]] if s == 0 else out[n[0]:]
+            ref = want[s].reshape(-1, H * E)[at[s]:at[s] + n[s]]
+            assert (got.double().cpu() - ref).abs().max() < 1e-5 * max(1.0, want[s].abs().max().item()), (i, s)
+            at[s] += n[s]
+    assert not state[1].any()
+
+
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("H,G,D,E,cap,page", [(4, 2, 24, 20, 30.0, 4), (8, 8, 32, 64, 0.0, 16), (6, 1, 50, 34, 12.0, 8), (3, 3, 128, 96, 25.0, 16),
                                               (10, 2, 64, 64, 20.0, 16), (2, 2, 15, 7, 15.0, 4)])
@@ -315,11 +349,11 @@ def test_normed_heads_with_a_temperature_made_sharp(device, dtype, H, G, D, E, c
     assert torch.allclose(q_got[:, :, :D], q_want, rtol=2e-6 if dtype == "float32" else 5e-3, atol=1e-6) and not q_got[:, :, D:].any()
 
 
+@pytest.mark.parametrize("n", [37, 203, 1001])
 @pytest.mark.parametrize("C,X,top", [(72, 70, 4), (90, 7, 3), (64, 1, 1), (2048, 24, 2), (88, 5, 5)])
-def test_router_with_a_correction(device, C, X, top):
+def test_router_with_a_correction(device, C, X, top, n):
     from tessweave_engine_amd.kernels import ops
     g = torch.Generator().manual_seed(C + X)
-    n = 37
     h = torch.randn(n, C, generator=g).to(device)
     router = (2.0 * torch.randn(X, C, generator=g) / math.sqrt(C)).to(device)
     correction = (0.3 * torch.randn(X, generator=g)).to(device)
@@ -343,7 +377,8 @@ def test_router_with_a_correction(device, C, X, top):
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("n,C,X,identity,top,F", [(1, 88, 5, 2, 2, 40), (9, 128, 16, 0, 4, 64), (300, 96, 3, 3, 3, 24), (130, 72, 64, 8, 1, 100),
-                                                  (17, 64, 1, 5, 2, 32), (40, 50, 2, 1, 3, 20)])
+                                                  (17, 64, 1, 5, 2, 32), (40, 50, 2, 1, 3, 20), (40, 64, 1, 0, 1, 48),
+                                                  (64, 256, 2, 1, 1, 40), (32, 128, 3, 1, 2, 17), (5, 64, 1, 9, 2, 24)])
 def test_grouped_experts_with_identities(device, dtype, n, C, X, identity, top, F):
     """Gated experts beside ones that return the input; a mixer's split-K sums go into the same result."""
     from tessweave_engine_amd.kernels import ops

@@ -167,13 +167,14 @@ def test_causal_conv_over_portions_and_reused_slots(device, dtype, taps, norm, C
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("taps,norm", [(4, True), (3, False), (1, True), (8, False), (2, True)])
-def test_causal_conv_of_many_rows(device, dtype, taps, norm):
+@pytest.mark.parametrize("taps,norm,C", [(4, True, 48), (3, False, 48), (1, True, 48), (8, False, 48), (2, True, 48), (4, False, 2308),
+                                         (5, True, 1028)])
+def test_causal_conv_of_many_rows(device, dtype, taps, norm, C):
     """A step of 640 rows (the kernel that walks tiles of rows): a sequence that starts in it, one that goes on from
     its state (whose first tokens come mid-tile), one of two tokens, one of one token that began steps ago."""
     from tessweave_engine_amd.kernels import ops
     g = torch.Generator().manual_seed(taps + 10 * norm)
-    C, dt = 48, tdtype(dtype)
+    dt = tdtype(dtype)
     w = torch.randn(C, taps, generator=g)
     bias = None if norm else torch.randn(C, generator=g)
     nw = 1 + 0.3 * torch.randn(C, generator=g)
