@@ -15,11 +15,12 @@
 //   p = s of the chosen over their sum (+ 1e-20)        expert(y): down( silu(gate y) * up y ); the last `identity`
 //   out = sum over the chosen experts e of  p_e * expert_e(h)          experts return h itself
 //
-// A step runs in six launches (four where there are few pairs: see PLAN below) whose shapes depend only on the number of rows: route; plan (every expert's rows are
-// laid out one expert after the other, each expert's share padded to whole tiles of 16 rows; which expert a tile
-// belongs to is a table on the device, tiles nobody uses say -1); gather (the scaled, rounded input rows in that
-// order); two grouped products on the matrix unit, one workgroup a (tile, range of columns), whose weights are the
-// tile's expert's; combine (each token adds its experts' rows in the order it chose them). No launch waits for the
+// A step runs in six launches (four where there are few pairs: see PLAN below) whose shapes depend only on the number
+// of rows: route; plan (every expert's rows are laid out one expert after the other, each expert's share padded to whole
+// tiles of 16 rows; which expert a tile belongs to is a table on the device, tiles nobody uses say -1); gather (the
+// scaled, rounded input rows in that order); two grouped products on the matrix unit, one workgroup a (tile, range of
+// columns), whose weights are the tile's expert's; combine (each token adds its experts' rows in the order it chose
+// them; a choice of an identity expert adds the input row itself). No launch waits for the
 // host, so the whole runs inside a captured graph.
 //
 // The experts' matrices lie stacked, K padded to a multiple of 32 by zeros and rows to a multiple of 16, in the order the
@@ -556,8 +557,9 @@ static void moe_run(const MoeStep& s, hipStream_t stream) {
 }
 
 // h [n][C] (compute type) -> x [n][C] float32 += the routed experts' results. ids, weights [n * top] come from
-// tw_moe_route (ids of X and above, where the weights multiply outputs: experts that return h). Scratch: pos [n * top], src_item [capacity], tile_expert [capacity / 16] (int32), xs [capacity][Cd],
-// act [capacity][Fd] (compute type), ys [capacity][C] (float32), capacity = tw_moe_capacity(n * top, X).
+// tw_moe_route (ids of X and above, where the weights multiply outputs: experts that return h). Scratch: pos [n * top],
+// src_item [capacity], tile_expert [capacity / 16] (int32), xs [capacity][Cd], act [capacity][Fd] (compute type),
+// ys [capacity][C] (float32), capacity = tw_moe_capacity(n * top, X).
 extern "C" int tw_moe_experts(int dtype, const void* h, long ld_h, const int* ids, const float* weights, int n, int top, int X,
                               const void* gate, const void* up, const void* down, int C, int Cd, int Fd, float limit,
                               int* pos, int* src_item, int* tile_expert, void* xs, void* act, float* ys, int capacity,
