@@ -2,12 +2,12 @@
 
 For every live request (`Sequence`) it keeps, per group, the list of physical
 pages that hold the request's logical blocks (-1 where a block is not held: a
-window has passed it, or it is not yet allocated), and one slot index into the
+window or chunk has passed it, or it is not yet allocated), and one slot index into the
 fixed-size state arrays. Position p of a request lives in
 `table[p // page_size] * page_size + p % page_size` (flow_engine/cache.py:93-95).
 
 Pages come back when a request closes (flow_engine/engine.py:132-133) and,
-for a windowed group, as soon as no later query can see them.
+for a windowed or chunked group, as soon as no later query can see them.
 """
 from __future__ import annotations
 
@@ -154,11 +154,11 @@ class CacheManager:
         """Most pages of GROUP a request of TOTAL_TOKENS holds at once."""
         spec = self.layout.groups[group].spec
         full = math.ceil(total_tokens / self.page_size)
-        if spec.window is None:
+        if spec.keeps_all:
             return full
-        # Live positions span at most window - 1 old keys plus one step's tokens;
+        # Live positions span at most window - 1 old keys plus one step's tokens (as many of a chunk);
         # such a span touches at most ceil(span / page) + 1 pages.
-        span = spec.window - 1 + max(1, largest_step)
+        span = spec.span - 1 + max(1, largest_step)
         return min(full, math.ceil(span / self.page_size) + 1 + self.kept_blocks(group))
 
     def fits(self, total_tokens, largest_step):
@@ -240,10 +240,7 @@ class CacheManager:
 
     def first_needed_block(self, group, computed):
         """First logical block of GROUP that a query at position >= COMPUTED can see."""
-        window = self.layout.groups[group].spec.window
-        if window is None:
-            return 0
-        return max(0, computed - window + 1) // self.page_size
+        return self.layout.groups[group].spec.first_position(computed) // self.page_size
 
     def ensure(self, seq, n_tokens):
         """Hold pages for positions [seq.computed, n_tokens) in every group; all or nothing."""
@@ -279,12 +276,12 @@ class CacheManager:
             seq.promised[g] -= from_promise
 
     def advance(self, seq, computed):
-        """Record that the cache now holds COMPUTED tokens; give back pages a window has passed."""
+        """Record that the cache now holds COMPUTED tokens; give back pages that no later query sees."""
         if computed < seq.computed:
             raise ValueError("a request's computed length cannot shrink")
         seq.computed = computed
         for g, pool in enumerate(self.pools):
-            if self.layout.groups[g].spec.window is None:
+            if self.layout.groups[g].spec.keeps_all:
                 continue
             table = seq.tables[g]
             first = min(self.first_needed_block(g, computed), len(table))

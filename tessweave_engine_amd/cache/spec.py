@@ -14,14 +14,20 @@ from dataclasses import dataclass
 @dataclass(frozen=True)
 class PagedKV:
     """Keys and values of every token (window None) or of the last `window` tokens; with a window, `keep_first` says
-    how many of a request's first tokens stay held whatever the window has passed."""
+    how many of a request's first tokens stay held whatever the window has passed. `chunks`, in place of a window: sizes of
+    chunks of positions, counted from a request's start, whose queries see their own chunk only (several readers of one
+    cache may have several sizes); tokens are held until every one of these chunks has ended."""
     kv_heads: int
     head_dim: int
     window: int | None = None
     value_dim: int | None = None      # size of a value if it differs from a key's (None: head_dim)
     keep_first: int = 0
+    chunks: tuple = ()
 
     def __post_init__(self):
+        object.__setattr__(self, "chunks", tuple(sorted({int(c) for c in self.chunks})))
+        if any(c <= 0 for c in self.chunks) or (self.chunks and self.window is not None):
+            raise ValueError("chunk sizes must be positive and take the place of a window")
         if self.value_dim == self.head_dim:
             object.__setattr__(self, "value_dim", None)
         if self.kv_heads <= 0 or self.head_dim <= 0 or (self.value_dim is not None and self.value_dim <= 0):
@@ -32,6 +38,28 @@ class PagedKV:
             raise ValueError("keep_first cannot be negative")
         if self.window is None:
             object.__setattr__(self, "keep_first", 0)          # (without a window everything is kept anyway)
+
+    @property
+    def keeps_all(self):
+        """Does a request hold every token's keys and values to its end?"""
+        return self.window is None and not self.chunks
+
+    @property
+    def span(self):
+        """Most positions a query sees, its own included (None: no bound)."""
+        return self.window if self.window is not None else max(self.chunks, default=None)
+
+    def first_position(self, position):
+        """The first position that a query at POSITION or later can see (kept first tokens aside); POSITION may be an array."""
+        if self.window is not None:
+            return (position - self.window + 1) * (position >= self.window)
+        if not self.chunks:
+            return position * 0
+        first = position // self.chunks[0] * self.chunks[0]
+        for c in self.chunks[1:]:
+            other = position // c * c
+            first = first * (first <= other) + other * (other < first)
+        return first
 
 
 @dataclass(frozen=True)
@@ -100,7 +128,7 @@ class CacheLayout:
     @property
     def shares_prefixes(self):
         """Full pages of a prompt prefix can be reused only if they are all a request holds."""
-        return (len(self.groups) == 1 and self.groups[0].spec.window is None
+        return (len(self.groups) == 1 and self.groups[0].spec.keeps_all
                 and not self.state_slots and not self.named_state_slots)
 
     def bytes_per_token(self, element_bytes):

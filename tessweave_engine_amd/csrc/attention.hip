@@ -5,7 +5,8 @@
 //   block_table[seq][b] = physical page of logical block b, or -1 if not held
 //
 // A query at absolute position t of a sequence with kv_len cached keys sees key
-// p iff p <= t, p < kv_len and (window == 0 or p > t - window). Scores are
+// p iff p <= t, p < kv_len and (window == 0 or p > t - window) and (chunk == 0 or
+// p / chunk == t / chunk: chunks are counted from the sequence's start). Scores are
 // q.k * scale; softmax statistics, probabilities and the output sum are float32.
 // Masked scores are SELECTED to -inf and keys outside the sequence are loaded
 // as zeros, so whatever an unowned or reused page holds (NaN included) never
@@ -70,12 +71,27 @@ struct AttnArgs {
   int tile_rows;          // rows of such a tile: 128, or 64 when there would be too few workgroups
   int kv_chunk, max_chunks;  // prefill (bfloat16 kernel): keys per workgroup (a multiple of 32) and the most
                              // chunks a tile can have; max_chunks == 1: a tile's keys are never split
-  const float* sink;         // prefill only. [q_heads] or null: exp(sink_h) more in head h's denominator (a score of its
-                             // own, not scaled, with no key and no value)
+  const float* sink;         // [q_heads] or null: exp(sink_h) more in head h's denominator (a score of its own, not scaled,
+                             // with no key and no value)
+  const float* gate;         // [token rows][q_heads] or null: a factor on a head's result
+  int chunk;                 // > 0: a query sees only keys of its own chunk of that many positions (then window is 0)
+  int out_f32;               // the result is written in float32 whatever the type of q
   float* stats;              // prefill only. [token rows][q_heads][2] or null: what a row's softmax was taken against (the
                              // reference, as a scaled score in natural units) and its sum relative to that, for whoever adds
                              // more keys to the row afterwards
 };
+
+// The first position that a query at position t sees.
+__device__ __forceinline__ int attn_first_seen(const AttnArgs& a, int t) {
+  if (a.window > 0) return max(0, t - a.window + 1);
+  return a.chunk > 0 ? t - t % a.chunk : 0;
+}
+
+// What a row's sums are multiplied by: one over its denominator, times the gate of its head.
+__device__ __forceinline__ float attn_row_factor(const AttnArgs& a, int row, int head, float l) {
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+  return a.gate ? inv * a.gate[(size_t)row * a.q_heads + head] : inv;
+}
 
 // Per-wave online-softmax state for one 16-row tile. Lane (r, g) belongs to row r.
 template <typename T, int DTMAX>
@@ -127,7 +143,7 @@ struct RowTile {
       }
     }
     // ---- mask, online softmax (this lane: row r, keys p0 + 4g + j) ------------
-    const int lo_row = a.window > 0 ? t_row - a.window + 1 : 0;
+    const int lo_row = attn_first_seen(a, t_row);
     float mx = -INFINITY;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
@@ -178,6 +194,26 @@ struct RowTile {
   }
 };
 
+// A lane's elements of a row's result, 4 g .. 4 g + 3 of every 16: times the row's factor, into the output's type.
+template <typename T, int DTMAX, bool EXACT>
+__device__ __forceinline__ void attn_store_row(const AttnArgs& a, int row, int head, int D, int g, const f32x4 (&acc)[DTMAX],
+                                               float factor) {
+  const size_t at = (size_t)row * a.ldo + (size_t)head * D + 4 * g;
+  if (a.out_f32) {
+#pragma unroll
+    for (int dt = 0; dt < DTMAX; ++dt)
+      if (EXACT || dt * 16 < D)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) ((float*)a.out)[at + dt * 16 + j] = acc[dt][j] * factor;
+  } else {
+#pragma unroll
+    for (int dt = 0; dt < DTMAX; ++dt)
+      if (EXACT || dt * 16 < D)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) ((T*)a.out)[at + dt * 16 + j] = tw_from_float<T>(acc[dt][j] * factor);
+  }
+}
+
 // =====================================================================================
 // Decode: one token per sequence. grid = (splits, kv_heads * row_tiles, n_seqs).
 // =====================================================================================
@@ -204,7 +240,7 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(AttnArgs a) {
   RowTile<T, DTMAX> tile;
   tile.init(row_ok ? (const T*)a.q + (size_t)token * a.ldq + (size_t)head * D : nullptr, D, g);
 
-  const int lo = a.window > 0 ? max(0, t - a.window + 1) : 0;
+  const int lo = attn_first_seen(a, t);
   const int tile_lo = lo / 16, tile_hi = (kv_len + 15) / 16;     // key tiles [tile_lo, tile_hi)
   const int per_split = (tile_hi - tile_lo + a.splits - 1) / a.splits;
   const int begin = tile_lo + split * per_split;
@@ -248,13 +284,9 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(AttnArgs a) {
   }
   if (!row_ok) return;
   if (a.splits == 1) {
-    const float inv = l > 0.f ? 1.f / l : 0.f;
-    T* dst = (T*)a.out + (size_t)token * a.ldo + (size_t)head * D;
-#pragma unroll
-    for (int dt = 0; dt < DTMAX; ++dt)
-      if (dt < dts)
-#pragma unroll
-        for (int j = 0; j < 4; ++j) dst[dt * 16 + 4 * g + j] = tw_from_float<T>(tile.acc[dt][j] * inv);
+    if (a.sink) l += tw_exp<float>(a.sink[head] - m_use);
+    const float inv = attn_row_factor(a, token, head, l);
+    attn_store_row<T, DTMAX, false>(a, token, head, D, g, tile.acc, inv);
   } else {
     const size_t slot = ((size_t)blockIdx.z * a.q_heads + head) * a.splits + split;
     float* dst = a.part_o + slot * D;
@@ -329,7 +361,7 @@ __global__ __launch_bounds__(256) void attn_decode_bf16_kernel(AttnArgs a) {
   for (int dt = 0; dt < DTMAX; ++dt) acc[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
 
-  const int lo = a.window > 0 ? max(0, t - a.window + 1) : 0;
+  const int lo = attn_first_seen(a, t);
   const int blk_lo = lo / 32, blk_hi = (kv_len + 31) / 32;
   const int per_split = (blk_hi - blk_lo + a.splits - 1) / a.splits;
   const int begin = blk_lo + split * per_split;
@@ -509,13 +541,9 @@ __global__ __launch_bounds__(256) void attn_decode_bf16_kernel(AttnArgs a) {
   }
   if (!row_ok) return;
   if (a.splits == 1) {
-    const float inv = l > 0.f ? 1.f / l : 0.f;
-    bf16_t* dst = (bf16_t*)a.out + (size_t)token * a.ldo + (size_t)head * D;
-#pragma unroll
-    for (int dt = 0; dt < DTMAX; ++dt)
-      if (EXACT || dt < dts)
-#pragma unroll
-        for (int j = 0; j < 4; ++j) dst[dt * 16 + 4 * g + j] = (bf16_t)(acc[dt][j] * inv);
+    if (a.sink) l += __expf(a.sink[head] - m_use);
+    const float inv = attn_row_factor(a, token, head, l);
+    attn_store_row<bf16_t, DTMAX, EXACT>(a, token, head, D, g, acc, inv);
   } else {
     const size_t slot = ((size_t)blockIdx.z * a.q_heads + head) * a.splits + split;
     float* dst = a.part_o + slot * D;
@@ -538,7 +566,8 @@ __global__ __launch_bounds__(256) void attn_decode_bf16_kernel(AttnArgs a) {
 template <typename T>
 __global__ __launch_bounds__(TW_REDUCE_THREADS) void attn_decode_reduce_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml, const int* __restrict__ q_start,
-    int seq0, T* out, long ldo, int q_heads, int head_dim, int splits) {
+    int seq0, T* out, long ldo, int q_heads, int head_dim, int splits, const float* __restrict__ sink,
+    const float* __restrict__ gate) {
   __shared__ float s_w[64];                    // weight of each split: exp(m_s - m)
   __shared__ float s_acc[TW_REDUCE_THREADS];
   __shared__ float s_l;
@@ -565,6 +594,7 @@ __global__ __launch_bounds__(TW_REDUCE_THREADS) void attn_decode_reduce_kernel(
     // fixed-order sum over the splits
     float l = 0.f;
     for (int i = 0; i < 64; ++i) l += __shfl(lw, i, TW_WAVE);
+    if (sink) l += expf(sink[head] - m_use);
     if (tid == 0) s_l = l;
   }
   __syncthreads();
@@ -583,7 +613,9 @@ __global__ __launch_bounds__(TW_REDUCE_THREADS) void attn_decode_reduce_kernel(
     float total = 0.f;
     for (int i = 0; i < cols; ++i) total += s_acc[i * head_dim + tid];
     const float l = s_l;
-    out[(size_t)token * ldo + (size_t)head * head_dim + tid] = tw_from_float<T>(l > 0.f ? total / l : 0.f);
+    total = l > 0.f ? total / l : 0.f;
+    if (gate) total *= gate[(size_t)token * q_heads + head];
+    out[(size_t)token * ldo + (size_t)head * head_dim + tid] = tw_from_float<T>(total);
   }
 }
 
@@ -605,7 +637,7 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(AttnArgs a) {
   const int row0 = (blockIdx.x * 4 + wave) * 16;
   if (row0 >= rows) return;
   const int* table = a.block_table + (size_t)seq * a.table_stride;
-  const int D = a.head_dim, dts = D / 16;
+  const int D = a.head_dim;
 
   const int row = row0 + r;
   const bool row_ok = row < rows;
@@ -622,23 +654,18 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(AttnArgs a) {
 
   const int t_min = first_pos + row0 / G;
   const int t_max = first_pos + min(rows - 1, row0 + 15) / G;
-  const int lo = a.window > 0 ? max(0, t_min - a.window + 1) : 0;
+  const int lo = attn_first_seen(a, t_min);
   for (int kt = lo / 16; kt * 16 <= t_max; ++kt)
     tile.key_tile(a, table, kvh, kt * 16, kv_len, t_row, lo, r, g);
 
   if (!row_ok) return;
-  const float inv = tile.l > 0.f ? 1.f / tile.l : 0.f;
+  const float inv = attn_row_factor(a, token0 + tok, head, tile.l);
   if (a.stats && g == 0) {
     float* st = a.stats + ((size_t)(token0 + tok) * a.q_heads + head) * 2;
     st[0] = tile.m == -INFINITY ? 0.f : tile.m;
     st[1] = tile.l;
   }
-  T* dst = (T*)a.out + (size_t)(token0 + tok) * a.ldo + (size_t)head * D;
-#pragma unroll
-  for (int dt = 0; dt < DTMAX; ++dt)
-    if (dt < dts)
-#pragma unroll
-      for (int j = 0; j < 4; ++j) dst[dt * 16 + 4 * g + j] = tw_from_float<T>(tile.acc[dt][j] * inv);
+  attn_store_row<T, DTMAX, false>(a, token0 + tok, head, D, g, tile.acc, inv);
 }
 
 // =====================================================================================
@@ -764,7 +791,7 @@ __global__ __launch_bounds__(256) void attn_prefill_bf16_kernel(AttnArgs a) {
   // ---- the workgroup's key range ------------------------------------------------
   const int t_min = first_pos + wg_row0 / G;
   const int t_max = first_pos + min(rows - 1, wg_row0 + TR - 1) / G;
-  const int lo = a.window > 0 ? max(0, t_min - a.window + 1) : 0;       // keys below are never loaded
+  const int lo = attn_first_seen(a, t_min);                              // keys below are never loaded
   // The tile's key blocks, and the share of them this workgroup takes. A tile split into several
   // chunks leaves float32 partial results (running maximum, sum, output) that a second kernel merges.
   const int tile_begin = lo / 32, tile_end = t_max / 32 + 1;
@@ -775,7 +802,7 @@ __global__ __launch_bounds__(256) void attn_prefill_bf16_kernel(AttnArgs a) {
   const int wave_t_max = first_pos + min(rows - 1, wg_row0 + wave * 16 * RT + 16 * RT - 1) / G;
   const int wave_t_min = first_pos + min(rows - 1, wg_row0 + wave * 16 * RT) / G;
   const bool wave_live = wg_row0 + wave * 16 * RT < rows;
-  const int wave_lo_max = a.window > 0 ? wave_t_max - a.window + 1 : 0;  // largest lower bound among the wave's rows
+  const int wave_lo_max = attn_first_seen(a, wave_t_max);               // largest lower bound among the wave's rows
 
   // This thread's share of a block, fixed for the whole loop: K piece i is 16 bytes
   // (chunk k_chunk) of key k_key; V piece i is keys 8*v_oct .. +7 of output dim v_d.
@@ -944,7 +971,7 @@ __global__ __launch_bounds__(256) void attn_prefill_bf16_kernel(AttnArgs a) {
     if (edge) {
 #pragma unroll
       for (int rt = 0; rt < RT; ++rt) {
-        const int lo_row = a.window > 0 ? t_row[rt] - a.window + 1 : 0;
+        const int lo_row = attn_first_seen(a, t_row[rt]);
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
           const int p = p0 + 8 * g + e;
@@ -1349,18 +1376,13 @@ __global__ __launch_bounds__(256) void attn_prefill_bf16_kernel(AttnArgs a) {
 #pragma unroll
   for (int rt = 0; rt < RT; ++rt) {
     if (!row_ok[rt]) continue;
-    const float inv = l[rt] > 0.f ? 1.f / l[rt] : 0.f;
+    const float inv = attn_row_factor(a, token0 + tok[rt], head[rt], l[rt]);
     if (a.stats && g == 0) {
       float* st = a.stats + ((size_t)(token0 + tok[rt]) * a.q_heads + head[rt]) * 2;
       st[0] = m_use[rt] * 0.69314718055994530942f;           // (kept in the log2 domain here)
       st[1] = l[rt];
     }
-    bf16_t* dst = (bf16_t*)a.out + (size_t)(token0 + tok[rt]) * a.ldo + (size_t)head[rt] * D;
-#pragma unroll
-    for (int dt = 0; dt < DTMAX; ++dt)
-      if (EXACT || dt < dts)
-#pragma unroll
-        for (int j = 0; j < 4; ++j) dst[dt * 16 + 4 * g + j] = (bf16_t)(acc[rt][dt][j] * inv);
+    attn_store_row<bf16_t, DTMAX, EXACT>(a, token0 + tok[rt], head[rt], D, g, acc[rt], inv);
   }
 }
 
@@ -1383,7 +1405,7 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(AttnArgs a) {
   const int first_pos = kv_len - q_len;
   const int t_min = first_pos + wg_row0 / G;
   const int t_max = first_pos + min(rows - 1, wg_row0 + a.tile_rows - 1) / G;
-  const int lo = a.window > 0 ? max(0, t_min - a.window + 1) : 0;
+  const int lo = attn_first_seen(a, t_min);
   const int tile_begin = lo / 32, tile_end = t_max / 32 + 1;
   const int chunk_blocks = a.kv_chunk / 32;
   const int n_chunks = (tile_end - tile_begin + chunk_blocks - 1) / chunk_blocks;
@@ -1410,7 +1432,11 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(AttnArgs a) {
       st[0] = m_use * 0.69314718055994530942f;
       st[1] = l_all;
     }
-    const float inv = l_all > 0.f ? 1.f / l_all : 0.f;
+    const float inv = attn_row_factor(a, token0 + tok, head, l_all);
+    if (a.out_f32) {
+      *reinterpret_cast<f32x4*>((float*)a.out + (size_t)(token0 + tok) * a.ldo + (size_t)head * D + grp * 4) = o * inv;
+      continue;
+    }
     bf16_t packed[4];
 #pragma unroll
     for (int e = 0; e < 4; ++e) packed[e] = (bf16_t)(o[e] * inv);
@@ -1514,7 +1540,7 @@ static int check_common(const AttnArgs& a) {
   TW_REQUIRE(a.q_heads > 0 && a.kv_heads > 0 && a.q_heads % a.kv_heads == 0);
   TW_REQUIRE(a.head_dim >= 16 && a.head_dim <= 256 && a.head_dim % 16 == 0);
   TW_REQUIRE(a.page_size >= 4 && a.page_size % 4 == 0);
-  TW_REQUIRE(a.window >= 0 && a.table_stride > 0);
+  TW_REQUIRE(a.window >= 0 && a.chunk >= 0 && (a.window == 0 || a.chunk == 0) && a.table_stride > 0);
   TW_REQUIRE(a.ldq >= (long)a.q_heads * a.head_dim && a.ldo >= (long)a.q_heads * a.head_dim);
   TW_REQUIRE(a.ldq % 8 == 0 && ((uintptr_t)a.q % 16 == 0));
   return 0;
@@ -1575,8 +1601,13 @@ static int decode_launch(AttnArgs a, int n_seqs, int generic, hipStream_t stream
     attn_decode_kernel<T, 16><<<grid, 256, 0, stream>>>(a);
   int err = TW_LAUNCH_RESULT();
   if (err || a.splits == 1) return err;
-  attn_decode_reduce_kernel<T><<<dim3(a.q_heads, n_seqs), TW_REDUCE_THREADS, 0, stream>>>(
-      a.part_o, a.part_ml, a.q_start, a.seq0, (T*)a.out, a.ldo, a.q_heads, a.head_dim, a.splits);
+  const dim3 rgrid(a.q_heads, n_seqs);
+  if (a.out_f32)
+    attn_decode_reduce_kernel<float><<<rgrid, TW_REDUCE_THREADS, 0, stream>>>(
+        a.part_o, a.part_ml, a.q_start, a.seq0, (float*)a.out, a.ldo, a.q_heads, a.head_dim, a.splits, a.sink, a.gate);
+  else
+    attn_decode_reduce_kernel<T><<<rgrid, TW_REDUCE_THREADS, 0, stream>>>(
+        a.part_o, a.part_ml, a.q_start, a.seq0, (T*)a.out, a.ldo, a.q_heads, a.head_dim, a.splits, a.sink, a.gate);
   return TW_LAUNCH_RESULT();
 }
 
@@ -1587,14 +1618,14 @@ extern "C" int tw_attn_decode(int dtype, const void* q, long ldq, const void* ke
                               const int* block_table, int table_stride, const int* q_start,
                               const int* kv_len, int seq0, int n_seqs, void* out, long ldo,
                               float* workspace, long workspace_floats, int q_heads, int kv_heads,
-                              int head_dim, int page_size, int window, float scale, float softcap, int splits,
-                              int generic, hipStream_t stream) {
+                              int head_dim, int page_size, int window, int chunk, float scale, float softcap, int splits,
+                              int generic, const float* sink, const float* gate, int out_f32, hipStream_t stream) {
   AttnArgs a;
   a.q = q; a.ldq = ldq; a.keys = keys; a.values = values; a.block_table = block_table;
   a.table_stride = table_stride; a.q_start = q_start; a.kv_len = kv_len; a.seq0 = seq0;
   a.out = out; a.ldo = ldo; a.q_heads = q_heads; a.kv_heads = kv_heads; a.head_dim = head_dim;
   a.page_size = page_size; a.window = window; a.scale = scale; a.splits = splits;
-  a.sink = nullptr; a.stats = nullptr;
+  a.sink = sink; a.stats = nullptr; a.gate = gate; a.chunk = chunk; a.out_f32 = out_f32;
   TW_REQUIRE(softcap >= 0.f);
   a.softcap = softcap;
   a.part_o = nullptr; a.part_ml = nullptr;
@@ -1644,10 +1675,11 @@ extern "C" int tw_attn_prefill(int dtype, const void* q, long ldq, const void* k
                                const int* kv_len, int seq0, int n_seqs, int max_q_len, void* out,
                                long ldo, float* workspace, long workspace_floats, int n_tokens, int max_chunks,
                                int kv_chunk, int tile_rows, int q_heads, int kv_heads, int head_dim, int page_size,
-                               int window, float scale, float softcap, int generic, const float* sink, float* stats,
-                               hipStream_t stream) {
+                               int window, int chunk, float scale, float softcap, int generic, const float* sink,
+                               float* stats, const float* gate, int out_f32, hipStream_t stream) {
   AttnArgs a;
-  a.sink = sink; a.stats = stats;
+  a.sink = sink; a.stats = stats; a.gate = gate; a.chunk = chunk; a.out_f32 = out_f32;
+  TW_REQUIRE(!stats || !gate);                     // (whoever adds more keys to a row would have to take its gate off again)
   TW_REQUIRE(tile_rows == 0 || tile_rows == 64 || tile_rows == 128);
   a.tile_rows = tile_rows;
   a.q = q; a.ldq = ldq; a.keys = keys; a.values = values; a.block_table = block_table;

@@ -340,22 +340,34 @@ extern "C" int tw_rmsnorm(int out_dtype, float* x, const float* w, void* out, co
 
 // ---- rotary tables: cos/sin[n, j] of angle = float(position[n]) * inv_freq[j], times `magnitude` -----
 // (1 for the plain encoding; encodings that stretch their frequencies for longer contexts also scale both tables)
-__global__ void rope_table_kernel(const int* __restrict__ positions, const float* __restrict__ inv_freq,
+// rest (or null): what float32 rounded off the frequencies; the angle then carries the product's rounding error and this
+// one beside it (at position 1,000 a float32 product alone is off by up to 3e-5).
+__global__ void rope_table_kernel(const int* __restrict__ positions, const float* __restrict__ inv_freq, const float* __restrict__ rest,
                                   float* __restrict__ cos_out, float* __restrict__ sin_out, int n, int half,
                                   float magnitude) {
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= n * half) return;
   const int t = i / half, j = i % half;
-  const float angle = (float)positions[t] * inv_freq[j];
-  cos_out[i] = cosf(angle) * magnitude;
-  sin_out[i] = sinf(angle) * magnitude;
+  const float p = (float)positions[t], f = inv_freq[j];
+  const float angle = __fmul_rn(p, f);
+  float c = cosf(angle), s = sinf(angle);
+  if (rest) {
+    const float off = __fmaf_rn(p, rest[j], __fmaf_rn(p, f, -angle));      // (a few hundredths at most)
+    const float off2 = off * off;
+    const float so = off * __fmaf_rn(-off2, 1.f / 6.f, 1.f), co = -0.5f * off2;
+    const float sine = __fmaf_rn(so, c, __fmaf_rn(co, s, s));
+    c = __fmaf_rn(-so, s, __fmaf_rn(co, c, c));
+    s = sine;
+  }
+  cos_out[i] = c * magnitude;
+  sin_out[i] = s * magnitude;
 }
 
-extern "C" int tw_rope_table(const int* positions, const float* inv_freq, float* cos_out, float* sin_out,
+extern "C" int tw_rope_table(const int* positions, const float* inv_freq, const float* rest, float* cos_out, float* sin_out,
                              int n, int half, float magnitude, hipStream_t stream) {
   TW_REQUIRE(n >= 0 && half > 0);
   if (n == 0) return 0;
-  rope_table_kernel<<<tw_div_up((long)n * half, 256), 256, 0, stream>>>(positions, inv_freq, cos_out,
+  rope_table_kernel<<<tw_div_up((long)n * half, 256), 256, 0, stream>>>(positions, inv_freq, rest, cos_out,
                                                                        sin_out, n, half, magnitude);
   return TW_LAUNCH_RESULT();
 }

@@ -15,6 +15,11 @@
 //   p = s of the chosen over their sum (+ 1e-20)        expert(y): down( silu(gate y) * up y ); the last `identity`
 //   out = sum over the chosen experts e of  p_e * expert_e(h)          experts return h itself
 //
+// A fourth (`kind` 3, `mode` 0 with groups): plain experts whose weights are scaled scores that multiply their outputs,
+//   s = sigmoid(W_router h); the experts stand in `groups` equal groups of neighbours, a group's score is the sum of its two
+//   largest s, only experts of the best `keep` groups can be chosen;     p = scale * s of the chosen
+//   out = sum over the chosen experts e of  p_e * expert_e(h)         expert(y): down( max(up y, 0)^2 )
+//
 // A step runs in six launches (four where there are few pairs: see PLAN below) whose shapes depend only on the number
 // of rows: route; plan (every expert's rows are laid out one expert after the other, each expert's share padded to whole
 // tiles of 16 rows; which expert a tile belongs to is a table on the device, tiles nobody uses say -1); gather (the
@@ -50,9 +55,10 @@ __device__ __forceinline__ f32x4 moe_four(const bf16_t* p) {
 template <typename T, int R, int WAVES>
 __global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(const T* __restrict__ h, long ld_h, const float* __restrict__ router,
                                                                const float* __restrict__ bias, int mode, int n, int C, int X,
-                                                               int top, int* __restrict__ ids, float* __restrict__ weights) {
+                                                               int top, int* __restrict__ ids, float* __restrict__ weights,
+                                                               int groups, int keep, float scale) {
   __shared__ float z_s[R][TW_MOE_MAX_EXPERTS];
-  __shared__ float score_s[R][TW_MOE_MAX_EXPERTS];   // mode 2: the softmax over all logits (z: what decides the choice)
+  __shared__ float score_s[R][TW_MOE_MAX_EXPERTS];   // mode 2: the softmax over all logits (z: what decides the choice); groups: theirs
   const int row0 = blockIdx.x * R, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const T* x[R];
 #pragma unroll
@@ -120,6 +126,47 @@ __global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(const T* __restri
     __builtin_amdgcn_wave_barrier();
     __threadfence_block();
   }
+  if (keep < groups) {
+    // the two largest logits of every group (lanes share a group where there are few), then the groups' ranks
+    const int size = X / groups;
+    int share = 1;
+    while (2 * share * groups <= 64) share *= 2;
+    for (int g0 = 0; g0 < groups; g0 += 64 / share) {
+      const int grp = g0 + lane / share;
+      float b1 = -INFINITY, b2 = -INFINITY;
+      if (grp < groups)
+        for (int e = lane % share; e < size; e += share) {
+          const float v = z[grp * size + e];
+          b2 = fmaxf(b2, fminf(b1, v));
+          b1 = fmaxf(b1, v);
+        }
+      for (int o = share / 2; o > 0; o >>= 1) {
+        const float o1 = __shfl_xor(b1, o, TW_WAVE), o2 = __shfl_xor(b2, o, TW_WAVE);
+        b2 = fmaxf(fminf(b1, o1), fmaxf(b2, o2));
+        b1 = fmaxf(b1, o1);
+      }
+      if (grp < groups && lane % share == 0)
+        score[grp] = 1.f / (1.f + expf(-b1)) + (size > 1 ? 1.f / (1.f + expf(-b2)) : 0.f);
+    }
+    __builtin_amdgcn_wave_barrier();
+    __threadfence_block();
+    unsigned kept = 0;                               // of groups lane, lane + 64, ..
+    for (int i = 0, grp = lane; grp < groups; grp += 64, ++i) {
+      const float mine = score[grp];
+      int rank = 0;
+      for (int j = 0; j < groups; ++j) rank += score[j] > mine || (score[j] == mine && j < grp) ? 1 : 0;
+      kept |= rank < keep ? 1u << i : 0u;
+    }
+    __builtin_amdgcn_wave_barrier();
+    __threadfence_block();
+    for (int i = 0, grp = lane; grp < groups; grp += 64, ++i) score[grp] = (kept >> i) & 1u ? 1.f : 0.f;
+    __builtin_amdgcn_wave_barrier();
+    __threadfence_block();
+    for (int e = lane; e < X; e += 64)
+      if (score[e / size] == 0.f) z[e] = -INFINITY;
+    __builtin_amdgcn_wave_barrier();
+    __threadfence_block();
+  }
   for (int r = 0; r < top; ++r) {
     float best = -INFINITY;
     int at = 0x7fffffff;
@@ -136,7 +183,7 @@ __global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(const T* __restri
     at = min(at, X - 1);                             // (no logit compares as the largest if all are NaN)
     if (lane == 0) {
       ids[(size_t)row * top + r] = at;
-      weights[(size_t)row * top + r] = mode == 2 ? score[at] : mode == 1 ? best : 1.f / (1.f + expf(-best));
+      weights[(size_t)row * top + r] = mode == 2 ? score[at] : mode == 1 ? best : scale / (1.f + expf(-best));
       z[at] = -INFINITY;
     }
     __builtin_amdgcn_wave_barrier();
@@ -162,15 +209,17 @@ __global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(const T* __restri
 }
 
 extern "C" int tw_moe_route(int dtype, const void* h, long ld_h, const float* router, const float* bias, int mode, int n, int C,
-                            int X, int top, int* ids, float* weights, hipStream_t stream) {
+                            int X, int top, int* ids, float* weights, int groups, int keep, float scale, hipStream_t stream) {
   TW_REQUIRE(h && router && ids && weights && n >= 0 && C > 0 && ld_h >= C && mode >= 0 && mode <= 2);
   TW_REQUIRE(X > 0 && X <= TW_MOE_MAX_EXPERTS && top > 0 && top <= X);
+  TW_REQUIRE(groups >= 1 && X % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (X / groups));
+  TW_REQUIRE(mode == 0 || (keep == groups && scale == 1.f));
   if (n == 0) return 0;
 #define TW_MOE_ROUTE(T)                                                                                                 \
   do {                                                                                                                  \
-    if (n <= 64) moe_route_kernel<T, 1, 16><<<n, 1024, 0, stream>>>((const T*)h, ld_h, router, bias, mode, n, C, X, top, ids, weights);                \
-    else if (n <= 512) moe_route_kernel<T, 1, 4><<<n, 256, 0, stream>>>((const T*)h, ld_h, router, bias, mode, n, C, X, top, ids, weights);            \
-    else moe_route_kernel<T, 4, 8><<<tw_div_up(n, 4), 512, 0, stream>>>((const T*)h, ld_h, router, bias, mode, n, C, X, top, ids, weights);            \
+    if (n <= 64) moe_route_kernel<T, 1, 16><<<n, 1024, 0, stream>>>((const T*)h, ld_h, router, bias, mode, n, C, X, top, ids, weights, groups, keep, scale); \
+    else if (n <= 512) moe_route_kernel<T, 1, 4><<<n, 256, 0, stream>>>((const T*)h, ld_h, router, bias, mode, n, C, X, top, ids, weights, groups, keep, scale); \
+    else moe_route_kernel<T, 4, 8><<<tw_div_up(n, 4), 512, 0, stream>>>((const T*)h, ld_h, router, bias, mode, n, C, X, top, ids, weights, groups, keep, scale); \
   } while (0)
   if (dtype == TW_DTYPE_BF16) TW_MOE_ROUTE(bf16_t);
   else if (dtype == TW_DTYPE_F32) TW_MOE_ROUTE(float);
@@ -266,7 +315,7 @@ __global__ __launch_bounds__(256) void moe_gather_kernel(const T* __restrict__ h
 // against every fragment of the expert's matrices it reads.
 template <int N> struct MoeCount { static constexpr int value = N; };
 // ACT 0: the float32 product; 1: gate and up with the limited swish; 2: one matrix with the exact gelu; 3: gate and up with
-// SiLU (1 to 3 write the next product's rows in the compute type).
+// SiLU; 4: one matrix with the square of relu (1 to 4 write the next product's rows in the compute type).
 // PLAN (the first product of steps of at most 64 (token, choice) pairs whose weights multiply outputs): there is no plan
 // and no gather launch. Every wave finds the tiles itself, lane i holding pair i: a pair whose expert has 16 m pairs before
 // it opens a tile, the tiles are numbered in the order of the pairs that open them, and the rows are read where they lie in
@@ -418,6 +467,7 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(const T* __restrict__ 
           const float z = acc[m][t][j];
           ((T*)out)[at] = tw_from_float<T>(ACT == 1 ? tw_swish_limited(z, acc2[m][t][j], limit)
                                                : ACT == 3 ? tw_silu(z) * acc2[m][t][j]
+                                               : ACT == 4 ? fmaxf(z, 0.f) * fmaxf(z, 0.f)
                                                : 0.5f * z * (1.f + erff(z * 0.70710678118654752f)));
         } else {
           ((float*)out)[(size_t)((tile + m) * TW_MOE_TILE + 4 * g + j) * ldo + col] = acc[m][t][j];
@@ -472,12 +522,14 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x,
   }
 }
 
-// The two grouped products of a step: kind 0 gated with the limited swish, 1 up alone with gelu, 2 gated with SiLU.
+// The two grouped products of a step: kind 0 gated with the limited swish, 1 up alone with gelu, 2 gated with SiLU, 3 up alone
+// with the square of relu.
 template <typename T, int ACT>
 static void moe_products(const T* xs, const T* gate, const T* up, const T* down, const int* tile_expert, T* act, float* ys, int C,
                          int Cd, int Fd, float limit, int tiles, bool wide, hipStream_t stream) {
-  const T* first = ACT == 2 ? up : gate;
-  const T* second = ACT == 2 ? nullptr : up;
+  constexpr bool PLAIN = ACT == 2 || ACT == 4;
+  const T* first = PLAIN ? up : gate;
+  const T* second = PLAIN ? nullptr : up;
   if (tiles <= TW_MOE_SPLITK_TILES) {
     // few rows: most tiles hold one or two rows and each streams its expert's matrices once; the waves then split K
     moe_grouped_kernel<T, ACT, 2, true><<<dim3(tiles, tw_div_up(Fd, 16 * 2)), 256, 0, stream>>>(
@@ -512,11 +564,12 @@ struct MoeStep {
 
 template <typename T, int ACT>
 static void moe_products_few(const MoeStep& s, hipStream_t stream) {
+  constexpr bool PLAIN = ACT == 2 || ACT == 4;
   // (every tile is opened by a pair of its own, and the tiles in use never exceed what a plan could need)
   const int tiles = s.n * s.top < s.capacity / TW_MOE_TILE ? s.n * s.top : s.capacity / TW_MOE_TILE;
   const MoePairs pairs{s.ids, s.n * s.top, s.top, s.X, s.ld_h, const_cast<int*>(s.tile_expert), const_cast<int*>(s.pos)};
   moe_grouped_kernel<T, ACT, 2, true, 1, true><<<dim3(tiles, tw_div_up(s.Fd, 16 * 2)), 256, 0, stream>>>(
-      (const T*)s.h, s.Cd, (const T*)(ACT == 2 ? s.up : s.gate), (const T*)(ACT == 2 ? nullptr : s.up), nullptr, s.act, s.Fd, s.Fd,
+      (const T*)s.h, s.Cd, (const T*)(PLAIN ? s.up : s.gate), (const T*)(PLAIN ? nullptr : s.up), nullptr, s.act, s.Fd, s.Fd,
       s.Cd, s.limit, pairs);
   moe_grouped_kernel<T, 0, 2, true><<<dim3(tiles, tw_div_up(s.C, 16 * 2)), 256, 0, stream>>>(
       (const T*)s.act, s.Fd, (const T*)s.down, nullptr, s.tile_expert, s.ys, s.C, s.C, s.Fd, 0.f);
@@ -532,7 +585,8 @@ template <typename T>
 static void moe_run(const MoeStep& s, hipStream_t stream) {
   if (s.few) {
     if (s.kind == 1) moe_products_few<T, 2>(s, stream);
-    else moe_products_few<T, 3>(s, stream);
+    else if (s.kind == 2) moe_products_few<T, 3>(s, stream);
+    else moe_products_few<T, 4>(s, stream);
   } else {
     moe_gather_kernel<T><<<s.capacity, 256, 0, stream>>>((const T*)s.h, s.ld_h, s.kind == 0 ? s.weights : nullptr, s.src_item,
                                                          s.tile_expert, (T*)s.xs, s.C, s.Cd, s.top);
@@ -542,9 +596,11 @@ static void moe_run(const MoeStep& s, hipStream_t stream) {
                          s.ys, s.C, s.Cd, s.Fd, s.limit, tiles, s.wide, stream)
     if (s.kind == 0) TW_MOE_PRODUCTS(1);
     else if (s.kind == 1) TW_MOE_PRODUCTS(2);
-    else TW_MOE_PRODUCTS(3);
+    else if (s.kind == 2) TW_MOE_PRODUCTS(3);
+    else TW_MOE_PRODUCTS(4);
 #undef TW_MOE_PRODUCTS
   }
+  if (!s.x) return;                                  // (whoever reads ys and pos adds them up)
   const dim3 grid(s.n, tw_div_up(s.C, 1024));
   const size_t more_stride = (size_t)s.n * s.C;
   const float* weights = s.kind == 0 ? nullptr : s.weights;
@@ -559,17 +615,18 @@ static void moe_run(const MoeStep& s, hipStream_t stream) {
 // h [n][C] (compute type) -> x [n][C] float32 += the routed experts' results. ids, weights [n * top] come from
 // tw_moe_route (ids of X and above, where the weights multiply outputs: experts that return h). Scratch: pos [n * top],
 // src_item [capacity], tile_expert [capacity / 16] (int32), xs [capacity][Cd], act [capacity][Fd] (compute type),
-// ys [capacity][C] (float32), capacity = tw_moe_capacity(n * top, X).
+// ys [capacity][C] (float32), capacity = tw_moe_capacity(n * top, X). x null: the experts' rows stay in ys, unweighted, pair i's
+// in row pos[i] (kinds whose weights multiply outputs).
 extern "C" int tw_moe_experts(int dtype, const void* h, long ld_h, const int* ids, const float* weights, int n, int top, int X,
                               const void* gate, const void* up, const void* down, int C, int Cd, int Fd, float limit,
                               int* pos, int* src_item, int* tile_expert, void* xs, void* act, float* ys, int capacity,
                               float* x, long ld_x, int kind, int accumulate, const float* more, int more_splits,
                               hipStream_t stream) {
-  TW_REQUIRE(h && ids && weights && up && down && pos && src_item && tile_expert && xs && act && ys && x);
-  TW_REQUIRE(((kind == 0 || kind == 2) && gate) || kind == 1);
+  TW_REQUIRE(h && ids && weights && up && down && pos && src_item && tile_expert && xs && act && ys && (x || (kind != 0 && !more)));
+  TW_REQUIRE(((kind == 0 || kind == 2) && gate) || kind == 1 || kind == 3);
   TW_REQUIRE(more == nullptr || more_splits > 0);
-  if (kind == 1) gate = up;            // (never read: the alignment test below wants a pointer)
-  TW_REQUIRE(n >= 0 && top > 0 && C > 0 && Cd >= C && Cd % 32 == 0 && Fd > 0 && Fd % 32 == 0 && ld_h >= C && ld_x >= C);
+  if (kind == 1 || kind == 3) gate = up;            // (never read: the alignment test below wants a pointer)
+  TW_REQUIRE(n >= 0 && top > 0 && C > 0 && Cd >= C && Cd % 32 == 0 && Fd > 0 && Fd % 32 == 0 && ld_h >= C && (!x || ld_x >= C));
   TW_REQUIRE((uintptr_t)xs % 16 == 0 && (uintptr_t)act % 16 == 0 && (uintptr_t)gate % 16 == 0 && (uintptr_t)up % 16 == 0 &&
              (uintptr_t)down % 16 == 0);
   TW_REQUIRE(dtype == TW_DTYPE_BF16 || dtype == TW_DTYPE_F32);

@@ -2,10 +2,12 @@
 //
 //   S_t = d_t S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t         (S: [D][E] per head and request, float32)
 //
-// in two forms, chosen by what the decay depends on:
+// in two forms, chosen by what the decay depends on (`act`: q, k and v pass SiLU when they are read):
 //   head     d_t is one number: delta = softplus(raw + dt_bias_h), d_t = exp(-exp(A_log_h) delta), k_t = delta * b_t and
 //            o_t += skip_h v_t: the state-space recurrence of Mamba-2 (Dao and Gu, "Transformers are SSMs"). `share` heads
 //            in a row read the same q and b (the recurrence's C and B).
+//            Or d_t is a constant of the head (`decay`), k_t as it comes: lightning attention (Qin et al., "Lightning
+//            Attention-2: A Free Lunch for Handling Unlimited Sequence Lengths in Large Language Models").
 //   channel  d_t is a diagonal matrix over the key elements, given by its logarithms (float32 rows): gated linear
 //            attention (Yang et al., "Gated Linear Attention Transformers with Hardware-Efficient Training").
 //
@@ -28,6 +30,7 @@
 
 #define LS_L 16
 #define LS_RANGE (-60.f)
+enum { LS_HEAD, LS_CHANNEL, LS_FIXED };     // what a kernel's decay is: a step's number a head, a number a key element, a head's constant
 
 struct LsArgs {
   const float* src; long ld;            // q of head h at q_col + h / share * D, k at k_col + h / share * D, v at v_col + h * E
@@ -44,6 +47,8 @@ struct LsArgs {
   float* out; long ld_out;              // [rows][H E]
   int H, D, E, Dp, Ep;
   float q_scale;
+  const float* decay;                   // head: [H] constants in (0, 1] (then raw, dt_bias, A_log are not read), or null
+  bool act;                             // q, k and v pass SiLU
   bool vec;                             // q and k of every head and row are whole 16-byte pieces
 };
 
@@ -89,6 +94,8 @@ __device__ __forceinline__ float ls_sum(float v) {
   return v;
 }
 
+__device__ __forceinline__ float ls_silu(float z) { return z / (1.f + expf(-z)); }
+
 __device__ __forceinline__ void ls_lds_barrier() {            // (loads from memory stay on their way across it)
   asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
   __builtin_amdgcn_s_barrier();
@@ -111,8 +118,9 @@ __device__ __forceinline__ f32x4 ls_four(const float* p, int d0, int D, bool vec
 // ---- token by token -------------------------------------------------------------------------------------------------
 // grid (column blocks, H, n_seqs). LPC lanes hold a value column, four key elements each; a thread holds its elements of
 // CPT columns. Decays given by their low-rank product: the workgroup's threads share out (key element, part of the rank).
-template <int LPC, int CPT, bool CHANNEL>
+template <int LPC, int CPT, int FORM>
 __global__ __launch_bounds__(256) void ls_walk_kernel(LsArgs a) {
+  constexpr bool CHANNEL = FORM == LS_CHANNEL, fixed = FORM == LS_FIXED;
   constexpr int CW = 256 / LPC;                               // columns a pass
   const int seq = a.seq0 + blockIdx.z, head = blockIdx.y;
   const int r0 = a.q_start[seq], r1 = a.q_start[seq + 1];
@@ -129,8 +137,10 @@ __global__ __launch_bounds__(256) void ls_walk_kernel(LsArgs a) {
     if (held && e < a.Ep) S[c] = __builtin_nontemporal_load(reinterpret_cast<const f32x4*>(S_mem + (size_t)e * a.Dp + d0));
   }
   const int group = head / a.share;
-  float rate = 0.f, bias = 0.f, skip = 0.f;
-  if (!CHANNEL) {
+  float rate = 0.f, bias = 0.f, skip = 0.f;                  // (a constant decay: its value, or its logarithm, in `rate`)
+  if constexpr (fixed) {
+    rate = a.decay[head];
+  } else if (!CHANNEL) {
     rate = -expf(a.A_log[head]);
     bias = a.dt_bias[head];
     skip = a.skip ? a.skip[head] : 0.f;
@@ -143,6 +153,13 @@ __global__ __launch_bounds__(256) void ls_walk_kernel(LsArgs a) {
     const float* q = row + a.q_col + (size_t)group * a.D;
     const float* k = row + a.k_col + (size_t)group * a.D;
     f32x4 qv = ls_four(q, d0, a.D, a.vec), kv = ls_four(k, d0, a.D, a.vec), dv;
+    if (fixed && a.act) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        qv[j] = ls_silu(qv[j]);
+        kv[j] = ls_silu(kv[j]);
+      }
+    }
     if constexpr (CHANNEL) {
       if (a.logs) {
         dv = ls_four(a.logs + (size_t)t * a.ld_logs + (size_t)head * a.D, d0, a.D, false);
@@ -167,6 +184,8 @@ __global__ __launch_bounds__(256) void ls_walk_kernel(LsArgs a) {
         ls_lds_barrier();
         dv = *reinterpret_cast<const f32x4*>(&decay_s[d0]);
       }
+    } else if (fixed) {
+      dv = f32x4{rate, rate, rate, rate};
     } else {
       const float step = ls_softplus(a.raw[(size_t)t * a.ld_raw + a.raw_col + head] + bias);
       const float decay = expf(rate * step);
@@ -178,7 +197,8 @@ __global__ __launch_bounds__(256) void ls_walk_kernel(LsArgs a) {
 #pragma unroll
     for (int c = 0; c < CPT; ++c) {
       const int e = e0 + c * CW;
-      const float x = e < a.E ? v[e] : 0.f;
+      float x = e < a.E ? v[e] : 0.f;
+      if (fixed && a.act) x = ls_silu(x);
       float o = 0.f;
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
@@ -200,8 +220,9 @@ __global__ __launch_bounds__(256) void ls_walk_kernel(LsArgs a) {
 // grid (slices of 64 value columns * H, segments, n_seqs). A wave owns 16 value columns; lane (r, g) = (lane % 16,
 // lane / 16) holds S[16 dt + 4 g + 0..3][its column r] for every tile dt of the key elements: the layout that is both the
 // B operand of Q S and the accumulator of K^T V. BUILD: only the segment's own state, from zero.
-template <int DT, bool CHANNEL, bool BUILD>
+template <int DT, int FORM, bool BUILD>
 __global__ __launch_bounds__(256) void ls_chunk_kernel(LsArgs a, LsSegments sg) {
+  constexpr bool CHANNEL = FORM == LS_CHANNEL, fixed = FORM == LS_FIXED;
   constexpr int DM = 16 * DT, QS = DM + 4;
   constexpr int NU = (2 * DM + 255) / 256;                    // (key element, half of the chunk) pairs a thread stages
   __shared__ __attribute__((aligned(16))) float q_s[BUILD ? 1 : LS_L][QS];
@@ -234,8 +255,10 @@ __global__ __launch_bounds__(256) void ls_chunk_kernel(LsArgs a, LsSegments sg) 
     if (!BUILD && on && t < tiles)
       S[t] = *reinterpret_cast<const f32x4*>((sg.count > 1 ? seg_state : own_state) + (size_t)e_col * a.Dp + 16 * t + 4 * g);
   }
-  float rate = 0.f, bias = 0.f, skip = 0.f;
-  if (!CHANNEL) {
+  float rate = 0.f, bias = 0.f, skip = 0.f;                  // (a constant decay: its value, or its logarithm, in `rate`)
+  if constexpr (fixed) {
+    rate = logf(a.decay[head]);
+  } else if (!CHANNEL) {
     rate = -expf(a.A_log[head]);
     bias = a.dt_bias[head];
     skip = a.skip ? a.skip[head] : 0.f;
@@ -271,7 +294,7 @@ __global__ __launch_bounds__(256) void ls_chunk_kernel(LsArgs a, LsSegments sg) 
       const int e = slice * 64 + (threadIdx.x & 15) + 16 * x;
       rv[x] = ok && e < a.E ? row[e] : 0.f;
     }
-    if (!CHANNEL && threadIdx.x < LS_L) {
+    if (!CHANNEL && !fixed && threadIdx.x < LS_L) {
       const int tt = c0 + threadIdx.x;
       rraw = tt < last ? a.raw[(size_t)tt * a.ld_raw + a.raw_col + head] : 0.f;
     }
@@ -296,6 +319,17 @@ __global__ __launch_bounds__(256) void ls_chunk_kernel(LsArgs a, LsSegments sg) 
     const bool pairs = CHANNEL && (wide_s[0] | wide_s[1] | wide_s[2] | wide_s[3]) != 0;
 
     // ---- the chunk's rows into LDS --------------------------------------------------------------------------------
+    if (fixed && a.act) {
+#pragma unroll
+      for (int u = 0; u < NU; ++u)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          if (!BUILD) rq[u][i] = ls_silu(rq[u][i]);
+          rk[u][i] = ls_silu(rk[u][i]);
+        }
+#pragma unroll
+      for (int x = 0; x < 4; ++x) rv[x] = ls_silu(rv[x]);
+    }
     if (CHANNEL) {
 #pragma unroll
       for (int u = 0; u < NU; ++u) {
@@ -356,7 +390,7 @@ __global__ __launch_bounds__(256) void ls_chunk_kernel(LsArgs a, LsSegments sg) 
       }
       if (threadIdx.x < LS_L) {                               // (one row of 16 lanes)
         const bool in = c0 + (int)threadIdx.x < last;
-        const float step = in ? ls_softplus(rraw + bias) : 0.f;
+        const float step = !in ? 0.f : fixed ? 1.f : ls_softplus(rraw + bias);
         const float lg = rate * step;
         float L = lg;
         L += ls_below<1>(L);
@@ -480,8 +514,9 @@ __global__ __launch_bounds__(256) void ls_chunk_kernel(LsArgs a, LsSegments sg) 
 
 // Segments' own states -> the states they start from, in place; the request's state goes from old to new.
 // grid (groups of four state elements / 256, H, n_seqs)
-template <bool CHANNEL>
+template <int FORM>
 __global__ __launch_bounds__(256) void ls_scan_kernel(LsArgs a, LsSegments sg) {
+  constexpr bool CHANNEL = FORM == LS_CHANNEL;
   const int head = blockIdx.y, seq = a.seq0 + blockIdx.z;
   const int rows = a.q_start[seq + 1] - a.q_start[seq];
   const size_t one = (size_t)a.Ep * a.Dp;
@@ -532,18 +567,18 @@ extern "C" long tw_linear_state_workspace_floats(int n_seqs, int max_q_len, int 
   return count > 1 ? (long)n_seqs * H * count * ((long)Ep * Dp + 2L * Dp) : 0;
 }
 
-template <bool CHANNEL>
+template <int FORM>
 static int ls_walk_launch(const LsArgs& a, int n_seqs, hipStream_t stream) {
   // few (sequence, head) pairs: two columns a thread spread a head over more workgroups; else eight
 #define LS_WALK(LPC)                                                                                                   \
   do {                                                                                                                 \
     constexpr int CW = 256 / LPC;                                                                                      \
     if ((long)n_seqs * a.H >= 512 && a.Ep >= 8 * CW)                                                                   \
-      ls_walk_kernel<LPC, 8, CHANNEL><<<dim3(tw_div_up(a.Ep, 8 * CW), a.H, n_seqs), 256, 0, stream>>>(a);              \
+      ls_walk_kernel<LPC, 8, FORM><<<dim3(tw_div_up(a.Ep, 8 * CW), a.H, n_seqs), 256, 0, stream>>>(a);              \
     else if (a.Ep >= 2 * CW)                                                                                           \
-      ls_walk_kernel<LPC, 2, CHANNEL><<<dim3(tw_div_up(a.Ep, 2 * CW), a.H, n_seqs), 256, 0, stream>>>(a);              \
+      ls_walk_kernel<LPC, 2, FORM><<<dim3(tw_div_up(a.Ep, 2 * CW), a.H, n_seqs), 256, 0, stream>>>(a);              \
     else                                                                                                               \
-      ls_walk_kernel<LPC, 1, CHANNEL><<<dim3(tw_div_up(a.Ep, CW), a.H, n_seqs), 256, 0, stream>>>(a);                  \
+      ls_walk_kernel<LPC, 1, FORM><<<dim3(tw_div_up(a.Ep, CW), a.H, n_seqs), 256, 0, stream>>>(a);                  \
   } while (0)
   if (a.Dp <= 16) LS_WALK(4);
   else if (a.Dp <= 64) LS_WALK(16);
@@ -553,47 +588,48 @@ static int ls_walk_launch(const LsArgs& a, int n_seqs, hipStream_t stream) {
   return TW_LAUNCH_RESULT();
 }
 
-template <int DT, bool CHANNEL>
+template <int DT, int FORM>
 static int ls_chunk_launch(const LsArgs& a, const LsSegments& sg, int n_seqs, hipStream_t stream) {
   const dim3 grid((unsigned)((a.Ep + 63) / 64 * a.H), (unsigned)sg.count, (unsigned)n_seqs);
   if (sg.count > 1) {
-    ls_chunk_kernel<DT, CHANNEL, true><<<grid, 256, 0, stream>>>(a, sg);
-    ls_scan_kernel<CHANNEL><<<dim3(tw_div_up((long)a.Ep * a.Dp, 1024), a.H, n_seqs), 256, 0, stream>>>(a, sg);
+    ls_chunk_kernel<DT, FORM, true><<<grid, 256, 0, stream>>>(a, sg);
+    ls_scan_kernel<FORM><<<dim3(tw_div_up((long)a.Ep * a.Dp, 1024), a.H, n_seqs), 256, 0, stream>>>(a, sg);
   }
-  ls_chunk_kernel<DT, CHANNEL, false><<<grid, 256, 0, stream>>>(a, sg);
+  ls_chunk_kernel<DT, FORM, false><<<grid, 256, 0, stream>>>(a, sg);
   return TW_LAUNCH_RESULT();
 }
 
-template <bool CHANNEL>
+template <int FORM>
 static int ls_launch(const LsArgs& a, const LsSegments& sg, int n_seqs, int walk, hipStream_t stream) {
-  if (walk) return ls_walk_launch<CHANNEL>(a, n_seqs, stream);
-  if (a.Dp <= 64) return ls_chunk_launch<4, CHANNEL>(a, sg, n_seqs, stream);
-  if (a.Dp <= 128) return ls_chunk_launch<8, CHANNEL>(a, sg, n_seqs, stream);
-  return ls_chunk_launch<16, CHANNEL>(a, sg, n_seqs, stream);
+  if (walk) return ls_walk_launch<FORM>(a, n_seqs, stream);
+  if (a.Dp <= 64) return ls_chunk_launch<4, FORM>(a, sg, n_seqs, stream);
+  if (a.Dp <= 128) return ls_chunk_launch<8, FORM>(a, sg, n_seqs, stream);
+  return ls_chunk_launch<16, FORM>(a, sg, n_seqs, stream);
 }
 
 // Sequences seq0 .. seq0 + n_seqs - 1. logs given, or, walked, what they are formed from (low, up, up_bias, tau): the
-// channel form; else the head form (raw, dt_bias, A_log; skip or null). walk != 0: token by token; else chunks, for portions
+// channel form; else the head form (raw, dt_bias, A_log; skip or null; or decay [H] alone, then act != 0 puts q, k and v through SiLU). walk != 0: token by token; else chunks, for portions
 // of up to max_q_len tokens.
 extern "C" int tw_linear_state(const float* src, long ld, int q_col, int k_col, int v_col, int share, const float* logs,
                                long ld_logs, const float* low, long ld_low, int rank, const float* up,
                                const float* up_bias, float tau, const float* raw, long ld_raw, int raw_col, const float* dt_bias,
                                const float* A_log, const float* skip, float* state, const int* q_start,
                                const int* state_slots, int seq0, int n_seqs, int max_q_len, float* out, long ld_out, int H,
-                               int D, int E, float q_scale, int walk, float* workspace, long workspace_floats,
-                               hipStream_t stream) {
-  TW_REQUIRE(src && state && q_start && state_slots && out && (logs || low || (raw && dt_bias && A_log)));
+                               int D, int E, float q_scale, const float* decay, int act, int walk, float* workspace,
+                               long workspace_floats, hipStream_t stream) {
+  TW_REQUIRE(src && state && q_start && state_slots && out && (logs || low || decay || (raw && dt_bias && A_log)));
+  TW_REQUIRE((!decay || (!logs && !low)) && (!act || decay));
   TW_REQUIRE(!low || (walk && up && up_bias && rank > 0 && ld_low >= rank && tau > 0.f));
   TW_REQUIRE(seq0 >= 0 && n_seqs >= 0 && max_q_len >= 1 && H > 0 && D > 0 && D <= 256 && E > 0 && share > 0 && H % share == 0);
   TW_REQUIRE(q_col >= 0 && k_col >= 0 && v_col >= 0 && ld >= (long)max(q_col, k_col) + (long)(H / share) * D &&
              ld >= (long)v_col + (long)H * E && ld_out >= (long)H * E);
-  TW_REQUIRE(logs ? ld_logs >= (long)H * D : low ? true : (raw_col >= 0 && ld_raw >= (long)raw_col + H));
+  TW_REQUIRE(logs ? ld_logs >= (long)H * D : (low || decay) ? true : (raw_col >= 0 && ld_raw >= (long)raw_col + H));
   TW_REQUIRE((uintptr_t)state % 16 == 0 && n_seqs <= 65535 && H <= 65535);
   if (n_seqs == 0) return 0;
   const int Dp = (D + 15) / 16 * 16, Ep = (E + 15) / 16 * 16;
   LsArgs a{src, ld, q_col, k_col, v_col, share, logs, ld_logs, low, ld_low, rank, up, up_bias, tau, raw, ld_raw, raw_col,
            dt_bias, A_log, skip, state, q_start,
-           state_slots, seq0, out, ld_out, H, D, E, Dp, Ep, q_scale,
+           state_slots, seq0, out, ld_out, H, D, E, Dp, Ep, q_scale, decay, act != 0,
            D % 4 == 0 && ld % 4 == 0 && q_col % 4 == 0 && k_col % 4 == 0 && (uintptr_t)src % 16 == 0};
   LsSegments sg{nullptr, nullptr, 0, 1};
   if (!walk) {
@@ -606,7 +642,8 @@ extern "C" int tw_linear_state(const float* src, long ld, int q_col, int k_col, 
     }
     TW_REQUIRE(sg.count <= 65535);
   }
-  return logs || low ? ls_launch<true>(a, sg, n_seqs, walk, stream) : ls_launch<false>(a, sg, n_seqs, walk, stream);
+  if (logs || low) return ls_launch<LS_CHANNEL>(a, sg, n_seqs, walk, stream);
+  return decay ? ls_launch<LS_FIXED>(a, sg, n_seqs, walk, stream) : ls_launch<LS_HEAD>(a, sg, n_seqs, walk, stream);
 }
 
 // ---- the logarithms of a channel's decay --------------------------------------------------------------------------
@@ -657,11 +694,12 @@ extern "C" int tw_decay_logs(const float* low, long ld, const float* up, const f
 
 // ---- a gate, then a norm in equal parts -----------------------------------------------------------------------------
 // out[n] = [.. u_p / sqrt(mean(u_p^2) + eps) ..] * weight over `parts` equal parts u_p of u = y * silu(gate), rounded to the
-// compute type. THREADS 256: a block a (token, part); 64: a wave.
-template <typename T, int THREADS>
+// compute type. THREADS 256: a block a (token, part); 64: a wave. AFTER: u = y, and the normed row is multiplied by
+// sigmoid(gate) and by `scale` before it is rounded.
+template <typename T, int THREADS, bool AFTER>
 __global__ __launch_bounds__(256) void gate_group_norm_kernel(const float* __restrict__ y, long ld_y, const float* __restrict__ gate,
                                                               long ld_g, const float* __restrict__ weight, T* __restrict__ out,
-                                                              long ld_out, int n, int parts, int size, float eps) {
+                                                              long ld_out, int n, int parts, int size, float eps, float scale) {
   __shared__ float lds[16];
   const long unit = (long)blockIdx.x * (256 / THREADS) + threadIdx.x / THREADS;
   if (unit >= (long)n * parts) return;                        // (a whole block or a whole wave)
@@ -673,8 +711,13 @@ __global__ __launch_bounds__(256) void gate_group_norm_kernel(const float* __res
   float kept[KEEP];
   float ss = 0.f;
   auto value = [&](int c) {
+    if (AFTER) return src[c];
     const float z = g[c];
     return src[c] * (z / (1.f + expf(-z)));
+  };
+  auto finished = [&](float v, float rinv, int c) {
+    const float r = v * rinv * weight[c0 + c];
+    return AFTER ? r * (scale / (1.f + expf(-g[c]))) : r;
   };
 #pragma unroll
   for (int i = 0; i < KEEP; ++i) {
@@ -692,28 +735,36 @@ __global__ __launch_bounds__(256) void gate_group_norm_kernel(const float* __res
 #pragma unroll
   for (int i = 0; i < KEEP; ++i) {
     const int c = lane + i * THREADS;
-    if (c < size) dst[c] = tw_from_float<T>(kept[i] * rinv * weight[c0 + c]);
+    if (c < size) dst[c] = tw_from_float<T>(finished(kept[i], rinv, c));
   }
-  for (int c = lane + KEEP * THREADS; c < size; c += THREADS) dst[c] = tw_from_float<T>(value(c) * rinv * weight[c0 + c]);
+  for (int c = lane + KEEP * THREADS; c < size; c += THREADS) dst[c] = tw_from_float<T>(finished(value(c), rinv, c));
 }
 
-template <typename T>
+template <typename T, bool AFTER>
 static void gate_group_norm_launch(const float* y, long ld_y, const float* gate, long ld_g, const float* weight, void* out,
-                                   long ld_out, int n, int parts, int size, float eps, hipStream_t stream) {
+                                   long ld_out, int n, int parts, int size, float eps, float scale, hipStream_t stream) {
   const long units = (long)n * parts;
   if (size > 512)
-    gate_group_norm_kernel<T, 256><<<(unsigned)units, 256, 0, stream>>>(y, ld_y, gate, ld_g, weight, (T*)out, ld_out, n, parts, size, eps);
+    gate_group_norm_kernel<T, 256, AFTER><<<(unsigned)units, 256, 0, stream>>>(y, ld_y, gate, ld_g, weight, (T*)out, ld_out, n, parts, size, eps, scale);
   else
-    gate_group_norm_kernel<T, 64><<<tw_div_up(units, 4), 256, 0, stream>>>(y, ld_y, gate, ld_g, weight, (T*)out, ld_out, n, parts, size, eps);
+    gate_group_norm_kernel<T, 64, AFTER><<<tw_div_up(units, 4), 256, 0, stream>>>(y, ld_y, gate, ld_g, weight, (T*)out, ld_out, n, parts, size, eps, scale);
 }
 
+// after != 0: the gate (sigmoid) and `scale` behind the norm; else the gate (SiLU) in front of it.
 extern "C" int tw_gate_group_norm(int dtype, const float* y, long ld_y, const float* gate, long ld_g, const float* weight,
-                                  void* out, long ld_out, int n, int parts, int size, float eps, hipStream_t stream) {
+                                  void* out, long ld_out, int n, int parts, int size, float eps, int after, float scale,
+                                  hipStream_t stream) {
   TW_REQUIRE(y && gate && weight && out && n >= 0 && parts > 0 && size > 0 && eps > 0.f);
   TW_REQUIRE(ld_y >= (long)parts * size && ld_g >= (long)parts * size && ld_out >= (long)parts * size);
   if (n == 0) return 0;
-  if (dtype == TW_DTYPE_BF16) gate_group_norm_launch<bf16_t>(y, ld_y, gate, ld_g, weight, out, ld_out, n, parts, size, eps, stream);
-  else if (dtype == TW_DTYPE_F32) gate_group_norm_launch<float>(y, ld_y, gate, ld_g, weight, out, ld_out, n, parts, size, eps, stream);
+#define TW_GATE_NORM(T)                                                                                                      \
+  do {                                                                                                                       \
+    if (after) gate_group_norm_launch<T, true>(y, ld_y, gate, ld_g, weight, out, ld_out, n, parts, size, eps, scale, stream);  \
+    else gate_group_norm_launch<T, false>(y, ld_y, gate, ld_g, weight, out, ld_out, n, parts, size, eps, 1.f, stream);         \
+  } while (0)
+  if (dtype == TW_DTYPE_BF16) TW_GATE_NORM(bf16_t);
+  else if (dtype == TW_DTYPE_F32) TW_GATE_NORM(float);
   else return TW_ERR_BAD_ARGUMENT;
+#undef TW_GATE_NORM
   return TW_LAUNCH_RESULT();
 }

@@ -495,3 +495,178 @@ extern "C" int tw_add_values(float* x, const float* y, long total, hipStream_t s
   add_values_kernel<<<tw_div_up(total, 256), 256, 0, stream>>>(x, y, total);
   return TW_LAUNCH_RESULT();
 }
+
+// ---- layer norms: a sublayer's result normed into the stream, and the stream normed for the next sublayer ------------
+//   x <- x + [norm1](y),  out <- norm2(x),    norm(v) = (v - mean) / sqrt(mean((v - mean)^2) + eps) * w + b
+// Every step is optional: no y (norm2 alone), no norm1 (y is added as it is), no out. y is float32 rows, or split-K partial
+// sums that are added up here in index order, and / or the rows of a token's routed experts, weighted (pair i's row is
+// pos[i]; a choice without a row adds nothing). Statistics and sums are float32; out is rounded once to the compute type.
+// rows (or null): the rows of x and y that out's rows are formed from; x then stays as it is. A block a row.
+struct LayerNormArgs {
+  float* x;
+  const float* y; long ldy;
+  const float* add; int splits; size_t add_stride;
+  const float* pair_rows; const int* pos; const float* pair_weights; int top;      // [.][hidden], [n][top], [n][top]
+  const float* w1; const float* b1;
+  const float* w2; const float* b2;
+  void* out;
+  const int* rows;
+  int hidden;
+  float eps;
+};
+
+// PER groups of four consecutive elements a thread, the row in registers.
+template <typename T, int PER>
+__global__ __launch_bounds__(1024) void layer_norm_vec4_kernel(LayerNormArgs a) {
+  __shared__ float lds[16];
+  const int row = a.rows ? a.rows[blockIdx.x] : blockIdx.x;
+  const int chunks = a.hidden / 4;
+  float* x = a.x + (size_t)row * a.hidden;
+  const bool has_y = a.y || a.add || a.top > 0;
+  f32x4 xv[PER], yv[PER];
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = threadIdx.x + i * blockDim.x;
+    xv[i] = yv[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (c < chunks) {
+      xv[i] = *reinterpret_cast<const f32x4*>(x + 4 * c);
+      if (a.add) {
+        const float* p = a.add + (size_t)row * a.hidden + 4 * c;
+#pragma unroll 8
+        for (int s = 0; s < a.splits; ++s) yv[i] += *reinterpret_cast<const f32x4*>(p + s * a.add_stride);
+      } else if (a.y) {
+        yv[i] = *reinterpret_cast<const f32x4*>(a.y + (size_t)row * a.ldy + 4 * c);
+      }
+#pragma unroll 4
+      for (int r = 0; r < a.top; ++r) {
+        const int at = a.pos[(size_t)row * a.top + r];
+        if (at >= 0) yv[i] += a.pair_weights[(size_t)row * a.top + r] * *reinterpret_cast<const f32x4*>(a.pair_rows + (size_t)at * a.hidden + 4 * c);
+      }
+    }
+  }
+  // (mean, one over the deviation) of a row in registers
+  auto statistics = [&](const f32x4 (&v)[PER], float& mean, float& rinv) {
+    float s = 0.f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) s += (v[i][0] + v[i][1]) + (v[i][2] + v[i][3]);
+    mean = tw_block_sum(s, lds) / (float)a.hidden;
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i)
+      if (threadIdx.x + i * blockDim.x < chunks) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss = __fmaf_rn(v[i][e] - mean, v[i][e] - mean, ss);
+      }
+    rinv = 1.f / sqrtf(tw_block_sum(ss, lds) / (float)a.hidden + a.eps);
+  };
+  if (has_y) {
+    float mean = 0.f, rinv = 1.f;
+    if (a.w1) statistics(yv, mean, rinv);
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int c = threadIdx.x + i * blockDim.x;
+      if (c < chunks) {
+        if (a.w1) {
+          const f32x4 w = *reinterpret_cast<const f32x4*>(a.w1 + 4 * c), b = *reinterpret_cast<const f32x4*>(a.b1 + 4 * c);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) yv[i][e] = __fmaf_rn((yv[i][e] - mean) * rinv, w[e], b[e]);
+        }
+        xv[i] += yv[i];
+        if (!a.rows) *reinterpret_cast<f32x4*>(x + 4 * c) = xv[i];
+      }
+    }
+  }
+  if (!a.out) return;
+  float mean, rinv;
+  statistics(xv, mean, rinv);
+  T* out = (T*)a.out + (size_t)blockIdx.x * a.hidden;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = threadIdx.x + i * blockDim.x;
+    if (c < chunks) {
+      const f32x4 w = *reinterpret_cast<const f32x4*>(a.w2 + 4 * c), b = *reinterpret_cast<const f32x4*>(a.b2 + 4 * c);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) out[4 * c + e] = tw_from_float<T>(__fmaf_rn((xv[i][e] - mean) * rinv, w[e], b[e]));
+    }
+  }
+}
+
+// Any row length and alignment: what a pass needs is formed anew.
+template <typename T>
+__global__ __launch_bounds__(256) void layer_norm_kernel(LayerNormArgs a) {
+  __shared__ float lds[16];
+  const int row = a.rows ? a.rows[blockIdx.x] : blockIdx.x;
+  float* x = a.x + (size_t)row * a.hidden;
+  const bool has_y = a.y || a.add || a.top > 0;
+  auto result = [&](int c) {
+    float v = 0.f;
+    if (a.add) {
+      for (int s = 0; s < a.splits; ++s) v += a.add[s * a.add_stride + (size_t)row * a.hidden + c];
+    } else if (a.y) {
+      v = a.y[(size_t)row * a.ldy + c];
+    }
+    for (int r = 0; r < a.top; ++r) {
+      const int at = a.pos[(size_t)row * a.top + r];
+      if (at >= 0) v += a.pair_weights[(size_t)row * a.top + r] * a.pair_rows[(size_t)at * a.hidden + c];
+    }
+    return v;
+  };
+  auto statistics = [&](auto value, float& mean, float& rinv) {
+    float s = 0.f, ss = 0.f;
+    for (int c = threadIdx.x; c < a.hidden; c += 256) s += value(c);
+    mean = tw_block_sum(s, lds) / (float)a.hidden;
+    for (int c = threadIdx.x; c < a.hidden; c += 256) {
+      const float d = value(c) - mean;
+      ss = __fmaf_rn(d, d, ss);
+    }
+    rinv = 1.f / sqrtf(tw_block_sum(ss, lds) / (float)a.hidden + a.eps);
+  };
+  float mean1 = 0.f, rinv1 = 1.f, mean2 = 0.f, rinv2 = 1.f;
+  if (has_y && a.w1) statistics(result, mean1, rinv1);
+  auto sum = [&](int c) {
+    if (!has_y) return x[c];
+    const float y = result(c);
+    return x[c] + (a.w1 ? __fmaf_rn((y - mean1) * rinv1, a.w1[c], a.b1[c]) : y);
+  };
+  if (a.out) statistics(sum, mean2, rinv2);
+  T* out = (T*)a.out + (size_t)blockIdx.x * a.hidden;
+  for (int c = threadIdx.x; c < a.hidden; c += 256) {
+    const float v = sum(c);
+    if (has_y && !a.rows) x[c] = v;
+    if (a.out) out[c] = tw_from_float<T>(__fmaf_rn((v - mean2) * rinv2, a.w2[c], a.b2[c]));
+  }
+}
+
+template <typename T>
+static void layer_norm_launch(const LayerNormArgs& a, int n, hipStream_t stream) {
+  auto ok = [](const void* p) { return (uintptr_t)p % 16 == 0; };            // (null is)
+  const bool vec = a.hidden % 4 == 0 && ok(a.x) && ok(a.y) && a.ldy % 4 == 0 && ok(a.add) && a.add_stride % 4 == 0 &&
+                   ok(a.pair_rows) && ok(a.w1) && ok(a.b1) && ok(a.w2) && ok(a.b2);
+  const int chunks = a.hidden / 4;
+  if (vec && chunks <= 4096) {
+    const int per = chunks <= 1024 ? 1 : chunks <= 2048 ? 2 : 4;
+    const int threads = (tw_div_up(chunks, per) + 63) / 64 * 64;
+    if (per == 1) layer_norm_vec4_kernel<T, 1><<<n, threads, 0, stream>>>(a);
+    else if (per == 2) layer_norm_vec4_kernel<T, 2><<<n, threads, 0, stream>>>(a);
+    else layer_norm_vec4_kernel<T, 4><<<n, threads, 0, stream>>>(a);
+  } else {
+    layer_norm_kernel<T><<<n, 256, 0, stream>>>(a);
+  }
+}
+
+extern "C" int tw_layer_norm(int out_dtype, float* x, const float* y, long ldy, const float* add, int splits, long add_stride,
+                             const float* pair_rows, const int* pos, const float* pair_weights, int top, const float* w1,
+                             const float* b1, const float* w2, const float* b2, void* out, const int* rows, int n_out, int hidden,
+                             float eps, hipStream_t stream) {
+  TW_REQUIRE(x && n_out >= 0 && hidden > 0 && eps > 0.f && (out || !rows) && top >= 0);
+  TW_REQUIRE((!out || (w2 && b2)) && (!w1 || b1));
+  TW_REQUIRE(!add || (splits > 0 && !y));
+  TW_REQUIRE(!y || ldy >= hidden);
+  TW_REQUIRE(top == 0 || (pair_rows && pos && pair_weights));
+  if (n_out == 0) return 0;
+  LayerNormArgs a{x, y, ldy, add, splits, (size_t)add_stride, pair_rows, pos, pair_weights, top, w1, b1, w2, b2, out, rows, hidden, eps};
+  if (out_dtype == TW_DTYPE_BF16) layer_norm_launch<bf16_t>(a, n_out, stream);
+  else if (out_dtype == TW_DTYPE_F32) layer_norm_launch<float>(a, n_out, stream);
+  else return TW_ERR_BAD_ARGUMENT;
+  return TW_LAUNCH_RESULT();
+}

@@ -337,11 +337,8 @@ class Stepper:
         return ctx, ordered, graphable
 
     def _first_positions(self, group, computed):
-        """Per sequence, the first position whose page a windowed group must still hold."""
-        window = self.cache.layout.groups[group].spec.window
-        if window is None:
-            return np.zeros_like(computed)
-        return np.maximum(0, computed - window + 1) // self.cache.page_size * self.cache.page_size
+        """Per sequence, the first position whose page a windowed or chunked group must still hold."""
+        return self.cache.layout.groups[group].spec.first_position(computed) // self.cache.page_size * self.cache.page_size
 
     # ---- HIP graphs for decode-only steps ------------------------------------------------
     def _capture(self, ctx):

@@ -21,7 +21,7 @@ _SIGNATURES = {
     "tw_upload_words": (I, [P, P, I, ctypes.POINTER(c_int), ctypes.POINTER(c_int), P]),
     "tw_embed_gather": (I, [I, P, P, P, I, I, I, P, I, P]),
     "tw_rmsnorm": (I, [I, P, P, P, P, I, I, F, P, I, L, P, P]),
-    "tw_rope_table": (I, [P, P, P, P, I, I, F, P]),
+    "tw_rope_table": (I, [P, P, P, P, P, I, I, F, P]),
     "tw_rope_kv_write": (I, [I, P, L, P, P, P, P, P, I, I, I, I, I, I, I, P, I, P, I, P]),
     "tw_silu_mul": (I, [I, P, P, I, I, P]),
     "tw_linear_workspace_bytes": (L, [I, I, I, I]),
@@ -33,10 +33,10 @@ _SIGNATURES = {
     "tw_linear_act": (I, [I, P, L, P, L, I, P, P, L, P, L, I, I, I, I, P]),
     "tw_attn_decode_splits": (I, [I, I, I, I]),
     "tw_attn_decode_workspace_floats": (L, [I, I, I, I]),
-    "tw_attn_decode": (I, [I, P, L, P, P, P, I, P, P, I, I, P, L, P, L, I, I, I, I, I, F, F, I, I, P]),
+    "tw_attn_decode": (I, [I, P, L, P, P, P, I, P, P, I, I, P, L, P, L, I, I, I, I, I, I, F, F, I, I, P, P, I, P]),
     "tw_attn_prefill_split": (I, [I, I, I, I, I, I, ctypes.POINTER(c_int), ctypes.POINTER(c_int)]),
     "tw_attn_prefill_workspace_floats": (L, [I, I, I, I]),
-    "tw_attn_prefill": (I, [I, P, L, P, P, P, I, P, P, I, I, I, P, L, P, L, I, I, I, I, I, I, I, I, I, F, F, I, P, P, P]),
+    "tw_attn_prefill": (I, [I, P, L, P, P, P, I, P, P, I, I, I, P, L, P, L, I, I, I, I, I, I, I, I, I, I, F, F, I, P, P, P, I, P]),
     "tw_attn_kept_keys": (I, [I, P, L, P, P, P, I, P, P, I, I, I, I, P, L, P, P, I, I, I, I, I, I, F, P]),
     "tw_add_table_rows": (I, [I, P, P, P, I, I, I, P, P]),
     "tw_causal_conv": (I, [I, I, P, L, P, F, P, P, F, P, P, P, P, P, P, L, P, L, I, I, I, I, P, I, P]),
@@ -70,7 +70,7 @@ _SIGNATURES = {
     "tw_scale_values": (I, [P, L, F, P]),
     "tw_delta_rule": (I, [P, L, I, I, I, P, L, I, I, P, P, P, P, P, P, L, I, I, I, I, I, I, I, I, F, P]),
     "tw_head_norm_gate": (I, [I, P, L, P, L, P, P, L, I, I, I, F, I, I, P]),
-    "tw_moe_route": (I, [I, P, L, P, P, I, I, I, I, I, P, P, P]),
+    "tw_moe_route": (I, [I, P, L, P, P, I, I, I, I, I, P, P, I, I, F, P]),
     "tw_moe_capacity": (L, [L, I]),
     "tw_moe_experts": (I, [I, P, L, P, P, I, I, I, P, P, P, I, I, I, F, P, P, P, P, P, P, I, P, L, I, I, P, I, P]),
     "tw_add_normed": (I, [I, P, P, L, P, I, L, P, P, I, I, F, F, P]),
@@ -85,9 +85,12 @@ _SIGNATURES = {
                               ctypes.POINTER(c_float), I, I, F, P]),
     "tw_add_values": (I, [P, P, L, P]),
     "tw_linear_state_workspace_floats": (L, [I, I, I, I, I]),
-    "tw_linear_state": (I, [P, L, I, I, I, I, P, L, P, L, I, P, P, F, P, L, I, P, P, P, P, P, P, I, I, I, P, L, I, I, I, F, I, P, L, P]),
+    "tw_linear_state": (I, [P, L, I, I, I, I, P, L, P, L, I, P, P, F, P, L, I, P, P, P, P, P, P, I, I, I, P, L, I, I, I, F, P, I, I, P, L, P]),
     "tw_decay_logs": (I, [P, L, P, P, F, P, L, I, I, I, P]),
-    "tw_gate_group_norm": (I, [I, P, L, P, L, P, P, L, I, I, I, F, P]),
+    "tw_gate_group_norm": (I, [I, P, L, P, L, P, P, L, I, I, I, F, I, F, P]),
+    "tw_rows_finish": (I, [I, P, L, I, L, P, I, I, I, I, I, P, P, P, P, I, I, P, L, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P]),
+    "tw_map_difference": (I, [I, P, L, P, P, L, I, I, I, I, I, F, F, F, P]),
+    "tw_layer_norm": (I, [I, P, P, L, P, I, L, P, P, P, I, P, P, P, P, P, P, I, I, F, P]),
     "tw_sampling_uniform": (F, [c_uint64, c_uint64]),
     "tw_sample_workspace_bytes": (L, [I]),
     "tw_sample_rows": (I, [P, L, I, I, P, P, P, P, P, L, P]),

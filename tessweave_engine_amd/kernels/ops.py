@@ -115,13 +115,16 @@ def rmsnorm(x, weight, eps, out, rows=None, add=None, row_scratch=None):
     return out
 
 
-def rope_table(positions, inv_freq, cos, sin, magnitude=1.0):
-    """cos/sin[n, j] of float32(positions[n]) * inv_freq[j], both times MAGNITUDE."""
+def rope_table(positions, inv_freq, cos, sin, magnitude=1.0, rest=None):
+    """cos/sin[n, j] of float32(positions[n]) * inv_freq[j], both times MAGNITUDE. rest (float32, like inv_freq): what float32
+    rounded off the frequencies; the angles are then exact to twice float32's precision."""
     n, half = positions.numel(), inv_freq.numel()
     _need(cos.is_contiguous() and sin.is_contiguous() and tuple(cos.shape) == (n, half)
           and tuple(sin.shape) == (n, half), "rotary tables must be [n, rot/2]")
+    _need(rest is None or (rest.is_contiguous() and rest.numel() == half), "the frequencies' remainders must be as many")
     check(library().tw_rope_table(_dev(positions, torch.int32, "positions"),
                                   _dev(inv_freq, torch.float32, "inv_freq"),
+                                  _dev(rest, torch.float32, "rest") if rest is not None else None,
                                   _dev(cos, torch.float32, "cos"), _dev(sin, torch.float32, "sin"),
                                   n, half, float(magnitude), _stream()), "rope_table")
 
@@ -381,7 +384,7 @@ def _check_attention(q, keys, values, block_table, q_start, kv_len, out, q_heads
     nq, wq, ldq = _rows(q, "q")
     no, wo, ldo = _rows(out, "out")
     _need(wq >= q_heads * head_dim and wo == q_heads * head_dim and no == nq, "attention q/out shapes do not agree")
-    _need(out.dtype == q.dtype == keys.dtype == values.dtype, "attention operand types differ")
+    _need(q.dtype == keys.dtype == values.dtype and out.dtype in (q.dtype, torch.float32), "attention operand types differ")
     _need(keys.dim() == 4 and keys.is_contiguous() and values.is_contiguous() and values.numel() == keys.numel(),
           "keys must be contiguous [pages, kv_heads, page_size, head_dim] and values the same size")
     _need(keys.shape[1] == kv_heads and keys.shape[3] == head_dim, "cache shape does not match the head sizes")
@@ -393,9 +396,23 @@ def _check_attention(q, keys, values, block_table, q_start, kv_len, out, q_heads
     return ldq, ldo
 
 
+def _attention_extras(q, out, q_heads, sink, gate):
+    """(sink pointer, gate pointer, is the output float32) for the attention launchers, checked."""
+    _need(sink is None or (sink.dtype == torch.float32 and sink.is_contiguous() and sink.numel() == q_heads), "sink must be float32 [q_heads]")
+    _need(gate is None or (gate.dtype == torch.float32 and gate.is_contiguous() and tuple(gate.shape) == (q.shape[0], q_heads)),
+          "gate must be float32 [rows of q, q_heads]")
+    return (_dev(sink) if sink is not None else None, _dev(gate) if gate is not None else None,
+            1 if out.dtype == torch.float32 else 0)
+
+
 def attn_decode(q, keys, values, block_table, q_start, kv_len, seq0, n_seqs, out, q_heads, kv_heads,
-                head_dim, scale, window=0, splits=1, workspace=None, generic=False, softcap=0.0):
+                head_dim, scale, window=0, splits=1, workspace=None, generic=False, softcap=0.0, chunk=0, sink=None,
+                gate=None):
     """Attention of sequences seq0..seq0+n_seqs-1, each with ONE query token, over their pages.
+
+    out may be float32 for bfloat16 operands. chunk > 0: a query sees only the keys of its own chunk of that many positions,
+    counted from the sequence's start. sink float32 [q_heads]: exp(sink_h) more in head h's softmax denominator (a score of
+    its own, not scaled, with no key and no value). gate float32 [rows of q, q_heads]: a factor on each head's result.
 
     generic=True forces the kernel that takes every type and page size (bfloat16 with
     pages of a multiple of 8 keys otherwise runs a faster kernel of its own). softcap > 0 passes the scaled
@@ -411,8 +428,8 @@ def attn_decode(q, keys, values, block_table, q_start, kv_len, seq0, n_seqs, out
                                    _dev(block_table, torch.int32, "block_table"), block_table.stride(0),
                                    _dev(q_start, torch.int32, "q_start"), _dev(kv_len, torch.int32, "kv_len"),
                                    seq0, n_seqs, _dev(out), ldo, ws_ptr, ws_floats, q_heads, kv_heads, head_dim,
-                                   keys.shape[2], int(window or 0), float(scale), float(softcap or 0.0), int(splits),
-                                   1 if generic else 0, _stream()),
+                                   keys.shape[2], int(window or 0), int(chunk or 0), float(scale), float(softcap or 0.0), int(splits),
+                                   1 if generic else 0, *_attention_extras(q, out, q_heads, sink, gate), _stream()),
           "attn_decode")
     return out
 
@@ -434,11 +451,11 @@ def attn_prefill_workspace_floats(n_tokens, q_heads, head_dim, max_chunks):
 
 def attn_prefill(q, keys, values, block_table, q_start, kv_len, seq0, n_seqs, max_q_len, out, q_heads,
                  kv_heads, head_dim, scale, window=0, generic=False, split=None, workspace=None, softcap=0.0, sink=None,
-                 stats=None):
-    """Attention of sequences seq0..seq0+n_seqs-1 with up to max_q_len query tokens each.
+                 stats=None, chunk=0, gate=None):
+    """Attention of sequences seq0..seq0+n_seqs-1 with up to max_q_len query tokens each. chunk, sink, gate and a float32
+    out: as in `attn_decode`.
 
-    sink float32 [q_heads]: exp(sink_h) more in head h's softmax denominator (a score of its own, not scaled, with
-    no key and no value). stats float32 [rows of q, q_heads, 2]: gets what each row's softmax was taken against (a scaled
+    stats float32 [rows of q, q_heads, 2]: gets what each row's softmax was taken against (a scaled
     score) and the row's sum relative to it, for `attn_kept_keys`.
 
     split = (max_chunks, kv_chunk[, tile_rows]) from attn_prefill_split with a float32 workspace of
@@ -447,7 +464,6 @@ def attn_prefill(q, keys, values, block_table, q_start, kv_len, seq0, n_seqs, ma
     """
     ldq, ldo = _check_attention(q, keys, values, block_table, q_start, kv_len, out, q_heads, kv_heads, head_dim)
     _need(seq0 + n_seqs <= kv_len.numel() and seq0 + n_seqs <= block_table.shape[0], "sequence range exceeds the metadata")
-    _need(sink is None or (sink.dtype == torch.float32 and sink.is_contiguous() and sink.numel() == q_heads), "sink must be float32 [q_heads]")
     _need(stats is None or (stats.dtype == torch.float32 and stats.is_contiguous() and stats.numel() >= q.shape[0] * q_heads * 2),
           "stats must be float32 [rows, q_heads, 2]")
     max_chunks, kv_chunk, ws_ptr, ws_floats = 1, 0, None, 0
@@ -456,14 +472,15 @@ def attn_prefill(q, keys, values, block_table, q_start, kv_len, seq0, n_seqs, ma
         max_chunks, kv_chunk = int(split[0]), int(split[1])
         _need(workspace is not None and workspace.dtype == torch.float32, "split prefill attention needs a float32 workspace")
         ws_ptr, ws_floats = _dev(workspace), workspace.numel()
+    extras = _attention_extras(q, out, q_heads, sink, gate)
     check(library().tw_attn_prefill(dtype_id(q.dtype), _dev(q), ldq, _dev(keys), _dev(values),
                                     _dev(block_table, torch.int32, "block_table"), block_table.stride(0),
                                     _dev(q_start, torch.int32, "q_start"), _dev(kv_len, torch.int32, "kv_len"),
                                     seq0, n_seqs, int(max_q_len), _dev(out), ldo, ws_ptr, ws_floats, q.shape[0],
                                     max_chunks, kv_chunk, tile_rows, q_heads, kv_heads, head_dim,
-                                    keys.shape[2], int(window or 0), float(scale), float(softcap or 0.0),
-                                    1 if generic else 0, _dev(sink) if sink is not None else None,
-                                    _dev(stats) if stats is not None else None, _stream()), "attn_prefill")
+                                    keys.shape[2], int(window or 0), int(chunk or 0), float(scale), float(softcap or 0.0),
+                                    1 if generic else 0, extras[0], _dev(stats) if stats is not None else None, *extras[1:],
+                                    _stream()), "attn_prefill")
     return out
 
 
@@ -475,7 +492,7 @@ def attn_kept_keys(q, keys, values, block_table, q_start, kv_len, seq0, n_seqs, 
     ldq, ldo = _check_attention(q, keys, values, block_table, q_start, kv_len, out, q_heads, kv_heads, head_dim)
     _need(stats.dtype == torch.float32 and stats.is_contiguous() and stats.numel() >= q.shape[0] * q_heads * 2,
           "stats must be float32 [rows, q_heads, 2]")
-    _need(row0 + n_rows <= q.shape[0] and seq0 + n_seqs <= kv_len.numel() and seq0 + n_seqs <= block_table.shape[0],
+    _need(out.dtype == q.dtype and row0 + n_rows <= q.shape[0] and seq0 + n_seqs <= kv_len.numel() and seq0 + n_seqs <= block_table.shape[0],
           "rows or sequences exceed the step")
     _need(sink is None or (sink.dtype == torch.float32 and sink.is_contiguous() and sink.numel() == q_heads), "sink must be float32 [q_heads]")
     check(library().tw_attn_kept_keys(dtype_id(q.dtype), _dev(q), ldq, _dev(keys), _dev(values),
@@ -1139,11 +1156,13 @@ MOE_MAX_EXPERTS = 1024
 MOE_WEIGHTS = {"sigmoid": 0, "softmax_chosen": 1, "softmax_all": 2}
 
 
-def moe_route(h, router, top, ids, weights, bias=None, weighting="sigmoid"):
+def moe_route(h, router, top, ids, weights, bias=None, weighting="sigmoid", groups=(1, 1), scale=1.0):
     """ids[n, top], weights[n, top]: per row of h the `top` experts with the largest router logits router @ h + bias
     (float32 products of h's values as they are; the lowest index wins a tie), and per chosen logit its sigmoid or
     ("softmax_chosen") its share of the softmax over the chosen logits alone. "softmax_all": s = softmax(router @ h), the
-    experts with the largest s + bias are chosen, their weights are their s over the chosen ones' sum (+ 1e-20)."""
+    experts with the largest s + bias are chosen, their weights are their s over the chosen ones' sum (+ 1e-20).
+    "sigmoid" alone: groups = (count, keep) cuts the experts into COUNT equal groups of neighbours, of which only the KEEP
+    with the largest sums of their two largest sigmoids can be chosen from; SCALE multiplies the weights."""
     _need(weighting in MOE_WEIGHTS, f"a router's weights are one of {sorted(MOE_WEIGHTS)}")
     n, C, ld_h = _rows(h, "h")
     X = router.shape[0]
@@ -1152,9 +1171,12 @@ def moe_route(h, router, top, ids, weights, bias=None, weighting="sigmoid"):
     _need(ids.is_contiguous() and weights.is_contiguous() and tuple(ids.shape) == (n, top) and tuple(weights.shape) == (n, top),
           "ids and weights are [n, top]")
     _need(bias is None or (bias.dtype == torch.float32 and bias.is_contiguous() and bias.numel() == X), "the router's bias is float32 [experts]")
+    count, keep = (int(v) for v in groups)
+    _need(count >= 1 and X % count == 0 and 1 <= keep <= count and top <= keep * (X // count), "the kept groups must hold `top` experts")
+    _need(weighting == "sigmoid" or (keep == count and float(scale) == 1.0), "groups and a scale go with sigmoid weights")
     check(library().tw_moe_route(dtype_id(h.dtype), _dev(h), ld_h, _dev(router), _dev(bias) if bias is not None else None,
                                  MOE_WEIGHTS[weighting], n, C, X, int(top), _dev(ids, torch.int32, "ids"),
-                                 _dev(weights, torch.float32, "weights"), _stream()), "moe_route")
+                                 _dev(weights, torch.float32, "weights"), count, keep, float(scale), _stream()), "moe_route")
     return ids, weights
 
 
@@ -1181,20 +1203,22 @@ def moe_blocked(w):
     return w.reshape(X, N16 // 16, 16, K // (4 * epf), 4, epf).permute(0, 1, 3, 4, 2, 5).contiguous().reshape(X, N16, K)
 
 
-MOE_KINDS = {"swish_limited": 0, "gelu": 1, "silu": 2}
+MOE_KINDS = {"swish_limited": 0, "gelu": 1, "silu": 2, "relu_squared": 3}
+MOE_PLAIN = ("gelu", "relu_squared")           # kinds without a gate
 
 
 def moe_experts(h, ids, weights, gate, up, down, limit, x, scratch, kind="swish_limited", accumulate=True, more=None):
     """kind "gelu" (gate None): x[n] (+)= sum over a row's chosen experts e of weights_e * down_e(gelu(up_e h[n])), the exact
     gelu; accumulate=False writes x instead of adding to it; more: float32 [splits, n, C] partial sums of something that
     belongs to the same result (a shared expert's last product), added up here as well. kind "silu": the same with
-    down_e(silu(gate_e h[n]) * (up_e h[n])); in these two kinds an id of X or above names an expert that returns h[n] itself.
+    down_e(silu(gate_e h[n]) * (up_e h[n])); kind "relu_squared" (gate None): down_e(max(up_e h[n], 0)^2). x None (and no more):
+    nothing is added up; returns (rows, pos), row pos[i] being what pair i's expert gives. In these kinds an id of X or above names an expert that returns h[n] itself.
     kind "swish_limited": x[n] += sum over a row's chosen experts e of down_e(glu(gate_e y, up_e y)), y = round(weights * h[n]), glu the
     limited swish with LIMIT. gate, up [X, Fd, Cd], down [X, C16, Fd] in h's type, zero padded (Fd, Cd: `moe_pad` of the
     sizes, C16: C rounded up to 16) and laid out by `moe_blocked`. scratch(tag, shape, dtype) hands out the step's scratch tensors."""
     n, C, ld_h = _rows(h, "h")
     top = ids.shape[1]
-    _need(kind in MOE_KINDS and (gate is None) == (kind == "gelu"), f"experts are one of {sorted(MOE_KINDS)}, all but 'gelu' with a gate")
+    _need(kind in MOE_KINDS and (gate is None) == (kind in MOE_PLAIN), f"experts are one of {sorted(MOE_KINDS)}, all but {MOE_PLAIN} with a gate")
     X, Fd, Cd = up.shape
     _need((gate is None or (gate.is_contiguous() and gate.dtype == h.dtype and tuple(gate.shape) == (X, Fd, Cd)))
           and up.is_contiguous() and down.is_contiguous() and up.dtype == down.dtype == h.dtype,
@@ -1203,8 +1227,12 @@ def moe_experts(h, ids, weights, gate, up, down, limit, x, scratch, kind="swish_
           "the experts' matrices are [X, Fd, Cd] and [X, C16, Fd]")
     _need(ids.is_contiguous() and weights.is_contiguous() and tuple(ids.shape) == (n, top) and tuple(weights.shape) == (n, top),
           "ids and weights are [n, top]")
-    nx, cx, ld_x = _rows(x, "x")
-    _need(nx == n and cx == C and x.dtype == torch.float32, "x must be float32 [n, C]")
+    ld_x = 0
+    if x is not None:
+        nx, cx, ld_x = _rows(x, "x")
+        _need(nx == n and cx == C and x.dtype == torch.float32, "x must be float32 [n, C]")
+    else:
+        _need(more is None and kind != "swish_limited", "rows left apart: no further sums, and weights on the outputs")
     if more is not None:
         _need(more.dim() == 3 and more.is_contiguous() and tuple(more.shape[1:]) == (n, C) and more.dtype == torch.float32,
               "more must be float32 [splits, n, C]")
@@ -1219,10 +1247,10 @@ def moe_experts(h, ids, weights, gate, up, down, limit, x, scratch, kind="swish_
                                    _dev(weights, torch.float32, "weights"), n, top, X, _dev(gate) if gate is not None else None,
                                    _dev(up), _dev(down), C, Cd, Fd,
                                    float(limit), _dev(pos), _dev(src_item), _dev(tile_expert), _dev(xs), _dev(act), _dev(ys),
-                                   capacity, _dev(x), ld_x, MOE_KINDS[kind], 1 if accumulate else 0,
+                                   capacity, _dev(x) if x is not None else None, ld_x, MOE_KINDS[kind], 1 if accumulate else 0,
                                    _dev(more) if more is not None else None, more.shape[0] if more is not None else 0,
                                    _stream()), "moe_experts")
-    return x
+    return x if x is not None else (ys, pos)
 
 
 # ---- a norm on a sublayer's result, output gates, convolved and normed queries and keys, the mLSTM ------------------------
@@ -1433,15 +1461,16 @@ def linear_state_workspace_floats(n_seqs, max_q_len, heads, dim, value_dim):
 
 
 def linear_state(src, q_col, k_col, v_col, state, q_start, state_slots, seq0, n_seqs, out, heads, dim, value_dim, groups=None,
-                 q_scale=1.0, logs=None, low_rank=None, raw=None, raw_col=0, dt_bias=None, A_log=None, skip=None, walk=True, max_q_len=1,
-                 workspace=None):
+                 q_scale=1.0, logs=None, low_rank=None, raw=None, raw_col=0, dt_bias=None, A_log=None, skip=None, decay=None,
+                 activation=None, walk=True, max_q_len=1, workspace=None):
     """S <- d S + k v^T, o = S^T (q_scale q) per head over sequences seq0 .. seq0 + n_seqs - 1, from and to state float32
     [requests, heads, Ep, Dp] (dim and value_dim rounded up to 16; a column of S is contiguous).
 
     src float32 [n, .]: q and k of head h at q_col / k_col + (h // (heads / groups)) * dim (groups None: one per head), v at
     v_col + h * value_dim. The decay d: logs float32 [n, >= heads * dim], its logarithm per key element, or, walked, low_rank =
     (low, up, bias, tau), what `decay_logs` forms it from (one launch less); with neither, one number a head: delta = softplus(raw[n, raw_col + h] + dt_bias_h), d = exp(-exp(A_log_h) delta), the key then is
-    delta k, and skip_h v is added to the result. out float32 [n, heads * value_dim]. walk: token by token (steps of a few
+    delta k, and skip_h v is added to the result. decay float32 [heads]: constants in (0, 1] instead, the key as it comes;
+    activation "silu" then puts q, k and v through SiLU as they are read. out float32 [n, heads * value_dim]. walk: token by token (steps of a few
     tokens a sequence), else chunks of 16 on the matrix unit for portions of up to max_q_len tokens, with a float32 workspace
     of `linear_state_workspace_floats` floats where that is not zero."""
     n, width, ld = _rows(src, "src")
@@ -1466,6 +1495,8 @@ def linear_state(src, q_col, k_col, v_col, state, q_start, state_slots, seq0, n_
         _need(walk and low.dtype == up.dtype == up_bias.dtype == torch.float32 and nl == n and up.is_contiguous()
               and tuple(up.shape) == (rank, heads * dim) and up_bias.is_contiguous() and up_bias.numel() == heads * dim and float(tau) > 0,
               "low_rank (for walked steps): low [n, rank], up [rank, heads * dim], bias [heads * dim], all float32, tau positive")
+    elif decay is not None:
+        _need(decay.dtype == torch.float32 and decay.is_contiguous() and decay.numel() == heads, "decay must be float32 [heads]")
     else:
         nr, wr, ld_raw = _rows(raw, "raw")
         _need(raw.dtype == torch.float32 and nr == n and 0 <= raw_col and raw_col + heads <= wr, "raw must be float32 rows with a column per head")
@@ -1476,7 +1507,9 @@ def linear_state(src, q_col, k_col, v_col, state, q_start, state_slots, seq0, n_
     if need:
         _need(workspace is not None and workspace.dtype == torch.float32 and workspace.is_contiguous() and workspace.numel() >= need,
               "long portions need a float32 workspace of linear_state_workspace_floats floats")
-    head = logs is None and low is None
+    _need(activation in (None, "silu") and (activation is None or decay is not None), "an activation goes with constant decays")
+    _need(decay is None or (logs is None and low is None and raw is None), "constant decays take the place of all others")
+    head = logs is None and low is None and decay is None
     check(library().tw_linear_state(_dev(src), ld, int(q_col), int(k_col), int(v_col), heads // groups,
                                     _dev(logs) if logs is not None else None, ld_logs, _dev(low) if low is not None else None, ld_low,
                                     rank, _dev(up) if low is not None else None, _dev(up_bias) if low is not None else None,
@@ -1485,7 +1518,8 @@ def linear_state(src, q_col, k_col, v_col, state, q_start, state_slots, seq0, n_
                                     _dev(skip) if head and skip is not None else None, _dev(state),
                                     _dev(q_start, torch.int32, "q_start"), _dev(state_slots, torch.int32, "state_slots"), int(seq0),
                                     int(n_seqs), max(1, int(max_q_len)), _dev(out), ld_out, int(heads), int(dim), int(value_dim),
-                                    float(q_scale), 1 if walk else 0, _dev(workspace) if need else None,
+                                    float(q_scale), _dev(decay) if decay is not None else None, 1 if activation else 0,
+                                    1 if walk else 0, _dev(workspace) if need else None,
                                     workspace.numel() if need else 0, _stream()), "linear_state")
     return out
 
@@ -1502,8 +1536,9 @@ def decay_logs(low, up, bias, tau, out):
     return out
 
 
-def gate_group_norm(y, gate, weight, out, parts, eps):
-    """out[n] = weight * (u in `parts` equal parts, each over its root mean square sqrt(mean + eps)), u = y * silu(gate); y and
+def gate_group_norm(y, gate, weight, out, parts, eps, after=False, scale=1.0):
+    """after: out[n] = scale * sigmoid(gate) * weight * (y in `parts` equal parts, each over its root mean square). Else:
+    out[n] = weight * (u in `parts` equal parts, each over its root mean square sqrt(mean + eps)), u = y * silu(gate); y and
     gate float32, weight float32 over the whole row, out of the compute type."""
     n, width, ld_y = _rows(y, "y")
     ng, wg, ld_g = _rows(gate, "gate")
@@ -1513,5 +1548,125 @@ def gate_group_norm(y, gate, weight, out, parts, eps):
     _need(parts > 0 and width % parts == 0 and weight.dtype == torch.float32 and weight.is_contiguous() and weight.numel() == width,
           "the parts must divide the row; the weight is float32 over the row")
     check(library().tw_gate_group_norm(dtype_id(out.dtype), _dev(y), ld_y, _dev(gate), ld_g, _dev(weight), _dev(out), ld_o, n,
-                                       int(parts), width // int(parts), float(eps), _stream()), "gate_group_norm")
+                                       int(parts), width // int(parts), float(eps), 1 if after else 0, float(scale), _stream()),
+          "gate_group_norm")
+    return out
+
+
+# ---- rotated queries and keys of a packed projection, two maps combined, layer norms -------------------------------------
+
+def rows_finish(src, columns, norm, q_weight, k_weight, cos, sin, q_out, keys, values, slots, gate, q_heads, kv_heads, dim,
+                value_dim, eps, maps=1, adjacent=False, value_scale=1.0, bias=None):
+    """Per token: q <- rotate(norm(q)), k <- rotate(norm(k)), v <- value_scale * v, gate <- sigmoid(g), from one projection.
+
+    src float32 [n, width], or [splits, n, width] split-K sums that are added up here (bias float32 [width], or None, is added
+    in both cases). columns = (q, k, v, g): where each begins; k (and v) None: no keys, g None: no gate. norm None, "head" (over
+    a head's dim elements, weights [dim]) or "row" (over all heads at once, weights over the row). cos, sin float32
+    [n, rot / 2]: the first rot elements of every head turn ("half" pairs, or neighbours with `adjacent`), None: no rotation.
+    maps 2: a head has two maps of dim elements, each turned by itself; its key holds them side by side, and q_out has a row of
+    2 * q_heads queries, each with zeros in the other map's place. q_out [n, q_heads * maps * dev] (dev: keys' last size), keys
+    [pages, kv_heads, page, dev], values the same number of elements, as [pages, kv_heads, dev, page]; slots[n] the token's
+    page slot (-1: not stored); gate float32 [n, q_heads]."""
+    splits, stride = 1, 0
+    rows = src
+    if src.dim() == 3:
+        _need(src.stride(2) == 1, "rows_finish: rows must be contiguous")
+        splits, stride, rows = src.shape[0], src.stride(0), src[0]
+    n, width, ld = _rows(rows, "src")
+    q_col, k_col, v_col, g_col = (-1 if c is None else int(c) for c in columns)
+    nq, wq, ld_q = _rows(q_out, "q_out")
+    _need(src.dtype == torch.float32 and nq == n and maps in (1, 2) and wq % (q_heads * maps) == 0, "rows_finish: src float32, q_out [n, q_heads * maps * dev]")
+    dev = wq // (q_heads * maps)
+    _need(q_col >= 0 and q_col + q_heads * maps * dim <= width and maps * dim <= dev, "rows_finish: columns exceed the rows")
+    page = 0
+    if k_col >= 0:
+        page = keys.shape[2]
+        _need(v_col >= 0 and k_col + kv_heads * maps * dim <= width and v_col + kv_heads * value_dim <= width and value_dim <= dev,
+              "rows_finish: columns exceed the rows")
+        _need(keys.is_contiguous() and values.is_contiguous() and keys.dtype == values.dtype == q_out.dtype
+              and tuple(keys.shape[1:]) == (kv_heads, page, dev) and values.numel() == keys.numel() and slots.numel() == n,
+              "keys [pages, kv_heads, page, dev], values as many elements, of q_out's type, and a slot per token")
+    if g_col >= 0:
+        _need(gate is not None and gate.dtype == torch.float32 and gate.is_contiguous() and tuple(gate.shape) == (n, q_heads)
+              and g_col + q_heads <= width, "gate must be float32 [n, q_heads]")
+    _need(norm in (None, "head", "row"), "norm is None, 'head' or 'row'")
+    for w, heads in ((q_weight, q_heads), (k_weight, kv_heads)) if norm else ():
+        if w is None and k_col < 0:
+            continue
+        want = dim if norm == "head" else heads * maps * dim
+        _need(w.dtype == torch.float32 and w.is_contiguous() and w.numel() == want, "the norms' weights are float32 over a head or the row")
+    rot = 0
+    if cos is not None:
+        rot = 2 * cos.shape[1]
+        _need(cos.dtype == torch.float32 == sin.dtype and cos.is_contiguous() and sin.is_contiguous() and cos.shape[0] == n
+              and sin.shape == cos.shape and rot <= dim, "cos and sin are float32 [n, rot / 2]")
+    if bias is not None:
+        _need(bias.dtype == torch.float32 and bias.is_contiguous() and bias.numel() == width, "bias must be float32 [width]")
+    opt = lambda t: _dev(t) if t is not None else None       # noqa: E731
+    check(library().tw_rows_finish(dtype_id(q_out.dtype), _dev(src), ld, splits, stride, opt(bias), q_col, k_col, v_col, g_col,
+                                   {None: 0, "head": 1, "row": 2}[norm], opt(q_weight if norm else None),
+                                   opt(k_weight if norm and k_col >= 0 else None), opt(cos), opt(sin), rot, 1 if adjacent else 0,
+                                   _dev(q_out), ld_q, _dev(keys) if k_col >= 0 else None, _dev(values) if k_col >= 0 else None,
+                                   _dev(slots, torch.int32, "slots") if k_col >= 0 else None, opt(gate if g_col >= 0 else None), n,
+                                   int(q_heads), int(kv_heads), int(maps), int(dim), int(value_dim), dev, page, float(eps),
+                                   float(value_scale), _stream()), "rows_finish")
+    return q_out
+
+
+def map_difference(src, out, heads, value_dim, weight, factor, eps, gate=None):
+    """out[n, h] = factor * gate[n, h] * d / sqrt(mean(d^2) + eps), d = a1 - weight * a2 over value_dim elements; src float32
+    [n, heads * 2 * dev] with a head's two maps side by side, out [n, heads * out_dev] in the compute type (tails of zeros)."""
+    n, w, ld = _rows(src, "src")
+    no, wo, ld_o = _rows(out, "out")
+    _need(src.dtype == torch.float32 and no == n and w % (2 * heads) == 0 and wo % heads == 0, "map_difference shapes do not agree")
+    dev, out_dev = w // (2 * heads), wo // heads
+    _need(value_dim <= min(dev, out_dev) and out_dev <= 256, "map_difference: heads of up to 256 elements")
+    _need(gate is None or (gate.dtype == torch.float32 and gate.is_contiguous() and tuple(gate.shape) == (n, heads)), "gate must be float32 [n, heads]")
+    check(library().tw_map_difference(dtype_id(out.dtype), _dev(src), ld, _dev(gate) if gate is not None else None, _dev(out), ld_o, n,
+                                      int(heads), int(value_dim), dev, out_dev, float(weight), float(factor), float(eps), _stream()),
+          "map_difference")
+    return out
+
+
+def layer_norm(x, eps, y=None, add=None, pairs=None, post=None, norm=None, out=None, rows=None):
+    """x <- x + post(y), out <- norm(x); post and norm are (weight, bias), norm(v) = (v - mean) / sqrt(mean((v - mean)^2) +
+    eps) * weight + bias; post None: y is added as it is; out None: no second norm; neither y, add nor pairs: out alone.
+
+    x float32 [n, hidden] in place; the result y: float32 [n, hidden] (rows may be strided), or add: float32
+    [splits, n, hidden] partial sums added up here; and / or pairs = (expert rows [., hidden] float32, pos int32 [n * top],
+    weights float32 [n, top]): sum_r weights[n, r] * expert rows[pos[n, r]] belongs to the result too. rows: int32 indices of
+    the rows that out's rows are formed from (x then stays as it is)."""
+    _need(x.dim() == 2 and x.is_contiguous() and x.dtype == torch.float32, "layer_norm: x must be contiguous float32 [n, hidden]")
+    n, hidden = x.shape
+    n_out = rows.numel() if rows is not None else n
+    _need(y is None or add is None, "either y or partial sums")
+    _need(rows is None or out is not None, "chosen rows are for an output")
+    ldy, splits, stride, top = 0, 0, 0, 0
+    if y is not None:
+        ny, cy, ldy = _rows(y, "y")
+        _need((ny, cy) == (n, hidden) and y.dtype == torch.float32, "y must be float32 [n, hidden]")
+    if add is not None:
+        _need(add.dim() == 3 and add.is_contiguous() and tuple(add.shape[1:]) == (n, hidden) and add.dtype == torch.float32,
+              "partial sums must be float32 [splits, n, hidden]")
+        splits, stride = add.shape[0], n * hidden
+    pair_rows = pos = pair_weights = None
+    if pairs is not None:
+        pair_rows, pos, pair_weights = pairs
+        top = pair_weights.shape[1]
+        _need(pair_rows.dtype == torch.float32 and pair_rows.is_contiguous() and pair_rows.dim() == 2 and pair_rows.shape[1] == hidden
+              and pos.dtype == torch.int32 and pos.numel() == n * top and pair_weights.dtype == torch.float32
+              and pair_weights.is_contiguous() and pair_weights.shape[0] == n, "pairs are (rows [., hidden], pos [n * top], weights [n, top])")
+    for p in (post, norm):
+        for t in p or ():
+            _need(t.dtype == torch.float32 and t.is_contiguous() and t.numel() == hidden, "norm weights and biases are float32 [hidden]")
+    out_dtype = F32
+    if out is not None:
+        _need(norm is not None and out.is_contiguous() and tuple(out.shape) == (n_out, hidden), "out must be contiguous [n, hidden], with a norm")
+        out_dtype = dtype_id(out.dtype)
+    opt = lambda t: _dev(t) if t is not None else None       # noqa: E731
+    w1, b1 = post or (None, None)
+    w2, b2 = norm if out is not None else (None, None)
+    check(library().tw_layer_norm(out_dtype, _dev(x), opt(y), ldy, opt(add), splits, stride, opt(pair_rows), opt(pos), opt(pair_weights),
+                                  top, opt(w1), opt(b1), opt(w2), opt(b2), opt(out), _dev(rows, torch.int32, "rows") if rows is not None else None,
+                                  n_out, hidden, float(eps), _stream()), "layer_norm")
     return out

@@ -5,3 +5,4 @@ from . import dinutar  # noqa: F401
 from . import rufusun  # noqa: F401
 from . import tadalorn  # noqa: F401
 from . import darolix  # noqa: F401
+from . import vulosun  # noqa: F401

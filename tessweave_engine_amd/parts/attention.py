@@ -17,31 +17,39 @@ from .linear import Linear
 import torch
 
 
-def paged_attention(ctx, q, keys, values, group, out, q_heads, kv_heads, head_dim, scale, window=0, softcap=0.0):
+TILE_TOKENS = 128          # most tokens that one tile of rows of the prompt kernel spans
+
+
+def paged_attention(ctx, q, keys, values, group, out, q_heads, kv_heads, head_dim, scale, window=0, softcap=0.0, chunk=0, sink=None,
+                    gate=None):
     """A step's causal attention over a cache group's pages: one-token sequences through the split-KV decode kernel, prompt
     portions through the prefill kernel. q [n, >= q_heads * head_dim], out [n, q_heads * head_dim]; keys and values as
-    `ctx.cache.keys_values` gives them."""
+    `ctx.cache.keys_values` gives them. chunk, sink, gate and a float32 out: see `ops.attn_decode`."""
     n = ctx.n_tokens
+    extras = dict(chunk=chunk, sink=sink, gate=gate)
+    span = window or chunk                                 # most keys a query sees (0: all before it)
     if ctx.n_decode:
         # A captured step is replayed for other lengths: its split count follows the step's length
         # class (the kernel itself cuts each sequence's own keys into that many ranges).
         longest = ctx.kv_bound if ctx.capturing else ctx.max_kv_len
-        if window:
-            longest = min(longest, window)
+        if span:
+            longest = min(longest, span)
         splits = ops.attn_decode_splits(ctx.n_decode, q_heads, kv_heads, longest)
         ws = None
         if splits > 1:
             # sized for the most splits any length class can ask for, so that it never grows under a capture
             most = max(splits, ops.attn_decode_splits(ctx.n_decode, q_heads, kv_heads,
-                                                      min(ctx.kv_capacity, window) if window else ctx.kv_capacity))
+                                                      min(ctx.kv_capacity, span) if span else ctx.kv_capacity))
             floats = ops.attn_decode_workspace_floats(ctx.n_decode, q_heads, head_dim, most)
             ws = ctx.workspace.get("attn.split", (floats,), torch.float32)
         ops.attn_decode(q, keys, values, group.block_table, ctx.q_start, ctx.kv_len, 0, ctx.n_decode, out,
                         q_heads, kv_heads, head_dim, scale, window=window,
-                        splits=splits, workspace=ws, softcap=softcap)
+                        splits=splits, workspace=ws, softcap=softcap, **extras)
     if ctx.n_seqs > ctx.n_decode:
         # long key ranges are cut into chunks for separate workgroups when there are few tiles of rows
-        longest = min(ctx.max_kv_len, window + ctx.max_q_len) if window else ctx.max_kv_len
+        longest = min(ctx.max_kv_len, span + ctx.max_q_len) if span else ctx.max_kv_len
+        if chunk:                                          # (a tile of rows sees its own tokens and what lies before them in a chunk)
+            longest = min(longest, chunk + TILE_TOKENS)
         split = ops.attn_prefill_split(ctx.n_seqs - ctx.n_decode, q_heads, kv_heads, ctx.max_q_len, longest)
         ws = None
         if split[0] > 1:
@@ -50,7 +58,7 @@ def paged_attention(ctx, q, keys, values, group, out, q_heads, kv_heads, head_di
         ops.attn_prefill(q, keys, values, group.block_table, ctx.q_start, ctx.kv_len, ctx.n_decode,
                          ctx.n_seqs - ctx.n_decode, ctx.max_q_len, out, q_heads, kv_heads,
                          head_dim, scale, window=window, split=split, workspace=ws,
-                         softcap=softcap)
+                         softcap=softcap, **extras)
     return out
 
 

@@ -20,6 +20,10 @@ import torch
 #: rounded to the compute type (in float32 runs: the stream itself), for a sublayer that reads the stream as it is
 ROUNDED_STREAM = "stream.rounded"
 
+#: key of `StepContext.shared` under which a block that has just written the residual stream may leave it NORMED for the
+#: block behind it: (the norm part it went through, rows in the compute type); only a block whose first norm is that part takes it
+NORMED_STREAM = "stream.normed"
+
 #: key of `StepContext.shared` under which an embedding that is asked to keeps its output (float32 [n, hidden]) for layer
 #: runs that add it to the stream again (`LayerRun.adds_embedding`)
 EMBEDDING_OUTPUT = "embedding.output"
@@ -134,6 +138,9 @@ class FeedForward(Part):
     #: True if `forward` takes `more`: pending partial sums (see `Mixer.forward`) of a mixer beside it, which it adds into
     #: X together with its own result
     folds_beside = False
+    #: True if `forward` takes `apart=True`: the result is not summed but left as an object with `add` (pending partial sums, or
+    #: None) and `pairs` (expert rows, their places, their weights; see `ops.layer_norm`), which the caller's norm adds up
+    leaves_apart = False
 
     def forward(self, ctx, h, x):
         """Add the feed-forward's output for normalised input H into X (float32, in place);

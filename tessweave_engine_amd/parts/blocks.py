@@ -9,7 +9,7 @@ import torch
 from ..cache.spec import CacheNeed
 from ..kernels import ops
 from ..weights.spec import AVERAGE, ONE_PLUS_NORMAL, VECTOR, TensorSpec
-from .base import ROUNDED_STREAM, Block, fold_pending
+from .base import NORMED_STREAM, ROUNDED_STREAM, Block, fold_pending
 
 
 class PreNormBlock(Block):
@@ -226,6 +226,65 @@ class ResultNormBlock(Block):
         if self.ffn is not None:
             left = self.ffn.forward(ctx, self._rounded(ctx, x), result, accumulate=False)
             self._sublayer(ctx, x, self.ffn_norm, result, left)
+        return None
+
+
+class SandwichBlock(Block):
+    """A layer norm before and after each sublayer:
+
+        x <- x + norm1b(mixer(norm1(x)));  x <- x + norm2b(ff(norm2(x)))
+
+    mixer_norms, ffn_norms: (before, after), `LayerNorm` parts of one eps. One kernel adds up a sublayer's pending split-K sums
+    (and a token's routed experts), norms the result, adds it into the stream and norms the stream for whoever reads it next:
+    the feed-forward, or the next block, whose first norm is given as `next_norm` by whoever builds the model (None: nobody).
+    ffn / ffn_norms may be None: the layer then has only the mixer. unused_names: tensors a checkpoint may hold for this layer
+    that nothing reads. The mixer and the feed-forward must take `accumulate=False`."""
+
+    def __init__(self, hidden, mixer, mixer_norms, ffn=None, ffn_norms=None, unused_names=()):
+        if (ffn is None) != (ffn_norms is None):
+            raise ValueError("a feed-forward and its norms come together")
+        self.hidden, self.mixer, self.ffn = int(hidden), mixer, ffn
+        self.mixer_norm, self.mixer_after = mixer_norms
+        self.ffn_norm, self.ffn_after = ffn_norms if ffn_norms is not None else (None, None)
+        if len({n.eps for n in (*mixer_norms, *(ffn_norms or ()))}) != 1:
+            raise ValueError("the norms of a layer share their eps")
+        self.next_norm = None
+        self.unused_names = tuple(unused_names)
+
+    def parts(self):
+        return [p for p in (self.mixer_norm, self.mixer, self.mixer_after, self.ffn_norm, self.ffn, self.ffn_after) if p is not None]
+
+    def tensor_specs(self):
+        specs = [s for p in self.parts() for s in p.tensor_specs()]
+        return specs + [TensorSpec(name, (1,), VECTOR, optional_alias_of="(unused)") for name in self.unused_names]
+
+    def bind(self, tensors, dtype, device):
+        for p in self.parts():
+            p.bind(tensors, dtype, device)
+
+    def _close(self, ctx, x, after, reader, result, left):
+        """x <- x + after(the sublayer's result); the stream normed by READER (None: nobody reads it)."""
+        add, pairs = left, None
+        if left is not None and hasattr(left, "pairs"):
+            add, pairs = left.add, left.pairs
+        y = result if add is None and (pairs is None or left.wrote) else None
+        out = ctx.scratch("norm.out", (ctx.n_tokens, self.hidden)) if reader is not None else None
+        ops.layer_norm(x, after.eps, y=y, add=add, pairs=pairs, post=after.pair, norm=reader.pair if reader is not None else None, out=out)
+        return out
+
+    def forward(self, ctx, run, x, pending=None):
+        norm, h = ctx.shared.pop(NORMED_STREAM, (None, None))
+        if norm is not self.mixer_norm or pending is not None:
+            h = normalise(self.mixer_norm, ctx, x, pending)
+        result = ctx.scratch("sublayer.result", (ctx.n_tokens, self.hidden), torch.float32)
+        left = self.mixer.forward(ctx, run, h, result, accumulate=False)
+        h = self._close(ctx, x, self.mixer_after, self.ffn_norm if self.ffn is not None else self.next_norm, result, left)
+        if self.ffn is not None:
+            options = {"apart": True} if self.ffn.leaves_apart else {}
+            left = self.ffn.forward(ctx, h, result, accumulate=False, **options)
+            h = self._close(ctx, x, self.ffn_after, self.next_norm, result, left)
+        if h is not None:
+            ctx.shared[NORMED_STREAM] = (self.next_norm, h)
         return None
 
 

@@ -14,12 +14,18 @@ down(silu(gate y) * up y); s = softmax(z) over all experts, the `top` largest of
 are its chosen s over their sum and multiply the OUTPUTS; the last `identity` experts of the router have no matrices and
 return h itself.
 
+A fourth kind (`kind="relu_squared"`, `weighting="sigmoid"`, `groups`, `weight_scale`): plain experts, expert(y) =
+down(max(up y, 0)^2); the experts stand in equal groups of neighbours, a group's score is the sum of its two largest sigmoids,
+and only experts of the best groups can be chosen; a token's weights are its chosen sigmoids times a scale, on the OUTPUTS.
+
 Experts have no biases. The experts' matrices are stacked on the device ([experts, inner, width] and [experts, width,
 inner], the reduction sizes padded to multiples of 32 with zeros, in the order the matrix unit's fragments are read:
 `ops.moe_blocked`) and all experts of a step run in two grouped
 products on the matrix unit, whose launch shapes depend on the step's rows only: nothing waits for the host.
 """
 from __future__ import annotations
+
+from collections import namedtuple
 
 import torch
 
@@ -28,15 +34,21 @@ from ..weights.spec import MATRIX, NORMAL, VECTOR, TensorSpec
 from .base import FeedForward, fold_pending
 
 
+#: a result left apart: `add` float32 [splits, n, hidden] or None, `pairs` (expert rows, places, weights), and whether a further
+#: summand was written to the result buffer
+ApartResult = namedtuple("ApartResult", "add pairs wrote")
+
+
 class RoutedExperts(FeedForward):
     folds_beside = True
 
     def __init__(self, prefix, hidden, experts, top, intermediate, limit=None, shared=None, router_name="router",
-                 expert_names=None, kind="swish_limited", weighting="sigmoid", router_bias=None, identity=0, correction=None):
+                 expert_names=None, kind="swish_limited", weighting="sigmoid", router_bias=None, identity=0, correction=None,
+                 groups=(1, 1), weight_scale=1.0):
         """shared: a `FeedForward` part that every token runs as well (or None). expert_names: the checkpoint's
         names, behind the prefix, of expert number {}'s matrices (gate, up, down; up, down for kind "gelu").
-        kind: "swish_limited" (gated, needs `limit`, weights on the experts' inputs), "gelu" (no gate, weights on the
-        outputs) or "silu" (gated, weights on the outputs); weighting: "sigmoid" of each chosen logit, "softmax_chosen" or
+        kind: "swish_limited" (gated, needs `limit`, weights on the experts' inputs), "gelu" or "relu_squared" (no gate, weights on
+        the outputs) or "silu" (gated, weights on the outputs); groups: (count, keep), weight_scale: of sigmoid weights; weighting: "sigmoid" of each chosen logit, "softmax_chosen" or
         "softmax_all"; router_bias: the checkpoint's name, behind the prefix, of a bias on the router's logits (or None);
         correction: the name of what is added to the scores of "softmax_all" for the choice alone (or None);
         identity: experts behind the others that return their input (kinds whose weights multiply outputs)."""
@@ -45,7 +57,14 @@ class RoutedExperts(FeedForward):
         if kind not in ops.MOE_KINDS or weighting not in ops.MOE_WEIGHTS:
             raise ValueError(f"experts are one of {sorted(ops.MOE_KINDS)}, their weights one of {sorted(ops.MOE_WEIGHTS)}")
         self.kind, self.weighting, self.identity = kind, weighting, int(identity)
-        self.gated = kind != "gelu"
+        self.gated = kind not in ops.MOE_PLAIN
+        self.leaves_apart = kind != "swish_limited" and not self.identity
+        self.groups, self.weight_scale = (int(groups[0]), int(groups[1])), float(weight_scale)
+        count, keep = self.groups
+        if not (1 <= keep <= count) or self.experts % count or self.top > keep * (self.experts // count):
+            raise ValueError("the groups must be equal, and those kept must hold `top` experts")
+        if weighting != "sigmoid" and (keep != count or self.weight_scale != 1.0):
+            raise ValueError("groups and a scale of the weights go with sigmoid weights")
         self.choices = self.experts + self.identity          # what the router scores
         if self.identity < 0 or (self.identity and kind == "swish_limited"):
             raise ValueError("identity experts go with weights on the experts' outputs")
@@ -106,7 +125,9 @@ class RoutedExperts(FeedForward):
         """Bytes of one expert's three matrices on the device."""
         return sum(t[0].numel() * t.element_size() for t in (self.gate, self.up, self.down) if t is not None)
 
-    def forward(self, ctx, h, x, accumulate=True, more=None):
+    def forward(self, ctx, h, x, accumulate=True, more=None, apart=False):
+        """apart (with accumulate=False): the experts' rows are not added up but left, with the shared expert's sums, as an
+        `ApartResult` for the caller's norm."""
         n = h.shape[0]
         # (with accumulate=False the shared expert writes x and the routed ones add to it, or it leaves the split-K sums of
         # its last product pending and the kernel that adds up a token's experts adds those too)
@@ -119,13 +140,17 @@ class RoutedExperts(FeedForward):
                 fold_pending(x, more)                        # (a shared expert left sums of its own: plain operations)
         ids = ctx.scratch("moe.ids", (n, self.top), torch.int32)
         weights = ctx.scratch("moe.weights", (n, self.top), torch.float32)
-        ops.moe_route(h, self.router, self.top, ids, weights, bias=self.router_bias, weighting=self.weighting)
+        ops.moe_route(h, self.router, self.top, ids, weights, bias=self.router_bias, weighting=self.weighting,
+                      groups=self.groups, scale=self.weight_scale)
 
         def scratch(tag, shape, dtype):
             # sized for the largest step: `capacity` rows for max_tokens rows of the stream
             most = ops.moe_capacity(ctx.max_tokens * self.top, self.experts)
             rows = {"moe.pos": ctx.max_tokens * self.top, "moe.tiles": most // 16}.get(tag, most)
             return ctx.workspace.get(f"{tag}.{self.top}.{self.experts}", shape, dtype, capacity=rows)
+        if apart:
+            rows, pos = ops.moe_experts(h, ids, weights, self.gate, self.up, self.down, self.limit, None, scratch, kind=self.kind)
+            return ApartResult(pending, (rows, pos, weights), wrote)
         ops.moe_experts(h, ids, weights, self.gate, self.up, self.down, self.limit, x, scratch, kind=self.kind,
                         accumulate=accumulate or wrote, more=pending)
         return None

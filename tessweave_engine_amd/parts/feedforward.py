@@ -95,6 +95,8 @@ class GatedFeedForward(FeedForward):
                 raise ValueError("silu with an output scale needs an intermediate size that is a multiple of 16")
             else:
                 ops.gelu_mul(gu, act, self.out_scale)
+        if not accumulate and ctx.defer_sums and self.down.deferrable(n):
+            return self.down.forward_partials(ctx, act, "down")          # the caller's norm adds them up
         self.down.forward(ctx, act, x, residual=x if accumulate else None)
         return None
 

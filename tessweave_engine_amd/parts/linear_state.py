@@ -13,6 +13,12 @@ branches of a `ParallelMixer`:
     q = W_q h * dim^-1/2, k = W_k h, v = W_v h;  log a = log sigmoid(W_up (W_low h) + b) / tau     (per head and key element)
     S <- diag(a) S + k v^T,  o = S^T q;   out = W_o [ .. norm_weight * unit(o_h) .. ] * silu(W_g h)
 
+`LightningAttention` (Qin et al., "Lightning Attention-2: A Free Lunch for Handling Unlimited Sequence Lengths in Large Language
+Models"), another branch:
+
+    q = silu(W_q h), k = silu(W_k h), v = silu(W_v h);  S <- decay_h S + k v^T,  o = S^T q          (decays: constants)
+    out = W_o ( norm_weight * unit(o over all heads) * sigmoid(W_g h) )
+
 The state S (and the convolution's last inputs) are float32 states of the cache slot, zero when a request opens. The
 packed products leave float32 rows; convolution, decays, states, norms and all products with a state are float32 in both
 precisions. One-token (and few-token) sequences are walked token by token, longer portions run in chunks on the matrix
@@ -186,3 +192,55 @@ class GatedLinearAttention(MixerBranch):
         run_linear_state(ctx, proj, ctx.cache.states[run.cache_slot][self.STATE], o, H, D, E, q_col=q, k_col=k, v_col=v,
                          q_scale=D ** -0.5, **decays)
         ops.head_norm_gate(o, proj[:, g:g + H * E], self.norm_weight, out, H, E, self.eps)
+
+
+class LightningAttention(MixerBranch):
+    STATE = "lightning_attention.s"
+
+    def __init__(self, prefix, heads, dim, value_dim, decay, eps, names=("q", "k", "v", "g", "norm", "o")):
+        """decay: one constant per head, in (0, 1]; eps: of the norm over all heads."""
+        if not 1 <= int(dim) <= MAX_KEY:
+            raise ValueError(f"the recurrence's kernels take keys of up to {MAX_KEY} elements")
+        self.decays = [float(d) for d in decay]
+        if len(self.decays) != int(heads) or not all(0.0 < d <= 1.0 for d in self.decays):
+            raise ValueError("one decay in (0, 1] per head is needed")
+        self.heads, self.dim, self.value_dim, self.eps = int(heads), int(dim), int(value_dim), float(eps)
+        self.names = [prefix + n for n in names]
+        self.norm_name, self.o_name = self.names[4:]
+        self.decay = self.norm_weight = None
+        H, D, E = self.heads, self.dim, self.value_dim
+        self.rows = [H * D, H * D, H * E, H * E]
+        self.columns, at = [], 0
+        for rows in self.rows:                                   # (every matrix's columns begin 16-byte aligned)
+            self.columns.append(at)
+            at += _round_up(rows, 4)
+        self.inner, self.inner_dev = H * E, _round_up(H * E, 8)  # (rows of the output product's input stay 16-byte aligned)
+
+    def in_matrices(self):
+        return [(name, rows, False, (rows, _round_up(rows, 4))) for name, rows in zip(self.names, self.rows)]
+
+    def out_matrix(self):
+        return (self.o_name, self.inner, (self.inner, self.inner_dev))
+
+    def tensor_specs(self):
+        return [TensorSpec(self.norm_name, (self.inner,), VECTOR, ONE_PLUS_NORMAL)]
+
+    def bind(self, tensors, dtype, device):
+        self.norm_weight = tensors.pop(self.norm_name).contiguous()
+        self.decay = torch.tensor(self.decays, dtype=torch.float32, device=device)        # constants of the configuration
+
+    def weight_tensors(self):
+        return [self.norm_weight]
+
+    def cache_need(self):
+        return CacheNeed(states=((self.STATE, state_need(self.heads, self.dim, self.value_dim)),))
+
+    def forward(self, ctx, run, proj, out, scale):
+        n, H, D, E = ctx.n_tokens, self.heads, self.dim, self.value_dim
+        q, k, v, g = self.columns
+        o = ctx.scratch("lightning_attention.o", (n, H * E), torch.float32)
+        run_linear_state(ctx, proj, ctx.cache.states[run.cache_slot][self.STATE], o, H, D, E, q_col=q, k_col=k, v_col=v,
+                         decay=self.decay, activation="silu")
+        if self.inner_dev != self.inner:
+            out[:, self.inner:].zero_()                          # (meets zero columns, but must not hold NaN)
+        ops.gate_group_norm(o, proj[:, g:g + self.inner], self.norm_weight, out[:, :self.inner], 1, self.eps, after=True, scale=scale)

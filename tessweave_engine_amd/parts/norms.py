@@ -1,4 +1,4 @@
-"""RMS norm: y = x * rsqrt(mean(x^2) + eps) * weight (flow_engine/model.py:15-23).
+"""Norms of the residual stream. RMS norm: y = x * rsqrt(mean(x^2) + eps) * weight (flow_engine/model.py:15-23).
 
 The residual stream it reads is float32; statistics and products are float32
 and the result is rounded once to the compute type. The weight is held in
@@ -44,3 +44,32 @@ class RMSNorm(Norm):
             import torch
             scratch = ctx.scratch(tag + ".rows", (n_out, self.size), torch.float32)
         return ops.rmsnorm(x, self.weight, self.eps, out, rows=rows, add=add, row_scratch=scratch)
+
+
+class LayerNorm(Norm):
+    """y = (x - mean) / sqrt(mean((x - mean)^2) + eps) * weight + bias, in float32, rounded once to the compute type."""
+    folds_pending = True
+
+    def __init__(self, name, size, eps, suffixes=(".weight", ".bias")):
+        self.name, self.suffixes = name, tuple(suffixes)         # what follows the name in the checkpoint
+        self.size, self.eps = int(size), float(eps)
+        self.weight = self.bias = None
+
+    def tensor_specs(self):
+        w, b = (self.name + s for s in self.suffixes)
+        return [TensorSpec(w, (self.size,), VECTOR, ONE_PLUS_NORMAL), TensorSpec(b, (self.size,), VECTOR, NORMAL)]
+
+    def bind(self, tensors, dtype, device):
+        self.weight, self.bias = (tensors.pop(self.name + s).contiguous() for s in self.suffixes)
+
+    def weight_tensors(self):
+        return [self.weight, self.bias]
+
+    @property
+    def pair(self):
+        return self.weight, self.bias
+
+    def forward(self, ctx, x, rows=None, add=None):
+        tag = "norm.out" if rows is None else "norm.rows"        # a model's last norm (chosen rows) keeps its own buffer
+        out = ctx.scratch(tag, (rows.numel() if rows is not None else x.shape[0], self.size))
+        return ops.layer_norm(x, self.eps, add=add, norm=self.pair, out=out, rows=rows)

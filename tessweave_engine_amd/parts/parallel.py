@@ -1,6 +1,6 @@
 """Mixers that run side by side on one input, and the two kinds of branch built here.
 
-`ParallelMixer` reads h once: the input matrices of all its branches are one packed product, each branch
+`ParallelMixer` reads h once: the input matrices of all its branches (or of its one branch) are one packed product, each branch
 works on its own columns of the result, writes its output (times its weight in the sum, times the
 block's residual multiplier) into its own columns of one buffer, and ONE joined output product adds
 sum_b scale_b * W_o,b out_b into the residual stream. With a norm on each branch's RESULT
@@ -39,7 +39,12 @@ class MixerBranch(Part):
     out_matrix():   (checkpoint name, columns, (unit, to) padding of the columns or None)
     forward(ctx, run, proj, out, scale): proj holds this branch's columns of the packed input product,
     out its columns of the joined output product's input; writes scale * (the branch's result) there.
+
+    takes_partials: proj may also be float32 [splits, n, columns] split-K sums of the product (a view into those of all
+    branches), which the branch adds up itself, with `bias` (float32 [columns], or None) then given apart. (Without, a
+    bias is in proj already, and `bias` is not given.)
     """
+    takes_partials = False
 
     def in_matrices(self):
         raise NotImplementedError
@@ -281,11 +286,28 @@ class ParallelMixer(Mixer):
             need = need.merged(b.cache_need())
         return need
 
-    def forward(self, ctx, run, h, x):
+    def _results(self, ctx, run, h, joined):
+        """Every branch's result into its columns of JOINED."""
         n = ctx.n_tokens
-        proj = ctx.scratch("parallel.proj", (n, sum(self.proj.device_out)), self.proj_dtype)
-        self.proj.forward(ctx, h, proj)
+        if n <= 64 and self.proj_dtype == torch.float32 and all(b.takes_partials for b in self.branches) and self.proj.deferrable(n):
+            proj = self.proj.forward_partials(ctx, h, "parallel")
+            bias = self.proj.biases[0] if self.proj.biases else None
+            extra = [dict(bias=bias[c0:c0 + w] if bias is not None else None) for c0, w in self.in_columns]
+        else:
+            proj = ctx.scratch("parallel.proj", (n, sum(self.proj.device_out)), self.proj_dtype)
+            self.proj.forward(ctx, h, proj)
+            extra = [{} for _ in self.branches]
+        for b, (c0, w), (o0, ow), scale, more in zip(self.branches, self.in_columns, self.out_columns, self.scales, extra):
+            b.forward(ctx, run, proj[..., c0:c0 + w], joined[:, o0:o0 + ow], scale, **more)
+
+    def forward(self, ctx, run, h, x, accumulate=True):
+        """accumulate=False: the sum alone is written to x, or left as pending partial sums (mixers without result norms)."""
+        n = ctx.n_tokens
         if self.result_norms:
+            if not accumulate:
+                raise ValueError("a mixer with result norms adds into the stream itself")
+            proj = ctx.scratch("parallel.proj", (n, sum(self.proj.device_out)), self.proj_dtype)
+            self.proj.forward(ctx, h, proj)
             results = []
             for i, (b, out, norm) in enumerate(zip(self.branches, self.outs, self.result_norms)):
                 c0, w = self.in_columns[i]
@@ -299,7 +321,8 @@ class ParallelMixer(Mixer):
             ops.add_normed_sum(x, results, self.result_norms[0].eps)
             return None
         joined = ctx.scratch("parallel.out", (n, self.out.device_in))
-        for b, (c0, w), (o0, ow), scale in zip(self.branches, self.in_columns, self.out_columns, self.scales):
-            b.forward(ctx, run, proj[:, c0:c0 + w], joined[:, o0:o0 + ow], scale)
-        self.out.forward(ctx, joined, x, residual=x)
+        self._results(ctx, run, h, joined)
+        if not accumulate and ctx.defer_sums and self.out.deferrable(n):
+            return self.out.forward_partials(ctx, joined, "o")          # whoever norms next adds them up
+        self.out.forward(ctx, joined, x, residual=x if accumulate else None)
         return None

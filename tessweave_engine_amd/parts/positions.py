@@ -13,6 +13,9 @@ hi = min(ceil(pair(slow)), rot - 1) and ramp_j = clamp((j - lo) / max(hi - lo, 0
 pair j turns with inv_freq[j] * (ramp_j / factor + 1 - ramp_j): pairs that turn
 often within the original context keep their frequency, slow ones are divided by
 the factor; cos and sin are both multiplied by 0.1 ln(factor) + 1.
+
+`divide` = factor divides every frequency (linear scaling; 1.0: none). Frequencies are then formed in float64 and kept
+as a float32 and what that rounded off, and the tables carry the angles' rounding errors: exact to float32 at any position.
 """
 from __future__ import annotations
 
@@ -25,7 +28,7 @@ from .base import PositionEncoding
 
 
 class RotaryEmbedding(PositionEncoding):
-    def __init__(self, head_dim, theta, rotary_dim=None, pairing="half", stretch=None):
+    def __init__(self, head_dim, theta, rotary_dim=None, pairing="half", stretch=None, divide=None):
         if pairing not in ("half", "adjacent"):
             raise ValueError("pairing must be 'half' or 'adjacent'")
         self.pairing = pairing
@@ -38,11 +41,16 @@ class RotaryEmbedding(PositionEncoding):
         if self.stretch and (len(self.stretch) != 4 or self.stretch[0] <= 0 or min(self.stretch[1:]) <= 0 or self.theta <= 1):
             raise ValueError("stretch is (factor, original context, fast, slow), all positive, with theta > 1")
         self.magnitude = 0.1 * math.log(self.stretch[0]) + 1.0 if self.stretch else 1.0
-        self.inv_freq = None
+        self.divide = float(divide) if divide is not None else None
+        if self.divide is not None and (self.stretch or not self.divide > 0):
+            raise ValueError("divide must be positive and takes the place of a stretch")
+        self.inv_freq = self.rest = None
 
     def frequencies(self):
         """The pairs' frequencies, float32 [rotary_dim / 2] on the host."""
         rot = self.rotary_dim
+        if self.divide is not None:
+            return self._exact_frequencies().to(torch.float32)
         if not self.stretch:
             return self.theta ** (-torch.arange(0, rot, 2, dtype=torch.float32) / rot)
         factor, original, fast, slow = self.stretch
@@ -55,8 +63,14 @@ class RotaryEmbedding(PositionEncoding):
         ramp = ((j - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
         return (inv / factor * ramp + inv * (1.0 - ramp)).to(torch.float32)
 
+    def _exact_frequencies(self):
+        return self.theta ** (-torch.arange(0, self.rotary_dim, 2, dtype=torch.float64) / self.rotary_dim) / self.divide
+
     def bind(self, tensors, dtype, device):
-        self.inv_freq = self.frequencies().to(device)          # a constant the tables are derived from, not a weight
+        freq = self.frequencies()
+        self.inv_freq = freq.to(device)          # a constant the tables are derived from, not a weight
+        if self.divide is not None:
+            self.rest = (self._exact_frequencies() - freq.double()).to(torch.float32).to(device)
 
     def tables(self, ctx):
         """(cos, sin), float32 [n_tokens, rotary_dim / 2], computed once per step."""
@@ -66,7 +80,7 @@ class RotaryEmbedding(PositionEncoding):
             half = self.rotary_dim // 2
             cos = ctx.scratch(f"rotary.cos.{id(self)}", (ctx.n_tokens, half), torch.float32)
             sin = ctx.scratch(f"rotary.sin.{id(self)}", (ctx.n_tokens, half), torch.float32)
-            ops.rope_table(ctx.positions[0], self.inv_freq, cos, sin, self.magnitude)
+            ops.rope_table(ctx.positions[0], self.inv_freq, cos, sin, self.magnitude, rest=self.rest)
             hit = ctx.shared[key] = (cos, sin)
         return hit
 
