@@ -19,7 +19,7 @@ as the weights; `prefill_32k_prompts`: tokens a second over those prompts, which
 go through in portions of 2,048); and 1,024-token prompts with 512 generated tokens at batch 1, 8 and 64
 (`gen512_b*`, decoded tokens a second over the generated part).
 
-Other sizes of the architecture: --shape 14b|32b. --design kanavik|dinutar|rufusun|tadalorn|darolix measures that
+Other sizes of the architecture: --shape 14b|32b. --design kanavik|dinutar|rufusun|tadalorn|darolix|vulosun measures that
 design's prefill and decode at a few layer sizes, each beside the Qwen2 decoder at equal
 width, heads, feed-forward and depth (one JSON line a size). --serve measures continuous
 batching under Poisson arrivals instead (prompts of 128..4,096 tokens, 256
@@ -89,7 +89,7 @@ def parse():
                    help="with --serve: the largest prompt portion in one step (larger: more prompt tokens a second and "
                         "a shorter time to the first token, longer steps for the requests that are decoding)")
     p.add_argument("--rate", type=float, default=16.0, help="mean arrivals a second (0: all at once)")
-    p.add_argument("--design", default="", choices=["", "kanavik", "dinutar", "rufusun", "tadalorn", "darolix"],
+    p.add_argument("--design", default="", choices=["", "kanavik", "dinutar", "rufusun", "tadalorn", "darolix", "vulosun"],
                    help="instead: prefill and decode throughput of another design at a few layer sizes (--design-sizes), "
                         "each beside the Qwen2 decoder at equal width, heads, feed-forward and depth; one JSON line a size")
     p.add_argument("--design-sizes", default="1b,3b,7b", help="which of the design's sizes to run, comma separated")
@@ -213,6 +213,32 @@ def darolix_config(size, layers, context):
             "embedding": {"scale": width ** 0.5}, "layers": out}
 
 
+# The Vulosun design at those widths: layers in the order differential attention, side by side, attention, differential
+# attention that reads the first one's keys and values; the first with a dense feed-forward and the others with routed experts
+# (16 of a quarter of the dense inner size in four groups of which two are kept, two a token, beside a shared expert of that
+# size, as in the Tadalorn run, which is measured beside it). Differential attention: half the size's heads and key heads, two
+# maps of half the head size, values of the head size, chunks of the size's window. Side by side: attention with the size's
+# heads and key heads (rotation over half of a head, sinks), lightning attention with the size's heads, keys of half the head
+# size and values of the head size (the linear attention of the Darolix run).
+def vulosun_config(size, layers, context):
+    width, heads, kv_heads, dim, ff, window = DESIGN_SIZES[size]
+    dense = {"kind": "dense", "ff": ff}
+    routed = {"kind": "moe", "router": {"experts": 16, "top": 2, "scale": 1.5, "groups": {"count": 4, "keep": 2}},
+              "expert": {"ff": ff // 4}, "shared": {"ff": ff // 4}}
+    plain = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5}
+    decay = [1.0 - 2.0 ** (-3 - 6 * h / max(1, heads - 1)) for h in range(heads)]
+    beside = {"left": dict(plain, rot={"base": 1e6, "dims": dim // 2}), "left_scale": 0.8,
+              "right": {"heads": heads, "dim": dim // 2, "vdim": dim, "decay": decay}, "right_scale": 0.5}
+    maps = {"heads": heads // 2, "kv_heads": kv_heads // 2, "dim": dim // 2, "vdim": dim, "scale": (dim // 2) ** -0.5, "diff": 0.3,
+            "mask": {"size": window}, "rot": {"base": 50000.0, "dims": dim // 2, "scaling": {"factor": 4.0}}}
+    out = []
+    for i in range(layers):
+        mixer, kind = {0: (maps, "attention_2"), 1: (beside, "parallel"), 2: (dict(plain, rot={"base": 1e6, "dims": dim}), "attention"),
+                       3: (dict(maps, kv_from=i - 3), "attention_2")}[i % 4]
+        out.append({"type": kind, "mixer": mixer, "mlp": routed if i % 4 else dense})
+    return {"architecture": "Vulosun", "vocab": DESIGN_VOCAB, "width": width, "norm": {"eps": 1e-6}, "layers": out}
+
+
 def qwen2_config_like(size, layers, context):
     width, heads, kv_heads, dim, ff, _ = DESIGN_SIZES[size]
     return dict(QWEN25_7B, num_hidden_layers=layers, hidden_size=width, num_attention_heads=heads,
@@ -234,11 +260,14 @@ def design_run(args, torch):
                 "batch": args.batch, "context": args.context, "prefill_tokens": args.prefill_tokens,
                 "data": "synthetic: uniform-random token ids, random weights"}
         make = {"kanavik": kanavik_config, "dinutar": dinutar_config, "rufusun": rufusun_config,
-                "tadalorn": tadalorn_config, "darolix": darolix_config}[args.design]
+                "tadalorn": tadalorn_config, "darolix": darolix_config, "vulosun": vulosun_config}[args.design]
         models = [(args.design, make(size, args.design_layers, args.context))]
         if not args.design_only:
             if args.design in ("tadalorn", "darolix"):          # the closest design of the engine (experts, a recurrence, attention)
                 models.append(("rufusun", rufusun_config(size, args.design_layers, args.context)))
+            if args.design == "vulosun":
+                models.append(("tadalorn", tadalorn_config(size, args.design_layers, args.context)))
+                models.append(("darolix", darolix_config(size, args.design_layers, args.context)))
             models.append(("qwen2", qwen2_config_like(size, args.design_layers, args.context)))
         for name, cfg in models:
             model = random_model(config_from_dict(cfg), args.seed, dtype=args.dtype, device="cuda:0")

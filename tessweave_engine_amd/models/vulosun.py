@@ -73,7 +73,7 @@ def _check_attention(m, where, i, maps=1):
         raise ConfigError(f"layer {i}: heads must be a multiple of kv_heads")
     if max(maps * m["dim"], m["vdim"]) > MAX_HEAD:
         raise ConfigError(f"layer {i}: the attention kernels take keys (all maps of a head together) and values of up to {MAX_HEAD} elements")
-    _number(_need(m, "scale", where), f"layer {i}: scale")
+    _positive_float(_need(m, "scale", where), f"layer {i}: scale")
     rot = _need(m, "rot", where)
     dims = _positive(_need(rot, "dims", where + "rot."), f"layer {i}: rot.dims")
     if dims % 2 or dims > m["dim"]:
