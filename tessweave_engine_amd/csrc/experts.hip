@@ -284,24 +284,36 @@ extern "C" int tw_moe_plan(const int* ids, int items, int X, int* pos, int* src_
 }
 
 // ---- gather: xs[row] = round(weight * h[token]) in the experts' order, zeros in padding rows and behind C ----------
+// A workgroup takes a tile's 16 rows and every gridDim.y-th group of 16 pieces of them: a thread a (row, piece), so that what
+// a wave writes is consecutive (xs lies in fragment order).
 template <typename T>
 __global__ __launch_bounds__(256) void moe_gather_kernel(const T* __restrict__ h, long ld_h, const float* __restrict__ weights,
                                                          const int* __restrict__ src_item, const int* __restrict__ tile_expert,
                                                          T* __restrict__ xs, int C, int Cd, int top) {
-  const int row = blockIdx.x;
-  if (tile_expert[row / TW_MOE_TILE] < 0) return;
-  const int item = src_item[row];
+  const int tile = blockIdx.x;
+  if (tile_expert[tile] < 0) return;
   constexpr int EPF = Elem<T>::kPerFrag;
-  // element c of the row: tile row / 16, step c / (4 EPF), piece c / EPF % 4, row row % 16 of the piece
-  T* dst = xs + (size_t)(row / TW_MOE_TILE) * Cd * TW_MOE_TILE + (row % TW_MOE_TILE) * EPF;
-  auto at = [](int c) { return (size_t)(c / EPF) * TW_MOE_TILE * EPF + c % EPF; };
-  if (item < 0) {
-    for (int c = threadIdx.x; c < Cd; c += blockDim.x) dst[at(c)] = tw_from_float<T>(0.f);
-    return;
+  const int r = threadIdx.x % TW_MOE_TILE;
+  const int item = src_item[tile * TW_MOE_TILE + r];
+  const float w = weights && item >= 0 ? weights[item] : 1.f;             // (no weights: they multiply the experts' outputs instead)
+  const T* src = h + (item >= 0 ? (size_t)(item / top) * ld_h : 0);
+  const bool vec = !weights && ld_h % EPF == 0 && (uintptr_t)h % 16 == 0;
+  T* dst = xs + (size_t)tile * Cd * TW_MOE_TILE;
+#pragma unroll 4
+  for (int p = threadIdx.x / TW_MOE_TILE + 16 * blockIdx.y; p < Cd / EPF; p += 16 * gridDim.y) {
+    typename Elem<T>::Frag v = Elem<T>::zero();
+    const int c = p * EPF;
+    if (item >= 0) {
+      if (vec && c + EPF <= C) {
+        v = tw_load_frag(src + c);
+      } else {
+#pragma unroll
+        for (int e = 0; e < EPF; ++e)
+          if (c + e < C) v[e] = tw_from_float<T>(w * tw_to_float(src[c + e]));
+      }
+    }
+    *reinterpret_cast<typename Elem<T>::Frag*>(dst + ((size_t)p * TW_MOE_TILE + r) * EPF) = v;
   }
-  const float w = weights ? weights[item] : 1.f;          // (no weights: they multiply the experts' outputs instead)
-  const T* src = h + (size_t)(item / top) * ld_h;
-  for (int c = threadIdx.x; c < Cd; c += blockDim.x) dst[at(c)] = tw_from_float<T>(c < C ? w * tw_to_float(src[c]) : 0.f);
 }
 
 // ---- the grouped products ---------------------------------------------------------------------------------------
@@ -588,7 +600,8 @@ static void moe_run(const MoeStep& s, hipStream_t stream) {
     else if (s.kind == 2) moe_products_few<T, 3>(s, stream);
     else moe_products_few<T, 4>(s, stream);
   } else {
-    moe_gather_kernel<T><<<s.capacity, 256, 0, stream>>>((const T*)s.h, s.ld_h, s.kind == 0 ? s.weights : nullptr, s.src_item,
+    const int pieces = tw_div_up(s.Cd, 16 * Elem<T>::kPerFrag);
+    moe_gather_kernel<T><<<dim3(s.capacity / TW_MOE_TILE, pieces < 4 ? pieces : 4), 256, 0, stream>>>((const T*)s.h, s.ld_h, s.kind == 0 ? s.weights : nullptr, s.src_item,
                                                          s.tile_expert, (T*)s.xs, s.C, s.Cd, s.top);
     const int tiles = s.capacity / TW_MOE_TILE;
 #define TW_MOE_PRODUCTS(ACT)                                                                                            \

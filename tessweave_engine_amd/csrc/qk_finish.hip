@@ -190,16 +190,18 @@ extern "C" int tw_head_finish(int dtype, const float* src, long ld, int q_col, i
 // every (head, map) is a query of its own whose other half is zeros, so that plain attention over M H query heads and G key
 // heads of M D elements gives every map's scores against the same values.
 //   src   float32 rows, or the split-K sums of the projection [splits][n][ld], added up here in index order
+// The angles are positions times freq + rest (rest, or null: what float32 rounded off the frequencies), formed here with the
+// product's rounding error beside it.
 //   q_out [n][H M][Dp], keys [pages][G][P][Dp], values [pages][G][Dp][P] in the compute type (tails of zeros)
 //   gate  float32 [n][H]
-// k_col < 0: no keys and values (a layer that reads another's pages); g_col < 0: no gate. One workgroup a token: q and k
+// k_col < 0: no keys and values (a layer that reads another's pages); g_col < 0: no gate. A token's q and k
 // meet in LDS.
 struct RowsFinishArgs {
   const float* src; long ld; int splits; size_t split_stride;
   const float* bias;
   int q_col, k_col, v_col, g_col;
   const float* wq; const float* wk; int norm;
-  const float* cos_t; const float* sin_t;
+  const int* positions; const float* freq; const float* rest;
   int rot, pairing;
   void* q_out; long ld_q;
   void* keys; void* values; const int* slots;
@@ -207,7 +209,11 @@ struct RowsFinishArgs {
   int H, G, M, D, E, Dp, P;
   float eps, v_scale;
   bool vec;                     // columns, row length and addresses allow 16-byte accesses
+  int n;                        // tokens
 };
+
+#define RF_TILE 16              /* tokens whose values one workgroup writes in steps of many rows */
+#define RF_FEW 64               /* up to this many rows a token's workgroup is wide and writes its own values */
 
 __device__ __forceinline__ float rf_rotated(const float* x, int d, int rot, int pairing, const float* cs, const float* sn) {
   if (d >= rot) return x[d];
@@ -227,6 +233,45 @@ __device__ __forceinline__ float rf_rotated(const float* x, int d, int rot, int 
   return first ? __fmaf_rn(x[d], c, -__fmul_rn(x[other], s)) : __fmaf_rn(x[d], c, __fmul_rn(x[other], s));
 }
 
+// Elements d .. d + 3 of a head; whole (sizes allow it): in 16-byte pieces, d a multiple of 4.
+__device__ __forceinline__ f32x4 rf_rotated4(const float* x, int d, int D, int rot, int pairing, const float* cs, const float* sn, bool whole) {
+  f32x4 v;
+  if (!whole) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = d + j >= 0 && d + j < D ? rf_rotated(x, d + j, rot, pairing, cs, sn) : 0.f;
+    return v;
+  }
+  if (d < 0 || d >= D) return f32x4{0.f, 0.f, 0.f, 0.f};
+  v = *reinterpret_cast<const f32x4*>(x + d);
+  if (d >= rot) return v;
+  if (pairing == 1) {
+    const float c0 = cs[d / 2], c1 = cs[d / 2 + 1], s0 = sn[d / 2], s1 = sn[d / 2 + 1];
+    return f32x4{__fmaf_rn(v[0], c0, -__fmul_rn(v[1], s0)), __fmaf_rn(v[1], c0, __fmul_rn(v[0], s0)),
+                 __fmaf_rn(v[2], c1, -__fmul_rn(v[3], s1)), __fmaf_rn(v[3], c1, __fmul_rn(v[2], s1))};
+  }
+  const int half = rot / 2;
+  const bool first = d < half;
+  const int pair = first ? d : d - half;
+  const f32x4 other = *reinterpret_cast<const f32x4*>(x + (first ? d + half : d - half));
+  const f32x4 c = *reinterpret_cast<const f32x4*>(cs + pair), s = *reinterpret_cast<const f32x4*>(sn + pair);
+#pragma unroll
+  for (int j = 0; j < 4; ++j) v[j] = first ? __fmaf_rn(v[j], c[j], -__fmul_rn(other[j], s[j])) : __fmaf_rn(v[j], c[j], __fmul_rn(other[j], s[j]));
+  return v;
+}
+
+// Sum over the 16 lanes of a row of the wave; every lane gets it.
+template <int CTRL>
+__device__ __forceinline__ float rf_turned_row(float v) {
+  return __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), CTRL, 0xf, 0xf, true));
+}
+__device__ __forceinline__ float rf_row_sum(float v) {
+  v += rf_turned_row<0x128>(v);
+  v += rf_turned_row<0x124>(v);
+  v += rf_turned_row<0x122>(v);
+  v += rf_turned_row<0x121>(v);
+  return v;
+}
+
 template <typename T>
 __device__ __forceinline__ void rf_store4(T* p, const float (&v)[4]) {
   struct alignas(4 * sizeof(T)) Four { T e[4]; };
@@ -237,124 +282,197 @@ __device__ __forceinline__ void rf_store4(T* p, const float (&v)[4]) {
 }
 
 template <typename T>
-__global__ __launch_bounds__(256) void rows_finish_kernel(RowsFinishArgs a) {
-  extern __shared__ __attribute__((aligned(16))) float rf_lds[];
-  __shared__ float red[16];
-  const int n = blockIdx.x, tid = threadIdx.x;
-  const float* row = a.src + (size_t)n * a.ld;
-  const int nq = a.H * a.M * a.D, nk = a.k_col >= 0 ? a.G * a.M * a.D : 0;
-  float* q_s = rf_lds;
-  float* k_s = rf_lds + (nq + 3) / 4 * 4;
-  auto column = [&](int c) {
-    float v = row[c];
-    for (int s = 1; s < a.splits; ++s) v += row[s * a.split_stride + c];
-    return a.bias ? v + a.bias[c] : v;
-  };
-  auto four = [&](int c) {
-    f32x4 v = *reinterpret_cast<const f32x4*>(row + c);
-#pragma unroll 8
-    for (int s = 1; s < a.splits; ++s) v += *reinterpret_cast<const f32x4*>(row + s * a.split_stride + c);
-    if (a.bias) v += *reinterpret_cast<const f32x4*>(a.bias + c);
-    return v;
-  };
-  // the row's queries and keys into LDS, their squares summed on the way
-  auto stage = [&](float* dst, int col, int count) {
-    float ss = 0.f;
-    if (a.vec) {
-      for (int i = 4 * tid; i < count; i += 1024) {
-        f32x4 v;
-        if (i + 4 <= count) v = four(col + i);
-        else {
+__device__ __forceinline__ void rf_store4(T* p, f32x4 v) {
+  const float e[4] = {v[0], v[1], v[2], v[3]};
+  rf_store4<T>(p, e);
+}
+
+// One column of a token's row: its split-K sums added up in index order, then the bias.
+__device__ __forceinline__ float rf_column(const RowsFinishArgs& a, const float* row, int c) {
+  float v = row[c];
+  for (int s = 1; s < a.splits; ++s) v += row[s * a.split_stride + c];
+  return a.bias ? v + a.bias[c] : v;
+}
+
+// The values of 16 tokens: a thread takes one element of one head and writes it for all of them, eight tokens a store where
+// they are neighbours in a page (values lie transposed there).
+template <typename T>
+__device__ void rf_values(const RowsFinishArgs& a, int tile, int column_block) {
+  const int i = column_block * blockDim.x + threadIdx.x;
+  if (i >= a.G * a.Dp) return;
+  const int g = i / a.Dp, e = i - g * a.Dp, t0 = tile * RF_TILE;
+  const bool real = e < a.E;
+  float v[RF_TILE];
 #pragma unroll
-          for (int j = 0; j < 4; ++j) v[j] = i + j < count ? column(col + i + j) : 0.f;
-        }
+  for (int j = 0; j < RF_TILE; ++j) v[j] = real && t0 + j < a.n ? rf_column(a, a.src + (size_t)(t0 + j) * a.ld, a.v_col + g * a.E + e) : 0.f;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) ss = __fmaf_rn(v[j], v[j], ss);
-        *reinterpret_cast<f32x4*>(dst + i) = v;
+  for (int half = 0; half < RF_TILE; half += 8) {
+    const int t = t0 + half;
+    if (t >= a.n) return;
+    const int first = a.slots[t];
+    bool together = first >= 0 && first % 8 == 0 && a.P % 8 == 0 && t + 8 <= a.n;
+    if (together) {
+#pragma unroll
+      for (int j = 1; j < 8; ++j) together = together && a.slots[t + j] == first + j;
+    }
+    auto place = [&](int slot) { return (T*)a.values + (((size_t)(slot / a.P) * a.G + g) * a.Dp + e) * a.P + slot % a.P; };
+    if (together) {
+      T* to = place(first);
+#pragma unroll
+      for (int q = 0; q < 8; q += 4) {
+        float four[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) four[j] = v[half + q + j] * a.v_scale;
+        rf_store4<T>(to + q, four);
       }
     } else {
-      for (int i = tid; i < count; i += 256) {
-        const float v = column(col + i);
-        ss = __fmaf_rn(v, v, ss);
-        dst[i] = v;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const int slot = t + j < a.n ? a.slots[t + j] : -1;
+        if (slot >= 0) *place(slot) = tw_from_float<T>(v[half + j] * a.v_scale);
       }
     }
-    return ss;
-  };
-  float sq = stage(q_s, a.q_col, nq), sk = nk ? stage(k_s, a.k_col, nk) : 0.f;
-  const int slot = nk ? a.slots[n] : -1;
-  const int page = slot >= 0 ? slot / a.P : 0, at = slot >= 0 ? slot % a.P : 0;
-  if (slot >= 0) {                                    // values: straight from the row into the page
-    for (int i = tid; i < a.G * a.Dp; i += 256) {
-      const int g = i / a.Dp, e = i - g * a.Dp;
-      const float v = e < a.E ? column(a.v_col + g * a.E + e) * a.v_scale : 0.f;
-      ((T*)a.values)[(((size_t)page * a.G + g) * a.Dp + e) * a.P + at] = tw_from_float<T>(v);
-    }
-  }
-  if (a.g_col >= 0)
-    for (int i = tid; i < a.H; i += 256) a.gate[(size_t)n * a.H + i] = 1.f / (1.f + expf(-column(a.g_col + i)));
-  if (a.norm == 2) {
-    sq = tw_block_sum(sq, red);
-    const float rq = 1.f / sqrtf(sq / (float)nq + a.eps);
-    for (int i = tid; i < nq; i += 256) q_s[i] = q_s[i] * rq * a.wq[i];
-    if (nk) {
-      sk = tw_block_sum(sk, red);
-      const float rk = 1.f / sqrtf(sk / (float)nk + a.eps);
-      for (int i = tid; i < nk; i += 256) k_s[i] = k_s[i] * rk * a.wk[i];
-    }
-  } else if (a.norm == 1) {
-    __syncthreads();
-    const int lane = tid & 63, heads_q = a.H * a.M, heads = heads_q + (nk ? a.G * a.M : 0);
-    for (int head = tid >> 6; head < heads; head += 4) {
-      float* x = head < heads_q ? q_s + head * a.D : k_s + (head - heads_q) * a.D;
-      const float* w = head < heads_q ? a.wq : a.wk;
-      float v[4], ss = 0.f;                           // D <= 256
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int d = lane + 64 * i;
-        v[i] = d < a.D ? x[d] : 0.f;
-        ss = __fmaf_rn(v[i], v[i], ss);
-      }
-      const float f = 1.f / sqrtf(tw_wave_sum(ss) / (float)a.D + a.eps);
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int d = lane + 64 * i;
-        if (d < a.D) x[d] = v[i] * f * w[d];
-      }
-    }
-  }
-  __syncthreads();
-  const float* cs = a.cos_t + (size_t)n * (a.rot / 2);
-  const float* sn = a.sin_t + (size_t)n * (a.rot / 2);
-  const int pieces = a.Dp / 4;
-  T* q = (T*)a.q_out + (size_t)n * a.ld_q;
-  for (int i = tid; i < a.H * a.M * pieces; i += 256) {
-    const int vh = i / pieces, d0 = (i - vh * pieces) * 4;
-    const int from = a.M == 2 ? (vh & 1) * a.D : 0;   // where the map's elements lie among the key's
-    float v[4];
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int d = d0 + j - from;
-      v[j] = d >= 0 && d < a.D ? rf_rotated(q_s + vh * a.D, d, a.rot, a.pairing, cs, sn) : 0.f;
-    }
-    rf_store4<T>(q + (size_t)vh * a.Dp + d0, v);
-  }
-  if (slot < 0) return;
-  for (int i = tid; i < a.G * pieces; i += 256) {
-    const int g = i / pieces, d0 = (i - g * pieces) * 4;
-    float v[4];
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int d = d0 + j, m = d >= a.D ? 1 : 0;
-      v[j] = d < a.M * a.D ? rf_rotated(k_s + (g * a.M + m) * a.D, d - m * a.D, a.rot, a.pairing, cs, sn) : 0.f;
-    }
-    rf_store4<T>((T*)a.keys + (((size_t)page * a.G + g) * a.P + at) * a.Dp + d0, v);
   }
 }
 
+// Workgroups 0 .. n - 1: a token each. Steps of many rows: the workgroups behind them write the values, 16 tokens each
+// (value_blocks a tile); else a token's workgroup writes its own. Every 16-byte piece of q, k and v is one thread's, so
+// that all of a row is on its way at once.
+template <typename T, int THREADS>
+__global__ __launch_bounds__(THREADS) void rows_finish_kernel(RowsFinishArgs a, int value_blocks) {
+  extern __shared__ __attribute__((aligned(16))) float rf_lds[];
+  __shared__ float red[16];
+  __shared__ __attribute__((aligned(16))) float cs[128], sn[128];                  // rot <= 256
+  const int n = blockIdx.x, tid = threadIdx.x;
+  if (n >= a.n) {
+    rf_values<T>(a, (n - a.n) / value_blocks, (n - a.n) % value_blocks);
+    return;
+  }
+  const float* row = a.src + (size_t)n * a.ld;
+  const bool keys = a.k_col >= 0;
+  const int nq = a.H * a.M * a.D, nk = keys ? a.G * a.M * a.D : 0, nv = keys && !value_blocks ? a.G * a.E : 0;
+  const int pq = (nq + 3) / 4, pk = (nk + 3) / 4, pv = (nv + 3) / 4;
+  float* q_s = rf_lds;
+  float* k_s = q_s + 4 * pq;
+  float* v_s = k_s + 4 * pk;
+  const int slot = keys ? a.slots[n] : -1;
+  float sq = 0.f, sk = 0.f;
+  for (int i = tid; i < pq + pk + pv; i += THREADS) {
+    const int in_q = i < pq, in_k = !in_q && i < pq + pk;
+    const int at = 4 * (in_q ? i : in_k ? i - pq : i - pq - pk);
+    const int count = in_q ? nq : in_k ? nk : nv;
+    const int col = (in_q ? a.q_col : in_k ? a.k_col : a.v_col) + at;
+    f32x4 v;
+    if (a.vec && at + 4 <= count) {
+      v = *reinterpret_cast<const f32x4*>(row + col);
+#pragma unroll 8
+      for (int s = 1; s < a.splits; ++s) v += *reinterpret_cast<const f32x4*>(row + s * a.split_stride + col);
+      if (a.bias) v += *reinterpret_cast<const f32x4*>(a.bias + col);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] = at + j < count ? rf_column(a, row, col + j) : 0.f;
+    }
+    if (a.norm == 2) {
+      float ss = 0.f;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) ss = __fmaf_rn(v[j], v[j], ss);
+      if (in_q) sq += ss;
+      else if (in_k) sk += ss;
+    }
+    *reinterpret_cast<f32x4*>(rf_lds + 4 * i) = v;
+  }
+  for (int i = THREADS - 1 - tid; i < a.rot / 2; i += THREADS) {    // (the last threads: they have the fewest pieces)
+    const float p = (float)a.positions[n], f = a.freq[i];
+    const float angle = __fmul_rn(p, f);
+    const float off = a.rest ? __fmaf_rn(p, a.rest[i], __fmaf_rn(p, f, -angle)) : 0.f;    // (a few hundredths at most)
+    float s, c;
+    sincosf(angle, &s, &c);
+    const float off2 = off * off, so = off * __fmaf_rn(-off2, 1.f / 6.f, 1.f), co = -0.5f * off2;
+    sn[i] = __fmaf_rn(so, c, __fmaf_rn(co, s, s));
+    cs[i] = __fmaf_rn(-so, s, __fmaf_rn(co, c, c));
+  }
+  if (a.g_col >= 0)
+    for (int i = THREADS - 1 - tid; i < a.H; i += THREADS)
+      a.gate[(size_t)n * a.H + i] = 1.f / (1.f + expf(-rf_column(a, row, a.g_col + i)));
+  auto scale_row = [&](float* x, int count, float f, const float* w) {
+    for (int i = 4 * tid; i < count; i += 4 * THREADS) {
+      f32x4 v = *reinterpret_cast<const f32x4*>(x + i) * f;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] *= i + j < count ? w[i + j] : 0.f;
+      *reinterpret_cast<f32x4*>(x + i) = v;
+    }
+  };
+  if (a.norm == 2) {
+    sq = tw_block_sum(sq, red);
+    const float rq = 1.f / sqrtf(sq / (float)nq + a.eps);
+    scale_row(q_s, nq, rq, a.wq);
+    if (nk) {
+      sk = tw_block_sum(sk, red);
+      const float rk = 1.f / sqrtf(sk / (float)nk + a.eps);
+      scale_row(k_s, nk, rk, a.wk);
+    }
+  } else if (a.norm == 1) {
+    __syncthreads();
+    // 16 lanes a head
+    const int lane = tid & 15, heads_q = a.H * a.M, heads = heads_q + (nk ? a.G * a.M : 0);
+    for (int head = tid >> 4; head < heads; head += THREADS / 16) {
+      float* x = head < heads_q ? q_s + head * a.D : k_s + (head - heads_q) * a.D;
+      const float* w = head < heads_q ? a.wq : a.wk;
+      float ss = 0.f;
+      for (int d = lane; d < a.D; d += 16) ss = __fmaf_rn(x[d], x[d], ss);
+      const float f = 1.f / sqrtf(rf_row_sum(ss) / (float)a.D + a.eps);
+      for (int d = lane; d < a.D; d += 16) x[d] = x[d] * f * w[d];
+    }
+  }
+  __syncthreads();
+  const int pieces = a.Dp / 4;
+  const int page = slot >= 0 ? slot / a.P : 0, at = slot >= 0 ? slot % a.P : 0;
+  T* q = (T*)a.q_out + (size_t)n * a.ld_q;
+  const int heads_q = a.H * a.M, heads_k = slot >= 0 ? a.G : 0;
+  const bool whole = a.D % 4 == 0 && a.rot % 8 == 0;                 // four elements turn alike, with four others or among themselves
+  for (int i = tid; i < (heads_q + heads_k) * pieces; i += THREADS) {
+    const int head = i / pieces, d0 = (i - head * pieces) * 4;
+    if (head < heads_q) {
+      const int from = a.M == 2 ? (head & 1) * a.D : 0;              // where the map's elements lie among the key's
+      rf_store4<T>(q + (size_t)head * a.Dp + d0, rf_rotated4(q_s + head * a.D, d0 - from, a.D, a.rot, a.pairing, cs, sn, whole));
+    } else {
+      const int g = head - heads_q;
+      f32x4 v;
+      if (whole || a.M == 1) {
+        const int m = a.M == 2 && d0 >= a.D ? 1 : 0;
+        v = rf_rotated4(k_s + (g * a.M + m) * a.D, d0 - m * a.D, a.D, a.rot, a.pairing, cs, sn, whole);
+      } else {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const int d = d0 + j, m = d >= a.D ? 1 : 0;
+          v[j] = d < 2 * a.D ? rf_rotated(k_s + (g * 2 + m) * a.D, d - m * a.D, a.rot, a.pairing, cs, sn) : 0.f;
+        }
+      }
+      rf_store4<T>((T*)a.keys + (((size_t)page * a.G + g) * a.P + at) * a.Dp + d0, v);
+    }
+  }
+  if (value_blocks || slot < 0) return;
+  for (int i = tid; i < a.G * a.Dp; i += THREADS) {
+    const int g = i / a.Dp, e = i - g * a.Dp;
+    ((T*)a.values)[(((size_t)page * a.G + g) * a.Dp + e) * a.P + at] = tw_from_float<T>(e < a.E ? v_s[g * a.E + e] * a.v_scale : 0.f);
+  }
+}
+
+template <typename T, int THREADS>
+static int rows_finish_launch(const RowsFinishArgs& a, size_t lds, int value_blocks, hipStream_t stream) {
+  static bool allowed = false;
+  if (!allowed) {
+    const hipError_t e = hipFuncSetAttribute((const void*)rows_finish_kernel<T, THREADS>, hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024);
+    if (e != hipSuccess) return (int)e;
+    allowed = true;
+  }
+  rows_finish_kernel<T, THREADS><<<a.n + value_blocks * tw_div_up(a.n, RF_TILE), THREADS, lds, stream>>>(a, value_blocks);
+  return TW_LAUNCH_RESULT();
+}
+
 extern "C" int tw_rows_finish(int dtype, const float* src, long ld, int splits, long split_stride, const float* bias, int q_col,
-                              int k_col, int v_col, int g_col, int norm, const float* wq, const float* wk, const float* cos_t,
-                              const float* sin_t, int rot, int pairing, void* q_out, long ld_q, void* keys, void* values,
+                              int k_col, int v_col, int g_col, int norm, const float* wq, const float* wk,
+                              const int* positions, const float* freq, const float* rest, int rot, int pairing, void* q_out, long ld_q, void* keys, void* values,
                               const int* slots, float* gate, int n, int H, int G, int M, int D, int E, int Dp, int page_size,
                               float eps, float v_scale, hipStream_t stream) {
   TW_REQUIRE(src && q_out && n >= 0 && H > 0 && G > 0 && (M == 1 || M == 2) && D > 0 && D <= 256 && splits >= 1);
@@ -364,28 +482,22 @@ extern "C" int tw_rows_finish(int dtype, const float* src, long ld, int splits, 
                            ld >= k_col + (long)G * M * D && ld >= v_col + (long)G * E));
   TW_REQUIRE(g_col < 0 || (gate && ld >= (long)g_col + H));
   TW_REQUIRE(norm >= 0 && norm <= 2 && (norm == 0 || (wq && (wk || k_col < 0) && eps > 0.f)));
-  TW_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= D && (rot == 0 || (cos_t && sin_t)) && (pairing == 0 || pairing == 1));
+  TW_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= D && (rot == 0 || (positions && freq)) && (pairing == 0 || pairing == 1));
   TW_REQUIRE((uintptr_t)q_out % 16 == 0 && ld_q % 4 == 0 && (k_col < 0 || (uintptr_t)keys % 16 == 0));
-  const int nq = H * M * D, nk = k_col < 0 ? 0 : G * M * D;
-  const size_t lds = ((size_t)(nq + 3) / 4 * 4 + (size_t)(nk + 3) / 4 * 4) * sizeof(float);
+  const int nq = H * M * D, nk = k_col < 0 ? 0 : G * M * D, nv = k_col < 0 ? 0 : G * E;
+  const size_t lds = ((size_t)(nq + 3) / 4 + (size_t)(nk + 3) / 4 + (n <= RF_FEW ? (size_t)(nv + 3) / 4 : 0)) * 16;
   TW_REQUIRE(lds <= 128 * 1024);
   if (n == 0) return 0;
-  const bool vec = ld % 4 == 0 && split_stride % 4 == 0 && q_col % 4 == 0 && (k_col < 0 || k_col % 4 == 0) &&
+  const bool vec = ld % 4 == 0 && split_stride % 4 == 0 && q_col % 4 == 0 && (k_col < 0 || (k_col % 4 == 0 && v_col % 4 == 0)) &&
                    (uintptr_t)src % 16 == 0 && (!bias || (uintptr_t)bias % 16 == 0);
-  RowsFinishArgs a{src, ld, splits, (size_t)split_stride, bias, q_col, k_col, v_col, g_col, wq, wk, norm, cos_t, sin_t, rot, pairing,
-                   q_out, ld_q, keys, values, slots, gate, H, G, M, D, E, Dp, page_size > 0 ? page_size : 1, eps, v_scale, vec};
-  static bool allowed = false;
-  if (!allowed) {
-    hipError_t e = hipFuncSetAttribute((const void*)rows_finish_kernel<bf16_t>, hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024);
-    if (e == hipSuccess)
-      e = hipFuncSetAttribute((const void*)rows_finish_kernel<float>, hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024);
-    if (e != hipSuccess) return (int)e;
-    allowed = true;
-  }
-  if (dtype == TW_DTYPE_BF16) rows_finish_kernel<bf16_t><<<n, 256, lds, stream>>>(a);
-  else if (dtype == TW_DTYPE_F32) rows_finish_kernel<float><<<n, 256, lds, stream>>>(a);
-  else return TW_ERR_BAD_ARGUMENT;
-  return TW_LAUNCH_RESULT();
+  const RowsFinishArgs a{src, ld, splits, (size_t)split_stride, bias, q_col, k_col, v_col, g_col, wq, wk, norm, positions, freq, rest, rot, pairing,
+                         q_out, ld_q, keys, values, slots, gate, H, G, M, D, E, Dp, page_size > 0 ? page_size : 1, eps, v_scale, vec, n};
+  const int value_blocks = k_col >= 0 && n > RF_FEW ? tw_div_up((long)G * Dp, 256) : 0;
+  if (dtype == TW_DTYPE_BF16)
+    return n <= RF_FEW ? rows_finish_launch<bf16_t, 1024>(a, lds, 0, stream) : rows_finish_launch<bf16_t, 256>(a, lds, value_blocks, stream);
+  if (dtype == TW_DTYPE_F32)
+    return n <= RF_FEW ? rows_finish_launch<float, 1024>(a, lds, 0, stream) : rows_finish_launch<float, 256>(a, lds, value_blocks, stream);
+  return TW_ERR_BAD_ARGUMENT;
 }
 
 // ---- two maps of a head combined -----------------------------------------------------------------------------------

@@ -88,7 +88,7 @@ _SIGNATURES = {
     "tw_linear_state": (I, [P, L, I, I, I, I, P, L, P, L, I, P, P, F, P, L, I, P, P, P, P, P, P, I, I, I, P, L, I, I, I, F, P, I, I, P, L, P]),
     "tw_decay_logs": (I, [P, L, P, P, F, P, L, I, I, I, P]),
     "tw_gate_group_norm": (I, [I, P, L, P, L, P, P, L, I, I, I, F, I, F, P]),
-    "tw_rows_finish": (I, [I, P, L, I, L, P, I, I, I, I, I, P, P, P, P, I, I, P, L, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P]),
+    "tw_rows_finish": (I, [I, P, L, I, L, P, I, I, I, I, I, P, P, P, P, P, I, I, P, L, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P]),
     "tw_map_difference": (I, [I, P, L, P, P, L, I, I, I, I, I, F, F, F, P]),
     "tw_layer_norm": (I, [I, P, P, L, P, I, L, P, P, P, I, P, P, P, P, P, P, I, I, F, P]),
     "tw_sampling_uniform": (F, [c_uint64, c_uint64]),

@@ -1555,14 +1555,15 @@ def gate_group_norm(y, gate, weight, out, parts, eps, after=False, scale=1.0):
 
 # ---- rotated queries and keys of a packed projection, two maps combined, layer norms -------------------------------------
 
-def rows_finish(src, columns, norm, q_weight, k_weight, cos, sin, q_out, keys, values, slots, gate, q_heads, kv_heads, dim,
+def rows_finish(src, columns, norm, q_weight, k_weight, rotation, q_out, keys, values, slots, gate, q_heads, kv_heads, dim,
                 value_dim, eps, maps=1, adjacent=False, value_scale=1.0, bias=None):
     """Per token: q <- rotate(norm(q)), k <- rotate(norm(k)), v <- value_scale * v, gate <- sigmoid(g), from one projection.
 
     src float32 [n, width], or [splits, n, width] split-K sums that are added up here (bias float32 [width], or None, is added
     in both cases). columns = (q, k, v, g): where each begins; k (and v) None: no keys, g None: no gate. norm None, "head" (over
-    a head's dim elements, weights [dim]) or "row" (over all heads at once, weights over the row). cos, sin float32
-    [n, rot / 2]: the first rot elements of every head turn ("half" pairs, or neighbours with `adjacent`), None: no rotation.
+    a head's dim elements, weights [dim]) or "row" (over all heads at once, weights over the row). rotation = (positions int32 [n],
+    frequencies float32 [rot / 2], what float32 rounded off those or None): the first rot elements of every head turn ("half"
+    pairs, or neighbours with `adjacent`) by position times frequency; None: no rotation.
     maps 2: a head has two maps of dim elements, each turned by itself; its key holds them side by side, and q_out has a row of
     2 * q_heads queries, each with zeros in the other map's place. q_out [n, q_heads * maps * dev] (dev: keys' last size), keys
     [pages, kv_heads, page, dev], values the same number of elements, as [pages, kv_heads, dev, page]; slots[n] the token's
@@ -1595,17 +1596,19 @@ def rows_finish(src, columns, norm, q_weight, k_weight, cos, sin, q_out, keys, v
             continue
         want = dim if norm == "head" else heads * maps * dim
         _need(w.dtype == torch.float32 and w.is_contiguous() and w.numel() == want, "the norms' weights are float32 over a head or the row")
-    rot = 0
-    if cos is not None:
-        rot = 2 * cos.shape[1]
-        _need(cos.dtype == torch.float32 == sin.dtype and cos.is_contiguous() and sin.is_contiguous() and cos.shape[0] == n
-              and sin.shape == cos.shape and rot <= dim, "cos and sin are float32 [n, rot / 2]")
+    rot, positions, freq, rest = 0, None, None, None
+    if rotation is not None:
+        positions, freq, rest = rotation
+        rot = 2 * freq.numel()
+        _need(positions.dtype == torch.int32 and positions.is_contiguous() and positions.numel() == n and rot <= dim, "one int32 position per row is needed")
+        for t in (freq, rest) if rest is not None else (freq,):
+            _need(t.dtype == torch.float32 and t.is_contiguous() and 2 * t.numel() == rot, "frequencies are float32 [rot / 2]")
     if bias is not None:
         _need(bias.dtype == torch.float32 and bias.is_contiguous() and bias.numel() == width, "bias must be float32 [width]")
     opt = lambda t: _dev(t) if t is not None else None       # noqa: E731
     check(library().tw_rows_finish(dtype_id(q_out.dtype), _dev(src), ld, splits, stride, opt(bias), q_col, k_col, v_col, g_col,
                                    {None: 0, "head": 1, "row": 2}[norm], opt(q_weight if norm else None),
-                                   opt(k_weight if norm and k_col >= 0 else None), opt(cos), opt(sin), rot, 1 if adjacent else 0,
+                                   opt(k_weight if norm and k_col >= 0 else None), opt(positions), opt(freq), opt(rest), rot, 1 if adjacent else 0,
                                    _dev(q_out), ld_q, _dev(keys) if k_col >= 0 else None, _dev(values) if k_col >= 0 else None,
                                    _dev(slots, torch.int32, "slots") if k_col >= 0 else None, opt(gate if g_col >= 0 else None), n,
                                    int(q_heads), int(kv_heads), int(maps), int(dim), int(value_dim), dev, page, float(eps),

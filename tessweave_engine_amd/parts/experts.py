@@ -48,8 +48,9 @@ class RoutedExperts(FeedForward):
         """shared: a `FeedForward` part that every token runs as well (or None). expert_names: the checkpoint's
         names, behind the prefix, of expert number {}'s matrices (gate, up, down; up, down for kind "gelu").
         kind: "swish_limited" (gated, needs `limit`, weights on the experts' inputs), "gelu" or "relu_squared" (no gate, weights on
-        the outputs) or "silu" (gated, weights on the outputs); groups: (count, keep), weight_scale: of sigmoid weights; weighting: "sigmoid" of each chosen logit, "softmax_chosen" or
-        "softmax_all"; router_bias: the checkpoint's name, behind the prefix, of a bias on the router's logits (or None);
+        the outputs) or "silu" (gated, weights on the outputs); weighting: "sigmoid" of each chosen logit, "softmax_chosen" or
+        "softmax_all"; groups (count, keep) and weight_scale: of sigmoid weights; router_bias: the checkpoint's name, behind the
+        prefix, of a bias on the router's logits (or None);
         correction: the name of what is added to the scores of "softmax_all" for the choice alone (or None);
         identity: experts behind the others that return their input (kinds whose weights multiply outputs)."""
         self.prefix, self.hidden, self.experts, self.top = prefix, int(hidden), int(experts), int(top)
@@ -59,13 +60,13 @@ class RoutedExperts(FeedForward):
         self.kind, self.weighting, self.identity = kind, weighting, int(identity)
         self.gated = kind not in ops.MOE_PLAIN
         self.leaves_apart = kind != "swish_limited" and not self.identity
+        self.choices = self.experts + self.identity          # what the router scores
         self.groups, self.weight_scale = (int(groups[0]), int(groups[1])), float(weight_scale)
         count, keep = self.groups
-        if not (1 <= keep <= count) or self.experts % count or self.top > keep * (self.experts // count):
+        if not (1 <= keep <= count) or self.choices % count or self.top > keep * (self.choices // count):
             raise ValueError("the groups must be equal, and those kept must hold `top` experts")
         if weighting != "sigmoid" and (keep != count or self.weight_scale != 1.0):
             raise ValueError("groups and a scale of the weights go with sigmoid weights")
-        self.choices = self.experts + self.identity          # what the router scores
         if self.identity < 0 or (self.identity and kind == "swish_limited"):
             raise ValueError("identity experts go with weights on the experts' outputs")
         if correction and (weighting != "softmax_all" or router_bias):

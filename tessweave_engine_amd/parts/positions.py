@@ -72,6 +72,12 @@ class RotaryEmbedding(PositionEncoding):
         if self.divide is not None:
             self.rest = (self._exact_frequencies() - freq.double()).to(torch.float32).to(device)
 
+    def angles(self, ctx):
+        """(positions, frequencies, what float32 rounded off those or None), for kernels that form the angles themselves."""
+        if self.magnitude != 1.0:
+            raise ValueError("a stretched encoding scales its cosines and sines: use its tables")
+        return ctx.positions[0], self.inv_freq, self.rest
+
     def tables(self, ctx):
         """(cos, sin), float32 [n_tokens, rotary_dim / 2], computed once per step."""
         key = ("rotary", id(self))

@@ -19,7 +19,7 @@ that layer's cache slot without writing it. A key lies in the page with its two 
 in the other map's place. So the engine's attention kernels run both maps as one attention of twice the heads.
 
 The packed product leaves float32 rows (or split-K sums): biases, norms, rotation, gates and the cache write are one kernel
-(`ops.rows_finish`), float32 with one rounding. Keys and values are laid out with the larger of their sizes, rounded up to
+(`ops.rows_finish`, which also forms the angles), float32 with one rounding. Keys and values are laid out with the larger of their sizes, rounded up to
 16, tails of zeros. A branch's weight in its mixer's sum multiplies the values before they are rounded into the pages
 (attention is linear in them), or the combined maps.
 """
@@ -113,13 +113,12 @@ class RotaryAttention(MixerBranch):
         n, H = ctx.n_tokens, self.q_heads
         if run.writes_cache == self.reads_other:
             raise ValueError("the schedule and the layer disagree about who writes the cache slot")
-        cos, sin = self.position.tables(ctx)
         keys, values, g = ctx.cache.keys_values(run.cache_slot)
         group = ctx.groups[g]
         q = ctx.scratch("rotary.q", (n, H * self.maps * self.head_dev))
         gate = ctx.scratch("rotary.gate", (n, H), torch.float32) if self.has_gate else None
-        ops.rows_finish(proj, self.columns, self.norm, self.q_weight, self.k_weight, cos, sin, q, keys, values, group.slot_mapping,
-                        gate, H, self.kv_heads, self.dim, self.value_dim, self.eps, maps=self.maps,
+        ops.rows_finish(proj, self.columns, self.norm, self.q_weight, self.k_weight, self.position.angles(ctx), q, keys, values,
+                        group.slot_mapping, gate, H, self.kv_heads, self.dim, self.value_dim, self.eps, maps=self.maps,
                         adjacent=self.position.pairing == "adjacent", value_scale=value_scale, bias=bias)
         return q, keys, values, group, gate
 

@@ -169,18 +169,17 @@ def rows_of(parts, lo, hi):
     return parts[lo:hi] if parts.dim() == 2 else parts[:, lo:hi].contiguous()
 
 
-def run_portions(ops, rows, T, columns, norm, weights, tables, keys, values, bt, slots, sizes, out, scale, maps, adjacent, device, bias=None,
+def run_portions(ops, rows, T, columns, norm, weights, rotation, keys, values, bt, slots, sizes, out, scale, maps, adjacent, device, bias=None,
                  chunk=0, sink=None, gated=True, splits_decode=1, value_scale=1.0):
     """Two prompt portions (the first cut where no page and no chunk ends), then single tokens, through the finishing kernel and
     the attention kernels."""
     H, G, D, E, dev = sizes
-    cos, sin = tables
     q = torch.empty(T, H * maps * dev, dtype=keys.dtype, device=device)
     for lo, hi in [(0, 37), (37, 170)] + [(t, t + 1) for t in range(170, T)]:
         n = hi - lo
         gate = torch.full((n, H), float("nan"), device=device) if columns[3] is not None else None
-        ops.rows_finish(rows_of(rows, lo, hi), columns, norm, *weights, cos[lo:hi].contiguous(), sin[lo:hi].contiguous(), q[lo:hi], keys,
-                        values, slots[lo:hi].contiguous(), gate, H, G, D, E, 1e-5, maps=maps, adjacent=adjacent, bias=bias, value_scale=value_scale)
+        ops.rows_finish(rows_of(rows, lo, hi), columns, norm, *weights, (ints(list(range(lo, hi)), device), *rotation), q[lo:hi], keys, values,
+                        slots[lo:hi].contiguous(), gate, H, G, D, E, 1e-5, maps=maps, adjacent=adjacent, bias=bias, value_scale=value_scale)
         starts, lens = ints([0, n], device), ints([hi], device)
         extra = dict(chunk=chunk, sink=sink, gate=gate if gated else None)
         if n > 1:
@@ -196,9 +195,10 @@ def run_portions(ops, rows, T, columns, norm, weights, tables, keys, values, bt,
     return
 
 
-def tables_of(T, r, device):
-    a = plain.angles(T, r, torch.float64)
-    return torch.cos(a).float().to(device), torch.sin(a).float().to(device)
+def frequencies(r, device):
+    """(frequencies, what float32 rounds off them) of a rotation."""
+    f = plain.angles(2, r, torch.float64)[1]
+    return f.float().to(device), (f - f.float().double()).float().to(device)
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
@@ -234,7 +234,7 @@ def test_head_norms_rotation_and_sinks_made_sharp(device, dtype, H, G, D, E, tur
     dt = tdtype(dtype)
     keys, values, bt, slots = pages_of(T, page, G, dev, dt, device)
     out = torch.full((T, H * dev), float("nan"), dtype=dt, device=device)
-    for _ in run_portions(ops, split_rows(src, splits, g, device), T, (0, at[1], at[2], None), "head", (wq.to(device), wk.to(device)), tables_of(T, r, device),
+    for _ in run_portions(ops, split_rows(src, splits, g, device), T, (0, at[1], at[2], None), "head", (wq.to(device), wk.to(device)), frequencies(r, device),
                           keys, values, bt, slots, (H, G, D, E, dev), out, scale, 1, False, device, sink=sink.to(device),
                           splits_decode=splits_decode, value_scale=vs):
         pass
@@ -277,7 +277,7 @@ def test_row_norms_rotation_and_gates_made_sharp(device, dtype, H, G, D, E, turn
     dt = tdtype(dtype)
     keys, values, bt, slots = pages_of(T, page, G, dev, dt, device)
     out = torch.full((T, H * dev), float("nan"), dtype=dt, device=device)
-    for lo, hi, gate in run_portions(ops, split_rows(src, splits, g, device), T, (0, *at[1:]), "row", (wq.to(device), wk.to(device)), tables_of(T, r, device),
+    for lo, hi, gate in run_portions(ops, split_rows(src, splits, g, device), T, (0, *at[1:]), "row", (wq.to(device), wk.to(device)), frequencies(r, device),
                                      keys, values, bt, slots, (H, G, D, E, dev), out, scale, 1, True, device, splits_decode=splits_decode):
         assert torch.allclose(gate.double().cpu(), torch.sigmoid(z[lo:hi].double()), atol=1e-6)
     err = (out.view(T, H, dev)[:, :, :E].double().cpu().reshape(T, H * E) - want).abs().amax(1)
@@ -328,7 +328,7 @@ def test_differential_maps_in_chunks_made_sharp(device, dtype, chunk, splits_dec
     maps = torch.full((T, 2 * H * dev), float("nan"), device=device)
     out = torch.full((T, H * ((E + 7) // 8 * 8)), float("nan"), dtype=dt, device=device)
     rows = split_rows(src, splits, g, device)
-    for lo, hi, gate in run_portions(ops, rows, T, (0, *at[1:]), None, (None, None), tables_of(T, r, device), keys, values, bt, slots,
+    for lo, hi, gate in run_portions(ops, rows, T, (0, *at[1:]), None, (None, None), frequencies(r, device), keys, values, bt, slots,
                                      (H, G, D, E, dev), maps, scale, 2, True, device, bias=bias.to(device), chunk=chunk, gated=False,
                                      splits_decode=splits_decode):
         ops.map_difference(maps[lo:hi], out[lo:hi], H, E, weight, 1.0 - diff, eps, gate=gate)
@@ -345,9 +345,8 @@ def test_differential_maps_in_chunks_made_sharp(device, dtype, chunk, splits_dec
     # a layer that reads these pages with queries alone: the same rows, none written
     before = keys.clone(), values.nan_to_num().clone()
     q = torch.empty(T, H * 2 * dev, dtype=dt, device=device)
-    cos, sin = tables_of(T, r, device)
     gate = torch.empty(T, H, device=device)
-    ops.rows_finish(rows, (0, None, None, at[3]), None, None, None, cos, sin, q, keys, values, slots, gate, H, G, D, E, eps, maps=2, adjacent=True,
+    ops.rows_finish(rows, (0, None, None, at[3]), None, None, None, (ints(list(range(T)), device), *frequencies(r, device)), q, keys, values, slots, gate, H, G, D, E, eps, maps=2, adjacent=True,
                     bias=bias.to(device))
     assert torch.equal(keys, before[0]) and torch.equal(values.nan_to_num(), before[1])
     ops.attn_prefill(q, keys, values, bt, ints([0, T], device), ints([T], device), 0, 1, T, maps, 2 * H, G, dev, scale, chunk=chunk)
