@@ -297,7 +297,7 @@ __global__ __launch_bounds__(256) void moe_gather_kernel(const T* __restrict__ h
   const int item = src_item[tile * TW_MOE_TILE + r];
   const float w = weights && item >= 0 ? weights[item] : 1.f;             // (no weights: they multiply the experts' outputs instead)
   const T* src = h + (item >= 0 ? (size_t)(item / top) * ld_h : 0);
-  const bool vec = !weights && ld_h % EPF == 0 && (uintptr_t)h % 16 == 0;
+  const bool vec = ld_h % EPF == 0 && (uintptr_t)h % 16 == 0;
   T* dst = xs + (size_t)tile * Cd * TW_MOE_TILE;
 #pragma unroll 4
   for (int p = threadIdx.x / TW_MOE_TILE + 16 * blockIdx.y; p < Cd / EPF; p += 16 * gridDim.y) {
@@ -306,6 +306,10 @@ __global__ __launch_bounds__(256) void moe_gather_kernel(const T* __restrict__ h
     if (item >= 0) {
       if (vec && c + EPF <= C) {
         v = tw_load_frag(src + c);
+        if (weights) {
+#pragma unroll
+          for (int e = 0; e < EPF; ++e) v[e] = tw_from_float<T>(w * tw_to_float(v[e]));
+        }
       } else {
 #pragma unroll
         for (int e = 0; e < EPF; ++e)

@@ -605,14 +605,15 @@ FEW_LAYERS = {
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("kind", list(FEW_LAYERS))
 def test_each_mechanism_alone_in_a_small_model(device, tmp_path, kind, dtype):
-    """One or two layers, whole and then cut (portions, single tokens, beside another request), pages of four tokens."""
+    """One or two layers, whole and then cut (portions, single tokens, beside another request), on small pages (bfloat16: the
+    smallest its fast attention kernels take)."""
     c = config(FEW_LAYERS[kind], width=72, vocab=120)
     weights = make_weights(c, seed=3)
     folder = write_folder(tmp_path, c, weights)
     g = torch.Generator().manual_seed(1)
     tokens = {"a": torch.randint(0, 120, (75,), generator=g).tolist(), "b": torch.randint(0, 120, (19,), generator=g).tolist()}
     want = {k: reference(c, weights, v) for k, v in tokens.items()}
-    d = Driver(folder, dtype, pages=60, page_size=4, max_requests=2)
+    d = Driver(folder, dtype, pages=60, page_size=4 if dtype == "float32" else 8, max_requests=2)
     whole = d.run([[("a", 75), ("b", 19)]], tokens)
     d.at.clear()
     cut = d.run([[("a", 33)], [("a", 2), ("b", 5)], [("a", 17), ("b", 1)]] + [[("a", 1), ("b", 1)]] * 13 + [[("a", 10)]], tokens)
@@ -766,13 +767,13 @@ def test_batch_of_many_single_tokens_beside_portions(model):
 def test_far_keys_over_a_long_prompt(device, tmp_path, dtype, name):
     """Query heads that match their own key head's rows: a token's score is by far the largest against the same token
     earlier on, hundreds of tokens back, at page borders, at chunk edges or before a portion's start. 600 tokens of a small
-    alphabet: 330 in one step, then portions of 64, 15, 2 and single tokens, on pages of four tokens in an order of their own."""
+    alphabet: 330 in one step, then portions of 64, 15, 2 and single tokens, on small pages in an order of their own."""
     c = CONFIGS[name]
     weights = make_weights(c, seed=13, sharp=2.0)
     folder = write_folder(tmp_path, c, weights)
     toks = torch.randint(0, 60, (600,), generator=torch.Generator().manual_seed(4)).tolist()
     want, margin = reference(c, weights, toks)
-    d = Driver(folder, dtype, pages=180, page_size=4, max_step_tokens=64)
+    d = Driver(folder, dtype, pages=180, page_size=4 if dtype == "float32" else 8, max_step_tokens=64)
     warm = {"w0": toks[:37], "w1": toks[:90]}
     d.step([("w0", 36), ("w1", 89)], warm)
     d.end("w0")
@@ -872,7 +873,7 @@ def test_configurations_drawn_at_random(device, tmp_path, seed):
     tokens = {"a": torch.randint(0, c["vocab"], (83,), generator=g).tolist(), "b": torch.randint(0, c["vocab"], (21,), generator=g).tolist()}
     want = {k: reference(c, weights, v) for k, v in tokens.items()}
     for dtype in ("float32", "bfloat16"):
-        d = Driver(folder, dtype, pages=40, page_size=4, max_requests=2)
+        d = Driver(folder, dtype, pages=40, page_size=4 if seed % 3 == 0 else 16, max_requests=2)
         whole = d.run([[("a", 83), ("b", 21)]], tokens)
         cut = d.run([[("a", 30)], [("a", 17), ("b", 2)], [("a", 2), ("b", 1)], [("a", 24), ("b", 9)]] + [[("a", 1), ("b", 1)]] * 10, tokens)
         for got in (whole, cut):
