@@ -287,7 +287,7 @@ def test_row_norms_rotation_and_gates_made_sharp(device, dtype, H, G, D, E, turn
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("chunk,splits_decode", [(1, 1), (7, 1), (16, 2), (64, 1), (50, 3), (128, 2), (1000, 1)])
-@pytest.mark.parametrize("H,G,D,E,turned,page,splits", [(4, 2, 24, 20, 10, 4, 1), (3, 3, 32, 64, 8, 16, 3), (8, 1, 15, 34, 2, 8, 1), (2, 1, 64, 128, 64, 16, 2),
+@pytest.mark.parametrize("H,G,D,E,turned,page,splits", [(4, 2, 24, 20, 10, 4, 1), (3, 3, 32, 64, 8, 16, 3), (12, 1, 15, 34, 2, 8, 1), (2, 1, 64, 128, 64, 16, 2),
                                                         (6, 3, 11, 7, 6, 4, 1), (16, 2, 100, 200, 40, 16, 1)])
 def test_differential_maps_in_chunks_made_sharp(device, dtype, chunk, splits_decode, H, G, D, E, turned, page, splits):
     """Both maps' scores against the same values, in chunks counted from the sequence's start, and the maps combined. Each map's
